@@ -6,7 +6,8 @@ window of them form another, and so on. A group has a page pool of
 its own and, per request, one block table that serves all its layers: page p of
 a group exists once in each of the group's layers' planes. A request's pages
 go back to the pool when it ends, and, in a windowed group, as soon as every
-position a page covers lies behind the window. Mixers that keep a state of
+position a page covers lies behind the window. Tensors that grow by one element
+per complete run of tokens form groups of their own, whose pages count runs. Mixers that keep a state of
 fixed size get one slot per live request, the same slot number in all such
 groups; it is handed out at admission and taken back when the request ends.
 
@@ -40,6 +41,7 @@ from .pages import OutOfPages, PagePool
 class _Group:
     tensors: tuple                       # the PagedTensors that every layer of the group keeps
     window: int
+    every: int                           # tokens that one element stands for: 1, or a run's length
     planes: list
     pool: PagePool
 
@@ -75,7 +77,8 @@ class _Node:
 class CacheManager:
     def __init__(self, needs, page_size, num_pages, max_requests, prefix_cache=False):
         """`needs`: one CacheNeed (or None) per cache plane of the model.
-        `num_pages`: pages in every group's pool. `max_requests`: state slots.
+        `num_pages`: pages in every group's pool (a group that counts runs of tokens has as many as
+        the runs of that many tokens, held by that many requests, can fill). `max_requests`: state slots.
         `prefix_cache`: keep the prefix index, if the model's groups allow it."""
         if page_size <= 0:
             raise ValueError("page_size must be positive")
@@ -84,18 +87,16 @@ class CacheManager:
         self.groups = []
         self.state_groups = []
         self.group_of_plane = []
+        self.run_group_of_plane = []
         self.state_group_of_plane = []
         for plane, need in enumerate(needs):
-            g = s = -1
+            g = r = s = -1
             if need is not None and need.paged:
-                key = (tuple(need.paged), need.window)
-                for i, grp in enumerate(self.groups):
-                    if (grp.tensors, grp.window) == key:
-                        g = i
-                if g < 0:
-                    self.groups.append(_Group(*key, planes=[], pool=PagePool(num_pages)))
-                    g = len(self.groups) - 1
-                self.groups[g].planes.append(plane)
+                g = self._join_group((tuple(need.paged), need.window, 1), plane, num_pages)
+            if need is not None and need.runs:
+                every = int(need.run_length)
+                r = self._join_group((tuple(need.runs), 0, every), plane,
+                                     min(num_pages, -(-num_pages // every) + max_requests))
             if need is not None and need.has_state:
                 key = (tuple(need.state_shape), need.state_dtype)
                 for i, grp in enumerate(self.state_groups):
@@ -106,18 +107,28 @@ class CacheManager:
                     s = len(self.state_groups) - 1
                 self.state_groups[s].planes.append(plane)
             self.group_of_plane.append(g)
+            self.run_group_of_plane.append(r)
             self.state_group_of_plane.append(s)
         self._slots = list(range(max_requests - 1, -1, -1))
         self._requests = {}
         self._admissions = 0
         self.fresh_slots = []     # slots handed out since the storage last cleared them
         self.prefix_cache = bool(prefix_cache) and bool(self.groups) and not self.state_groups \
-            and all(g.window <= 0 for g in self.groups)
+            and all(g.window <= 0 and g.every == 1 for g in self.groups)
         self._nodes = {}                  # node id -> _Node
         self._index = {}                  # (parent id, tokens of the block) -> node id
         self._idle = OrderedDict()        # nodes without holders, the one left longest ago first
         self._next_node = 1               # 0 is the root
         self.prefix_hits = 0              # tokens that requests did not have to compute
+
+    def _join_group(self, key, plane, num_pages):
+        """The number of the group that keeps (tensors, window, tokens per element), made if it is new."""
+        for i, grp in enumerate(self.groups):
+            if (grp.tensors, grp.window, grp.every) == key:
+                grp.planes.append(plane)
+                return i
+        self.groups.append(_Group(*key, planes=[plane], pool=PagePool(num_pages)))
+        return len(self.groups) - 1
 
     # ---- requests ----
     def has(self, request_id):
@@ -149,15 +160,16 @@ class CacheManager:
         return held.slot
 
     # ---- growth ----
-    def _blocks_for(self, tokens):
-        return -(-tokens // self.page_size)
+    def _blocks_for(self, tokens, group):
+        """Pages that `tokens` tokens of a request fill in a group (of a run's tensors: its complete runs)."""
+        return -(-(tokens // self.groups[group].every) // self.page_size)
 
     def pages_missing(self, request_id, new_tokens):
         """Per group, the pages still to be taken before `new_tokens` more can be written."""
         held = self._requests.get(request_id)
         length = held.length if held else 0
-        target = self._blocks_for(length + new_tokens)
-        return [target - (len(held.tables[g]) if held else 0) for g in range(len(self.groups))]
+        return [self._blocks_for(length + new_tokens, g) - (len(held.tables[g]) if held else 0)
+                for g in range(len(self.groups))]
 
     def can_grow(self, request_id, new_tokens, spare=None):
         """True if every group's pool can cover `new_tokens` more for the request.
@@ -311,13 +323,13 @@ class CacheManager:
         page goes back (the entry turns -1), so kernels find a key's page by its position alone."""
         if not 0 <= group < len(self.groups):
             raise IndexError("no group %d" % group)
-        return -(-tokens // self.page_size)
+        return self._blocks_for(tokens, group)
 
     def capacity_tokens(self):
         """Tokens one request can hold at most (bounded by the smallest pool)."""
         if not self.groups:
             return 1 << 62
-        return min(g.pool.num_pages for g in self.groups) * self.page_size
+        return min(g.pool.num_pages * g.every for g in self.groups) * self.page_size
 
     def audit(self):
         """Every page is free, held by exactly one request, or owned by exactly

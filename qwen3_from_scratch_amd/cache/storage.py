@@ -13,6 +13,8 @@ class LayerCacheView:
     block_table: torch.Tensor = None            # int32 (B, W), this step's requests in batch order
     writes: bool = True
     state: torch.Tensor = None                  # (slots, *state_shape); index with batch.state_slots
+    runs: dict = field(default_factory=dict)    # name of a tensor per run of tokens -> (pages, *page shape)
+    run_table: torch.Tensor = None              # int32 (B, W): the pages of each request's runs
 
 
 class CacheStorage:
@@ -84,6 +86,11 @@ class CacheStorage:
             local = m.groups[g].planes.index(plane)
             view.paged = {name: tensor[local] for name, tensor in self.paged[g].items()}
             view.block_table = self._block_tables[g]
+        r = m.run_group_of_plane[plane]
+        if r >= 0:
+            local = m.groups[r].planes.index(plane)
+            view.runs = {name: tensor[local] for name, tensor in self.paged[r].items()}
+            view.run_table = self._block_tables[r]
         s = m.state_group_of_plane[plane]
         if s >= 0:
             local = m.state_groups[s].planes.index(plane)

@@ -204,7 +204,7 @@ __device__ __forceinline__ float capped(float v, const ScoreScale& s) {
   if (s.in == 0.f) return v;
   return s.out * (1.f - 2.f * __builtin_amdgcn_rcpf(fast_exp2(v * s.in) + 1.f));
 }
-static float g_score_cap = 0.f;
+static thread_local float g_score_cap = 0.f;
 extern "C" void q3_set_score_cap(float cap) { g_score_cap = cap; }
 static inline ScoreScale make_score_scale(float scale) {
   ScoreScale s;
@@ -217,6 +217,52 @@ static inline ScoreScale make_score_scale(float scale) {
 typedef float score_scale_t;
 __device__ __forceinline__ float scale_of(float s) { return s; }
 static inline float make_score_scale(float scale) { return scale * 1.4426950408889634f; }
+#endif
+
+// A build with Q3_SIGMOID (attention_sigmoid.hip) has no softmax: a visible key counts with
+// sigmoid(s * scale + bias[head]) and nothing is divided by a sum. In the place of a row's running
+// maximum stands -bias log2(e), which never moves, so that the argument is formed as an exponent is
+// elsewhere; wherever results are joined every weight is one. `q3_set_sigmoid_bias` names the
+// biases (one per query head) of the launches that follow in the calling thread.
+#ifdef Q3_SIGMOID
+#define Q3_BIAS_PARAM , const float* __restrict__ score_bias
+#define Q3_BIAS_ARG , g_score_bias
+static thread_local const float* g_score_bias = nullptr;
+extern "C" void q3_set_sigmoid_bias(const float* bias) { g_score_bias = bias; }
+// sigmoid of an argument that is given times log2(e); minus infinity gives nothing
+__device__ __forceinline__ float sigmoid_log2(float x) { return __builtin_amdgcn_rcpf(1.f + fast_exp2(-x)); }
+#else
+#define Q3_BIAS_PARAM
+#define Q3_BIAS_ARG
+#endif
+
+// A build with Q3_POOLED (attention_pooled.hip) sees, beside the window's tokens, one key and value per
+// run of `pool` tokens that ends at the row's position minus the window or before, from caches of
+// their own, laid out like the tokens' with a run in a token's place: a row at position p sees runs
+// 0 .. (p - window + 1) / pool - 1, which is causal attention with the row at that last run's number,
+// so the same tiles, masks and products serve both sources, one after the other, into the same
+// accumulators. `q3_set_runs` names the runs of the launches that follow in the calling thread.
+#ifdef Q3_POOLED
+struct RunSource {
+  const bf16_t* k;       // (pages, Hkv, page, D)
+  const bf16_t* v;       // (pages, Hkv, D, page)
+  const int* table;
+  int stride, num_pages, pool;
+};
+#define Q3_RUNS_PARAM , RunSource runs
+#define Q3_RUNS_ARG , g_runs
+static thread_local RunSource g_runs{};
+extern "C" void q3_set_runs(const void* k, const void* v, const int* table, int stride, int num_pages, int pool) {
+  g_runs = RunSource{(const bf16_t*)k, (const bf16_t*)v, table, stride, num_pages, pool};
+}
+// how many runs a row at position `pos` sees
+__device__ __forceinline__ int runs_seen(int pos, int window, int pool) {
+  const int behind = pos - window + 1;
+  return behind > 0 ? behind / pool : 0;
+}
+#else
+#define Q3_RUNS_PARAM
+#define Q3_RUNS_ARG
 #endif
 
 // The softmax update of one block of 16 rows for one 32-key tile. s: this lane's
@@ -245,6 +291,12 @@ __device__ __forceinline__ Pack16 softmax_step(const f32x4_t (&s)[2], bool full,
       if (!seen) v[j] = -INFINITY;
     }
   }
+#ifdef Q3_SIGMOID
+  Pack16 weights;
+#pragma unroll
+  for (int j = 0; j < 8; ++j) weights.e[j] = (__bf16)sigmoid_log2(fmaf(v[j], scale_of(scale_log2), -m_run));
+  return weights;
+#else
   float mx = fmaxf(fmaxf(fmaxf(v[0], v[1]), fmaxf(v[2], v[3])), fmaxf(fmaxf(v[4], v[5]), fmaxf(v[6], v[7])));
   mx = quad_rows_max(mx);
   const float m_new = fmaxf(m_run, mx * scale_of(scale_log2));
@@ -270,6 +322,7 @@ __device__ __forceinline__ Pack16 softmax_step(const f32x4_t (&s)[2], bool full,
   }
   l_run += sum;
   return p;
+#endif
 }
 
 // Where the two 16-key blocks of the tile that starts at key0 lie in the caches
@@ -649,7 +702,7 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(
     const bf16_t* __restrict__ v_cache, int num_pages, const int* __restrict__ block_table, int bt_stride,
     const int* __restrict__ cu_q, const int* __restrict__ kv_lens, int Hq, int Hkv, int page, score_scale_t scale_log2,
     int window, int splits, float* __restrict__ ws_acc, float* __restrict__ ws_ml, DecodePrep prep,
-    const float* __restrict__ sink) {
+    const float* __restrict__ sink Q3_BIAS_PARAM Q3_RUNS_PARAM) {
   const int b = blockIdx.z, g_kv = blockIdx.y, split = blockIdx.x;
   const int G = Hq / Hkv;
   // a step of single tokens (PREP): sequence b's token is row b, and nothing is read to know it
@@ -726,9 +779,18 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(
   if (window > 0) tile_lo = max(0, first_pos - window + 1) / FAST_TILE;
   int tile_hi = (kv_seen + FAST_TILE - 1) / FAST_TILE;
   if (fresh && window == 1) tile_hi = tile_lo;  // the new key alone is visible
+#ifdef Q3_POOLED
+  // the runs' tiles come first in the sequence of tiles that the splits share out
+  const int run_tiles = (runs_seen(first_pos + q_len - 1, window, runs.pool) + FAST_TILE - 1) / FAST_TILE;
+  const int all_tiles = run_tiles + max(tile_hi - tile_lo, 0);
+  const int per_split = (all_tiles + splits - 1) / splits;
+  const int s0 = min(split * per_split, all_tiles), s1 = min(s0 + per_split, all_tiles);
+  const int t0 = tile_lo + max(s0 - run_tiles, 0), t1 = tile_lo + max(s1 - run_tiles, 0);
+#else
   const int per_split = (max(tile_hi - tile_lo, 0) + splits - 1) / splits;
   const int t0 = tile_lo + split * per_split;
   const int t1 = min(tile_hi, t0 + per_split);
+#endif
   // the first tile's keys are on their way while the query rows are prepared
   if constexpr (!ahead)
     t_first = first_tile_keys<D>(a_first, k_cache, v_cache, num_pages, bt_row, Hkv, g_kv, page, t0 + wave, t1, kv_seen);
@@ -762,7 +824,11 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(
   f32x4_t acc[1][D / 16];
 #pragma unroll
   for (int nb = 0; nb < D / 16; ++nb) acc[0][nb] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#ifdef Q3_SIGMOID
+  float m_run[1] = {col < rows ? -score_bias[g_kv * G + col % G] * 1.4426950408889634f : 0.f}, l_run[1] = {0.f};
+#else
   float m_run[1] = {-INFINITY}, l_run[1] = {0.f};
+#endif
   if constexpr (ahead)
     attend_tiles_ahead<D, 1>(qreg, a_first, v_first, p_second, k_cache, v_cache, num_pages, bt_row, bt_stride, Hkv,
                              g_kv, page, ahead_first, tile_hi, ahead_step, kv_seen, row_pos, win, scale_log2, acc,
@@ -770,6 +836,21 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(
   else
     attend_tiles<D, 1>(qreg, a_first, t_first, k_cache, v_cache, num_pages, bt_row, Hkv, g_kv, page, t0 + wave, t1, 4,
                        kv_seen, row_pos, win, scale_log2, acc, m_run, l_run);
+#ifdef Q3_SIGMOID
+  m_run[0] = 0.f;
+#endif
+#ifdef Q3_POOLED
+  {
+    int run_pos[1];
+    run_pos[0] = runs_seen(row_pos[0], window, runs.pool) - 1;
+    const int* run_row = runs.table + (size_t)b * runs.stride;
+    const int run_first = s0 + wave, run_last = min(s1, run_tiles), run_count = kv_len / runs.pool;
+    t_first = first_tile_keys<D>(a_first, runs.k, runs.v, runs.num_pages, run_row, Hkv, g_kv, page, run_first, run_last,
+                                 run_count);
+    attend_tiles<D, 1>(qreg, a_first, t_first, runs.k, runs.v, runs.num_pages, run_row, Hkv, g_kv, page, run_first,
+                       run_last, 4, run_count, run_pos, 0, scale_log2, acc, m_run, l_run);
+  }
+#endif
 
   // this lane's sum covers its own keys only
   float l = l_run[0];
@@ -808,7 +889,11 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(
   const int token = q0 + r / G, head = g_kv * G + r % G;
   if (splits == 1) {
     // a sink joins the denominator once, as 2^(sink log2(e) - maximum): here, or in the merge of the splits
+#ifdef Q3_SIGMOID
+    const float inv = 1.f;
+#else
     const float inv = 1.f / (sink ? lr + exp2f(sink[head] * 1.4426950408889634f - mr) : lr);
+#endif
     for (int d = dd; d < D; d += 16) {
       float o = sh_acc[0][r][d] + sh_acc[1][r][d] + sh_acc[2][r][d] + sh_acc[3][r][d];
       if (PREP && w5 > 0.f) o += sh_v[d] * w5;
@@ -880,7 +965,11 @@ __global__ __launch_bounds__(256) void attn_decode_reduce_kernel(
       const float e = ml.x > -INFINITY ? exp2f(ml.x - m_all) : 0.f;
       float l_all = wave_sum(ml.y * e);
       if (sink) l_all += exp2f(sink[g_kv * G + r % G] * 1.4426950408889634f - m_all);
+#ifdef Q3_SIGMOID
+      if (lane < splits) sh_w[r][lane] = 1.f;
+#else
       if (lane < splits) sh_w[r][lane] = l_all > 0.f ? e / l_all : 0.f;   // a row that saw no key at all: zeros
+#endif
     }
   }
   __syncthreads();
@@ -1015,6 +1104,12 @@ __device__ __forceinline__ void softmax_tile(const f32x4_t (&s)[KB4], bool full,
       if (!seen) v[j] = -INFINITY;
     }
   }
+#ifdef Q3_SIGMOID
+#pragma unroll
+  for (int j = 0; j < N; ++j)
+    p[(j >> 2) % (KB4 / 2)].e[4 * ((j >> 2) / (KB4 / 2)) + (j & 3)] =
+        (__bf16)sigmoid_log2(fmaf(v[j], scale_of(scale_log2), -m_run));
+#else
   // the scores are matrix results or minus infinity, never NaN: the three-operand maximum as
   // it is (the compiler's own first makes every operand a quiet NaN, one instruction each)
   // (one statement for a tile of 64 keys: after every statement of assembly the compiler leaves a wait state)
@@ -1052,6 +1147,7 @@ __device__ __forceinline__ void softmax_tile(const f32x4_t (&s)[KB4], bool full,
     m_run = m_new;
   }
   l_run += sum;
+#endif
 }
 
 template <int D, int TILE, int STAGES>
@@ -1060,7 +1156,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
     const bf16_t* __restrict__ v_cache, int num_pages, const int* __restrict__ block_table, int bt_stride,
     const int* __restrict__ cu_q, const int* __restrict__ kv_lens, int Hq, int Hkv, int page, score_scale_t scale_log2,
     int window, int tokens_per_block, int key_splits, float* __restrict__ part_acc, float* __restrict__ part_ml,
-    const float* __restrict__ sink) {
+    const float* __restrict__ sink Q3_BIAS_PARAM Q3_RUNS_PARAM) {
   typedef PrefillSmem<D, TILE> SM;
   constexpr int KB4 = TILE / 16;  // 16-key blocks per tile
   __shared__ __attribute__((aligned(16))) unsigned char smem[STAGES * SM::STAGE];
@@ -1085,7 +1181,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
   // descending orders and the mirrored one: 87 us against 95, 89 and 88)
   const int half_tiles = (n_tiles + 1) / 2;
   const int tile = tile_index < half_tiles ? n_tiles - 1 - tile_index : tile_index - half_tiles;
-  const int kv_len = kv_lens[b];
+  int kv_len = kv_lens[b];
   const int tid = threadIdx.x;
   const int lane = tid & 63, wave = tid >> 6;
   const int col = lane & 15, grp = lane >> 4;
@@ -1129,7 +1225,13 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
   for (int qb = 0; qb < 2; ++qb)
 #pragma unroll
     for (int nb = 0; nb < D / 16; ++nb) acc[qb][nb] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#ifdef Q3_SIGMOID
+  float m_run[2], l_run[2] = {0.f, 0.f};
+#pragma unroll
+  for (int qb = 0; qb < 2; ++qb) m_run[qb] = -score_bias[row_head[qb]] * 1.4426950408889634f;
+#else
   float m_run[2] = {-INFINITY, -INFINITY}, l_run[2] = {0.f, 0.f};
+#endif
 
   // the block's range of tiles: from the window's start of its first row to its last row's position
   const int blk_first_tok = tile * tokens_per_block;
@@ -1140,6 +1242,22 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
   // and this wavefront's own (a wavefront whose rows do not exist has none)
   int my_lo = tile_lo, my_hi = pos_max >= 0 ? pos_max / TILE + 1 : 0;
   if (window > 0 && pos_max >= 0) my_lo = max(0, pos_min - window + 1) / TILE;
+#ifdef Q3_POOLED
+  // the same of the runs, ahead of the tokens in the sequence of tiles that the splits share out
+  int run_lo = 0, run_hi = (runs_seen(first_pos + blk_last_tok, window, runs.pool) + TILE - 1) / TILE;
+  if (key_splits > 1) {
+    const int run_tiles = run_hi, all = run_tiles + tile_hi - tile_lo;
+    const int share = (all + key_splits - 1) / key_splits;
+    const int s0 = min(all, split * share), s1 = min(all, s0 + share);
+    run_lo = min(s0, run_tiles);
+    run_hi = min(s1, run_tiles);
+    const int base = tile_lo;
+    tile_lo = base + max(s0 - run_tiles, 0);
+    tile_hi = base + max(s1 - run_tiles, 0);
+    my_lo = max(my_lo, tile_lo);
+    my_hi = min(my_hi, tile_hi);
+  }
+#else
   if (key_splits > 1) {  // this block's share of the range (it may be empty)
     const int share = (tile_hi - tile_lo + key_splits - 1) / key_splits;
     tile_lo = min(tile_hi, tile_lo + split * share);
@@ -1147,6 +1265,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
     my_lo = max(my_lo, tile_lo);
     my_hi = min(my_hi, tile_hi);
   }
+#endif
   const int* bt_row = block_table + (size_t)b * bt_stride;
 
   // The copy of a tile from the caches into a stage. Place s (a 16-byte piece) of the keys'
@@ -1208,7 +1327,9 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
     asm volatile("s_mov_b32 m0, %1\n\tglobal_load_lds_dwordx4 %0, off" ::"v"(src), "s"(lds) : "memory", "m0");
   };
 
-  auto plain_tile = [&](int t) { return t * TILE + TILE <= kv_len && window == 0; };
+  // (a page is given back only when every later row's window has left it, so a tile that the first row's
+  // window covers from its first key on is all there)
+  auto plain_tile = [&](int t) { return t * TILE + TILE <= kv_len && (window == 0 || t * TILE > first_pos - window); };
   auto copy_direct = [&](int t, int stage) {
     const int key0 = t * TILE;
     // this wavefront's kilobyte of each turn
@@ -1303,6 +1424,45 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
 #pragma unroll
     for (int i = 0; i < D / 32; ++i) asm volatile("" : "+v"(qreg[qb][i].v));
 
+#ifdef Q3_POOLED
+  // the runs first, then the tokens: what the tile loop works with is exchanged in between
+  const bf16_t *token_k = k_cache, *token_v = v_cache;
+  const int *token_row = bt_row;
+  const int token_pages = num_pages, token_len = kv_len, token_window = window;
+  const int token_lo = tile_lo, token_hi = tile_hi, token_my_lo = my_lo, token_my_hi = my_hi;
+  const int token_pos[2] = {row_pos[0], row_pos[1]}, token_max = pos_max, token_min = pos_min;
+  k_cache = runs.k;
+  v_cache = runs.v;
+  num_pages = runs.num_pages;
+  bt_row = runs.table + (size_t)b * runs.stride;
+  kv_len = token_len / runs.pool;
+  window = 0;
+#pragma unroll
+  for (int qb = 0; qb < 2; ++qb) row_pos[qb] = runs_seen(token_pos[qb], token_window, runs.pool) - 1;
+  pos_max = runs_seen(token_max, token_window, runs.pool) - 1;
+  pos_min = token_max >= 0 ? runs_seen(token_min, token_window, runs.pool) - 1 : -1;
+  tile_lo = my_lo = run_lo;
+  tile_hi = run_hi;
+  my_hi = min(run_hi, pos_max >= 0 ? pos_max / TILE + 1 : 0);
+#pragma nounroll
+  for (int source = 0; source < 2; ++source) {
+  if (source == 1) {
+    k_cache = token_k;
+    v_cache = token_v;
+    num_pages = token_pages;
+    bt_row = token_row;
+    kv_len = token_len;
+    window = token_window;
+    row_pos[0] = token_pos[0];
+    row_pos[1] = token_pos[1];
+    pos_max = token_max;
+    pos_min = token_min;
+    tile_lo = token_lo;
+    tile_hi = token_hi;
+    my_lo = token_my_lo;
+    my_hi = token_my_hi;
+  }
+#endif
   // tiles are worked through in spans whose table entries fit sh_pages
   const int tiles_per_span = max(1, (PREFILL_PAGES - 4) * page / TILE);
   for (int span_lo = tile_lo; span_lo < tile_hi; span_lo += tiles_per_span) {
@@ -1413,6 +1573,9 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
       __syncthreads();
     }
   }
+#ifdef Q3_POOLED
+  }
+#endif
 #pragma unroll
   for (int qb = 0; qb < 2; ++qb) {
     float l = l_run[qb];
@@ -1426,11 +1589,18 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
       for (int nb = 0; nb < D / 16; ++nb)
         *reinterpret_cast<float4*>(o + 16 * nb) =
             make_float4(acc[qb][nb][0], acc[qb][nb][1], acc[qb][nb][2], acc[qb][nb][3]);
+#ifdef Q3_SIGMOID
+      m_run[qb] = 0.f;
+#endif
       if (grp == 0) *reinterpret_cast<float2*>(part_ml + slot * 2) = make_float2(m_run[qb], l);
       continue;
     }
     if (sink) l += fast_exp2(sink[row_head[qb]] * 1.4426950408889634f - m_run[qb]);
+#ifdef Q3_SIGMOID
+    const float inv = 1.f;
+#else
     const float inv = 1.f / l;
+#endif
     bf16_t* o = out + (size_t)row_tok[qb] * Hq * D + (size_t)row_head[qb] * D + 4 * grp;
 #pragma unroll
     for (int nb = 0; nb < D / 16; ++nb) {
@@ -1477,7 +1647,11 @@ __global__ __launch_bounds__(256) void attn_prefill_merge_kernel(bf16_t* __restr
       l_all += ml.y * w;
     }
     if (sink) l_all += fast_exp2(sink[row] * 1.4426950408889634f - m_all);
+#ifdef Q3_SIGMOID
+    const float inv = 1.f;
+#else
     const float inv = 1.f / l_all;
+#endif
     union {
       uint2 u;
       bf16_t e[4];
@@ -1519,17 +1693,23 @@ static int launch_fast(const void* q, int q_stride, void* out, const void* k_cac
                        const float* sink, hipStream_t stream) {
   const int G = Hq / Hkv;
   const score_scale_t scale_log2 = make_score_scale(scale);
+#ifdef Q3_POOLED
+  if (window <= 0 || g_runs.k == nullptr || g_runs.pool <= 0) return Q3_ERR_BAD_ARGUMENT;
+#endif
+#ifdef Q3_SIGMOID
+  if (window != 0 || g_score_bias == nullptr || sink != nullptr) return Q3_ERR_BAD_ARGUMENT;
+#endif
   if (min_q_len * G <= 16) {
     if (window == 0)
       hipLaunchKernelGGL((attn_decode_kernel<D, false, float, true>), dim3(splits, Hkv, B), dim3(256), 0, stream,
                          (const bf16_t*)q, q_stride, (bf16_t*)out, (const bf16_t*)k_cache, (const bf16_t*)v_cache,
                          num_pages, block_table, bt_stride, cu_q, kv_lens, Hq, Hkv, page, scale_log2, window, splits,
-                         ws_acc, ws_ml, DecodePrep{}, sink);
+                         ws_acc, ws_ml, DecodePrep{}, sink Q3_BIAS_ARG Q3_RUNS_ARG);
     else
       hipLaunchKernelGGL((attn_decode_kernel<D, false, float, false>), dim3(splits, Hkv, B), dim3(256), 0, stream,
                          (const bf16_t*)q, q_stride, (bf16_t*)out, (const bf16_t*)k_cache, (const bf16_t*)v_cache,
                          num_pages, block_table, bt_stride, cu_q, kv_lens, Hq, Hkv, page, scale_log2, window, splits,
-                         ws_acc, ws_ml, DecodePrep{}, sink);
+                         ws_acc, ws_ml, DecodePrep{}, sink Q3_BIAS_ARG Q3_RUNS_ARG);
     if (splits > 1)
       hipLaunchKernelGGL(attn_decode_reduce_kernel<D>, dim3(Hkv, B), dim3(256), 0, stream, (bf16_t*)out, cu_q, Hq,
                          Hkv, splits, ws_acc, ws_ml, sink);
@@ -1543,7 +1723,7 @@ static int launch_fast(const void* q, int q_stride, void* out, const void* k_cac
     hipLaunchKernelGGL((attn_prefill_kernel<D, PF_TILE, PF_STAGES>), dim3(Hkv, tiles * key_splits, B), dim3(256), 0,
                        stream, (const bf16_t*)q, q_stride, (bf16_t*)out, (const bf16_t*)k_cache,
                        (const bf16_t*)v_cache, num_pages, block_table, bt_stride, cu_q, kv_lens, Hq, Hkv, page,
-                       scale_log2, window, tokens_per_block, key_splits, part_acc, part_ml, sink);
+                       scale_log2, window, tokens_per_block, key_splits, part_acc, part_ml, sink Q3_BIAS_ARG Q3_RUNS_ARG);
     if (key_splits > 1)
       hipLaunchKernelGGL(attn_prefill_merge_kernel<D>, dim3(max_q_len, B), dim3(256), 0, stream,
                          (bf16_t*)out, cu_q, Hq, Hkv, key_splits, part_acc, part_ml, sink);
@@ -1551,6 +1731,7 @@ static int launch_fast(const void* q, int q_stride, void* out, const void* k_cac
   return q3_launch_status();
 }
 
+#if !defined(Q3_POOLED) && !defined(Q3_SIGMOID)
 template <int D, typename W>
 static int launch_decode_prep(const void* qkv, void* out, const void* k_cache, const void* v_cache, int num_pages,
                               const int* block_table, int bt_stride, const int* cu_q, const int* kv_lens, int B,
@@ -1572,6 +1753,7 @@ static int launch_decode_prep(const void* qkv, void* out, const void* k_cache, c
                        (const int*)nullptr, Hq, Hkv, splits, ws_acc, ws_ml, (const float*)nullptr);
   return q3_launch_status();
 }
+#endif
 
 // Whether the matrix-core kernels take this problem; otherwise the general kernel does.
 extern "C" int q3_paged_attention_fast_path(int Hq, int Hkv, int D, int page, int dtype) {
@@ -1625,8 +1807,8 @@ extern "C" int q3_paged_attention(const void* q, int q_stride, void* out, const 
                             T_, Hq, Hkv, page, scale, window, max_q_len, min_q_len, splits, ws_acc, ws_ml,
                             prompt_splits, prompt_workspace, sink, stream);
   }
-#ifdef Q3_SCORE_CAP
-  return Q3_ERR_UNSUPPORTED;      // the capped build has the matrix-core kernels only
+#if defined(Q3_SCORE_CAP) || defined(Q3_POOLED) || defined(Q3_SIGMOID)
+  return Q3_ERR_UNSUPPORTED;      // these builds have the matrix-core kernels only
 #endif
   Q3_DISPATCH_DTYPE(dtype, TT, return launch_general<TT>(q, q_stride, out, k_cache, v_cache, num_pages,
                                                         block_table, bt_stride, cu_q, kv_lens, B, Hq, Hkv,
@@ -1634,6 +1816,7 @@ extern "C" int q3_paged_attention(const void* q, int q_stride, void* out, const 
   return Q3_ERR_BAD_ARGUMENT;
 }
 
+#if !defined(Q3_POOLED) && !defined(Q3_SIGMOID)
 // Whether `q3_decode_attention` takes a step of single tokens with these sizes: what the
 // matrix-core kernels take, with a rotation (if any) over the whole head.
 extern "C" int q3_decode_attention_takes(int Hq, int Hkv, int D, int page, int dtype, int rotary_dim) {
@@ -1681,3 +1864,4 @@ extern "C" int q3_decode_attention(const void* qkv, void* out, void* k_cache, vo
   Q3_DECODE_PREP(128, bf16_t);
 #undef Q3_DECODE_PREP
 }
+#endif

@@ -15,6 +15,26 @@ __global__ void embed_rows_kernel(const int* __restrict__ ids, const T* __restri
   for (int j = threadIdx.x; j < H; j += blockDim.x) dst[j] = ok ? to_float(row[j]) * scale : 0.f;
 }
 
+// x[i] <- cap * tanh(x[i] / cap), float32, in place; four numbers a thread where they are whole.
+__global__ void soft_cap_kernel(float* __restrict__ x, long n, float cap) {
+  const long i = ((long)blockIdx.x * blockDim.x + threadIdx.x) * 4;
+  if (i + 4 <= n) {
+    float4 v = *reinterpret_cast<float4*>(x + i);
+    v.x = cap * tanhf(v.x / cap), v.y = cap * tanhf(v.y / cap), v.z = cap * tanhf(v.z / cap), v.w = cap * tanhf(v.w / cap);
+    *reinterpret_cast<float4*>(x + i) = v;
+  } else {
+    for (long k = i; k < n; ++k) x[k] = cap * tanhf(x[k] / cap);
+  }
+}
+
+extern "C" int q3_soft_cap(float* x, long n, float cap, hipStream_t stream) {
+  if (n <= 0 || !(cap > 0.f) || (size_t)x % 16) return Q3_ERR_BAD_ARGUMENT;
+  const long blocks = (n + 1023) / 1024;
+  if (blocks > 0x7fffffffL) return Q3_ERR_UNSUPPORTED;
+  hipLaunchKernelGGL(soft_cap_kernel, dim3((unsigned)blocks), dim3(256), 0, stream, x, n, cap);
+  return q3_launch_status();
+}
+
 // out[t, j] = act(gate[t, j]) * up[t, j] for rows that interleave the two:
 // gate_up[t, 2j] = gate[t, j], gate_up[t, 2j + 1] = up[t, j]. ACT 0: silu(g) = g / (1 + exp(-g));
 // 1: the tanh form of gelu, 0.5 g (1 + tanh(sqrt(2/pi) (g + 0.044715 g^3))); 2: the exact gelu,

@@ -69,12 +69,186 @@ __global__ void softcap_prepare_kernel(const float* __restrict__ rows, long row_
   }
 }
 
+// Queries, keys and values without norms, turned by the position, i and i + half together. One block
+// per token, a wavefront per head in turn. The row is [q: H dim | k: G dim | v: G vdim | ...] float32,
+// `bias` covers q, k and v (null: none); with `values_are_keys` there is no v and a token's value is
+// its key before it turns. The first 2 * half numbers of every head of q and k turn by position *
+// inv_freq[i], cos and sin multiplied by `factor`; they are formed once per token, in shared memory. q
+// goes to `q_out`, k and v into the token's place in the cache.
+//
+// `runs` (single tokens only): a token that ends a run of `pool` tokens also leaves the means of the
+// run's keys and values, as the cache holds them, in the run's place: the others' are read from the
+// cache, where earlier steps have put them, its own are at hand.
+#define Q3_TURN_HALF_MOST 256
+struct RunPlaces {
+  void* k;               // (pages, G, page, dim)
+  void* v;               // (pages, G, vdim, page)
+  const int* table;
+  int width, pool;
+};
+
+template <typename TA>
+__device__ inline float rounded(float v) {
+  return to_float(from_float<TA>(v));
+}
+
+template <typename TA>
+__global__ void __launch_bounds__(256) turn_prepare_kernel(
+    const float* __restrict__ rows, long row_stride, const float* __restrict__ bias, const float* __restrict__ inv_freq,
+    int half, float factor, const int* __restrict__ positions, const int* __restrict__ seq_index,
+    const int* __restrict__ block_table, int table_width, TA* k_cache, TA* v_cache, int page, TA* __restrict__ q_out,
+    int H, int G, int dim, int vdim, int values_are_keys, RunPlaces runs) {
+  __shared__ float cs[Q3_TURN_HALF_MOST], sn[Q3_TURN_HALF_MOST];
+  const int t = blockIdx.x;
+  const int wave = threadIdx.x / Q3_WAVE, lane = threadIdx.x % Q3_WAVE, waves = blockDim.x / Q3_WAVE;
+  const float* row = rows + (size_t)t * row_stride;
+  const int nq = H * dim, nk = G * dim;
+  const int pos = positions[t];
+  for (int i = threadIdx.x; i < half; i += blockDim.x) {
+    const float angle = (float)pos * inv_freq[i];
+    cs[i] = cosf(angle) * factor;
+    sn[i] = sinf(angle) * factor;
+  }
+  const int* table = block_table + (size_t)seq_index[t] * table_width;
+  const int pg = pos / page < table_width ? table[pos / page] : -1;
+  const int off = pos % page;
+  const bool ends_run = runs.k && (pos + 1) % runs.pool == 0;
+  int run_page = -1, run_off = 0;
+  if (ends_run) {
+    const int r = pos / runs.pool;
+    if (r / page < runs.width) run_page = runs.table[(size_t)seq_index[t] * runs.width + r / page];
+    run_off = r % page;
+  }
+  __syncthreads();
+  auto turned = [&](const float* x, const float* add, int e) {
+    const float own = x[e] + (add ? add[e] : 0.f);
+    if (e >= 2 * half) return own;
+    const int p = e < half ? e + half : e - half;
+    const float other = x[p] + (add ? add[p] : 0.f);
+    return e < half ? own * cs[e] - other * sn[e] : own * cs[p] + other * sn[p];
+  };
+  for (int h = wave; h < H; h += waves) {
+    const float* x = row + h * dim;
+    const float* add = bias ? bias + h * dim : nullptr;
+    for (int e = lane; e < dim; e += Q3_WAVE) q_out[(size_t)t * nq + h * dim + e] = from_float<TA>(turned(x, add, e));
+  }
+  if (pg < 0) return;
+  for (int g = wave; g < G; g += waves) {
+    const float* x = row + nq + g * dim;
+    const float* add = bias ? bias + nq + g * dim : nullptr;
+    for (int e = lane; e < dim; e += Q3_WAVE) {
+      const TA key = from_float<TA>(turned(x, add, e));
+      k_cache[(((size_t)pg * G + g) * page + off) * dim + e] = key;
+      if (run_page >= 0) {
+        float sum = 0.f;
+        for (int j = pos - runs.pool + 1; j < pos; ++j) {
+          const int from = table[j / page];
+          sum += from < 0 ? 0.f : to_float(k_cache[(((size_t)from * G + g) * page + j % page) * dim + e]);
+        }
+        sum += to_float(key);
+        ((TA*)runs.k)[(((size_t)run_page * G + g) * page + run_off) * dim + e] = from_float<TA>(sum / (float)runs.pool);
+      }
+    }
+    const float* y = values_are_keys ? x : row + nq + nk + g * vdim;
+    const float* add_v = values_are_keys ? add : (bias ? bias + nq + nk + g * vdim : nullptr);
+    for (int e = lane; e < vdim; e += Q3_WAVE) {
+      const TA value = from_float<TA>(y[e] + (add_v ? add_v[e] : 0.f));
+      v_cache[(((size_t)pg * G + g) * vdim + e) * page + off] = value;
+      if (run_page >= 0) {
+        float sum = 0.f;
+        for (int j = pos - runs.pool + 1; j < pos; ++j) {
+          const int from = table[j / page];
+          sum += from < 0 ? 0.f : to_float(v_cache[(((size_t)from * G + g) * vdim + e) * page + j % page]);
+        }
+        sum += to_float(value);
+        ((TA*)runs.v)[(((size_t)run_page * G + g) * vdim + e) * page + run_off] = from_float<TA>(sum / (float)runs.pool);
+      }
+    }
+  }
+}
+
+extern "C" int q3_turn_prepare(const float* rows, long row_stride, const float* bias, const float* inv_freq, int half,
+                               float factor, const int* positions, const int* seq_index, const int* block_table,
+                               int table_width, void* k_cache, void* v_cache, int page, void* q_out, int T, int H, int G,
+                               int dim, int vdim, int values_are_keys, void* run_k, void* run_v, const int* run_table,
+                               int run_width, int pool, int act_dtype, hipStream_t stream) {
+  if (T <= 0 || H <= 0 || G <= 0 || H % G || dim <= 0 || vdim <= 0 || half < 0 || 2 * half > dim || !k_cache || !v_cache ||
+      !block_table || page <= 0 || table_width <= 0 || (half > 0 && !inv_freq) || (values_are_keys && dim != vdim))
+    return Q3_ERR_BAD_ARGUMENT;
+  if (run_k && (!run_v || !run_table || run_width <= 0 || pool <= 0)) return Q3_ERR_BAD_ARGUMENT;
+  if (half > Q3_TURN_HALF_MOST) return Q3_ERR_UNSUPPORTED;
+  const RunPlaces runs{run_k, run_v, run_table, run_width, pool};
+  Q3_DISPATCH_DTYPE(act_dtype, TA,
+                    hipLaunchKernelGGL(turn_prepare_kernel<TA>, dim3(T), dim3(256), 0, stream, rows, row_stride, bias,
+                                       inv_freq, half, factor, positions, seq_index, block_table, table_width,
+                                       (TA*)k_cache, (TA*)v_cache, page, (TA*)q_out, H, G, dim, vdim, values_are_keys,
+                                       runs));
+  return q3_launch_status();
+}
+
+// The same means for steps of any rows, after the step's keys and values are in the cache: grid (runs
+// that a sequence may complete, G, B), a block per run; a run is formed if the step brought its last
+// token. Sums take the tokens in their order, as above.
+template <typename TA>
+__global__ void __launch_bounds__(256) pool_runs_kernel(const TA* __restrict__ k_cache, const TA* __restrict__ v_cache,
+                                                        const int* __restrict__ block_table, int table_width,
+                                                        const int* __restrict__ cu, const int* __restrict__ kv_lens,
+                                                        TA* __restrict__ run_k, TA* __restrict__ run_v,
+                                                        const int* __restrict__ run_table, int run_width, int pool, int G,
+                                                        int dim, int vdim, int page) {
+  const int b = blockIdx.z, g = blockIdx.y;
+  const int kv_len = kv_lens[b], first_pos = kv_len - (cu[b + 1] - cu[b]);
+  const int r = first_pos / pool + blockIdx.x;          // first_pos's own run is the first that may end now
+  if (kv_len <= first_pos || (r + 1) * pool > kv_len || r / page >= run_width) return;
+  const int run_page = run_table[(size_t)b * run_width + r / page];
+  if (run_page < 0) return;
+  const int run_off = r % page;
+  const int* table = block_table + (size_t)b * table_width;
+  for (int e = threadIdx.x; e < dim + vdim; e += blockDim.x) {
+    const bool key = e < dim;
+    const int c = key ? e : e - dim;
+    float sum = 0.f;
+    for (int j = r * pool; j < (r + 1) * pool; ++j) {
+      const int pg = j / page < table_width ? table[j / page] : -1;
+      if (pg < 0) continue;
+      const size_t head = (size_t)pg * G + g;
+      sum += key ? to_float(k_cache[(head * page + j % page) * dim + c]) : to_float(v_cache[(head * vdim + c) * page + j % page]);
+    }
+    const size_t head = (size_t)run_page * G + g;
+    const TA mean = from_float<TA>(sum / (float)pool);
+    if (key)
+      run_k[(head * page + run_off) * dim + c] = mean;
+    else
+      run_v[(head * vdim + c) * page + run_off] = mean;
+  }
+}
+
+extern "C" int q3_pool_runs(const void* k_cache, const void* v_cache, const int* block_table, int table_width,
+                            const int* cu, const int* kv_lens, void* run_k, void* run_v, const int* run_table,
+                            int run_width, int pool, int B, int max_q_len, int G, int dim, int vdim, int page,
+                            int act_dtype, hipStream_t stream) {
+  if (B <= 0 || max_q_len <= 0 || G <= 0 || dim <= 0 || vdim <= 0 || page <= 0 || pool <= 0 || table_width <= 0 ||
+      run_width <= 0 || !k_cache || !v_cache || !run_k || !run_v || !block_table || !run_table)
+    return Q3_ERR_BAD_ARGUMENT;
+  if (B > 65535 || G > 65535) return Q3_ERR_UNSUPPORTED;
+  // a step of n tokens ends at most (n + pool - 1) / pool runs
+  const int most = (max_q_len + pool - 1) / pool;
+  Q3_DISPATCH_DTYPE(act_dtype, TA,
+                    hipLaunchKernelGGL(pool_runs_kernel<TA>, dim3(most, G, B), dim3(256), 0, stream, (const TA*)k_cache,
+                                       (const TA*)v_cache, block_table, table_width, cu, kv_lens, (TA*)run_k, (TA*)run_v,
+                                       run_table, run_width, pool, G, dim, vdim, page));
+  return q3_launch_status();
+}
+
 // The general form: one wavefront per (token, head). Keys are taken in tiles of 64 that start at
 // absolute positions in steps of 64, one key a lane: score = (q . k) scale, capped as
 // cap * tanh(score / cap) when cap > 0; running maximum and sum in float32; then every lane sums
 // its columns of the values with the tile's weights. The result is divided by the sum and
-// multiplied by sigmoid(gate[t, h]) when a gate is given. With `sink` (H floats) the sum also holds
-// exp(sink[h]), a term that has no key and no value and is not scaled.
+// multiplied by sigmoid(gate) when a gate is given: a number per head, or one per column with
+// `gate_wide`. With `sink` (H floats) the sum also holds exp(sink[h]), a term that has no key and no
+// value and is not scaled. With `runs` the token also sees one key and value per run of `pool` tokens
+// that ends at its position minus the window or before, in the same softmax, ahead of the tokens.
+// With `score_bias` (H floats) there is no softmax: a key counts with sigmoid(score + score_bias[h]).
 #define Q3_CAP_DIM_MOST 512
 #define Q3_CAP_VSLICES 8
 template <typename TA>
@@ -82,67 +256,83 @@ __global__ void __launch_bounds__(64) softcap_attention_kernel(
     const TA* __restrict__ q, const TA* __restrict__ k_cache, const TA* __restrict__ v_cache,
     const int* __restrict__ block_table, int table_width, const int* __restrict__ seq_index,
     const int* __restrict__ positions, float scale, float cap, int window, const float* __restrict__ gate,
-    long gate_stride, TA* __restrict__ out, int H, int G, int dim, int vdim, int page, int v_transposed,
-    const float* __restrict__ sink) {
+    long gate_stride, int gate_wide, TA* __restrict__ out, int H, int G, int dim, int vdim, int page, int v_transposed,
+    const float* __restrict__ sink, RunPlaces runs, const float* __restrict__ score_bias) {
   __shared__ float sq[Q3_CAP_DIM_MOST];
   __shared__ float sp[64];
   const int lane = threadIdx.x;
   const int t = blockIdx.x, h = blockIdx.y;
   const int g = h / (H / G);
   const int pos = positions[t];
-  const int* table = block_table + (size_t)seq_index[t] * table_width;
   const TA* qr = q + ((size_t)t * H + h) * dim;
   for (int e = lane; e < dim; e += 64) sq[e] = to_float(qr[e]);
   __syncthreads();
-  const int lo = window > 0 ? (pos - window + 1 > 0 ? pos - window + 1 : 0) : 0;
-  float m = -INFINITY, l = 0.f;
+  const bool weighed = score_bias != nullptr;          // sigmoids, not a softmax
+  const float bias = weighed ? score_bias[h] : 0.f;
+  float m = weighed ? 0.f : -INFINITY, l = 0.f;
   float acc[Q3_CAP_VSLICES];
 #pragma unroll
   for (int i = 0; i < Q3_CAP_VSLICES; ++i) acc[i] = 0.f;
-  for (int j0 = lo / 64 * 64; j0 <= pos; j0 += 64) {
-    const int j = j0 + lane;
-    const bool valid = j >= lo && j <= pos;
-    float s = -INFINITY;
-    if (valid) {
-      const int pg = table[j / page];
-      const TA* kr = k_cache + (((size_t)(pg < 0 ? 0 : pg) * G + g) * page + j % page) * dim;
-      float dot = 0.f;
-      for (int e = 0; e < dim; ++e) dot += sq[e] * to_float(kr[e]);
-      s = dot * scale;
-      if (cap > 0.f) s = cap * tanhf(s / cap);
-    }
-    const float m_new = fmaxf(m, wave_max(s));
-    const float p = valid ? expf(s - m_new) : 0.f;
-    const float keep = m == -INFINITY ? 0.f : expf(m - m_new);
-    l = l * keep + wave_sum(p);
-    m = m_new;
-#pragma unroll
-    for (int i = 0; i < Q3_CAP_VSLICES; ++i) acc[i] *= keep;
-    sp[lane] = p;
-    __syncthreads();
-    const int last = pos - j0 < 63 ? pos - j0 : 63;
-    for (int jj = (lo > j0 ? lo - j0 : 0); jj <= last; ++jj) {
-      const float pj = sp[jj];
-      const int key = j0 + jj;
-      const int pg = table[key / page];
-      const size_t head = (size_t)(pg < 0 ? 0 : pg) * G + g;
-      const TA* vr = v_transposed ? v_cache + head * vdim * page + key % page : v_cache + (head * page + key % page) * vdim;
-      const int apart = v_transposed ? page : 1;
-#pragma unroll
-      for (int i = 0; i < Q3_CAP_VSLICES; ++i) {
-        const int c = lane + 64 * i;
-        if (c < vdim) acc[i] += pj * to_float(vr[(size_t)c * apart]);
+  // keys lo .. hi of one paged source
+  auto walk = [&](const TA* ks, const TA* vs, const int* table, int lo, int hi) {
+    for (int j0 = lo / 64 * 64; j0 <= hi; j0 += 64) {
+      const int j = j0 + lane;
+      const bool valid = j >= lo && j <= hi;
+      float s = -INFINITY;
+      if (valid) {
+        const int pg = table[j / page];
+        const TA* kr = ks + (((size_t)(pg < 0 ? 0 : pg) * G + g) * page + j % page) * dim;
+        float dot = 0.f;
+        for (int e = 0; e < dim; ++e) dot += sq[e] * to_float(kr[e]);
+        s = dot * scale;
+        if (cap > 0.f) s = cap * tanhf(s / cap);
       }
+      float p;
+      if (weighed) {
+        p = valid ? 1.f / (1.f + expf(-(s + bias))) : 0.f;
+      } else {
+        const float m_new = fmaxf(m, wave_max(s));
+        p = valid ? expf(s - m_new) : 0.f;
+        const float keep = m == -INFINITY ? 0.f : expf(m - m_new);
+        l = l * keep + wave_sum(p);
+        m = m_new;
+#pragma unroll
+        for (int i = 0; i < Q3_CAP_VSLICES; ++i) acc[i] *= keep;
+      }
+      sp[lane] = p;
+      __syncthreads();
+      const int last = hi - j0 < 63 ? hi - j0 : 63;
+      for (int jj = (lo > j0 ? lo - j0 : 0); jj <= last; ++jj) {
+        const float pj = sp[jj];
+        const int key = j0 + jj;
+        const int pg = table[key / page];
+        const size_t head = (size_t)(pg < 0 ? 0 : pg) * G + g;
+        const TA* vr = v_transposed ? vs + head * vdim * page + key % page : vs + (head * page + key % page) * vdim;
+        const int apart = v_transposed ? page : 1;
+#pragma unroll
+        for (int i = 0; i < Q3_CAP_VSLICES; ++i) {
+          const int c = lane + 64 * i;
+          if (c < vdim) acc[i] += pj * to_float(vr[(size_t)c * apart]);
+        }
+      }
+      __syncthreads();
     }
-    __syncthreads();
+  };
+  if (runs.k && pos - window + 1 > 0) {
+    const int seen = (pos - window + 1) / runs.pool;
+    walk((const TA*)runs.k, (const TA*)runs.v, runs.table + (size_t)seq_index[t] * runs.width, 0, seen - 1);
   }
-  const float open = gate ? 1.f / (1.f + expf(-gate[(size_t)t * gate_stride + h])) : 1.f;
+  walk(k_cache, v_cache, block_table + (size_t)seq_index[t] * table_width,
+       window > 0 ? (pos - window + 1 > 0 ? pos - window + 1 : 0) : 0, pos);
   if (sink) l += expf(sink[h] - m);
-  const float norm = open / l;
+  const float norm = weighed ? 1.f : 1.f / l;
 #pragma unroll
   for (int i = 0; i < Q3_CAP_VSLICES; ++i) {
     const int c = lane + 64 * i;
-    if (c < vdim) out[((size_t)t * H + h) * vdim + c] = from_float<TA>(acc[i] * norm);
+    if (c < vdim) {
+      const float open = gate ? 1.f / (1.f + expf(-gate[(size_t)t * gate_stride + (gate_wide ? h * vdim + c : h)])) : 1.f;
+      out[((size_t)t * H + h) * vdim + c] = from_float<TA>(acc[i] * (open * norm));
+    }
   }
 }
 
@@ -203,21 +393,23 @@ extern "C" int q3_headnorm_prepare(const float* rows, long row_stride, const flo
   return q3_launch_status();
 }
 
-// out[t, h, :] *= sigmoid(gate[t, h]) for a result that another kernel has left ungated.
+// out[t, h, :] *= sigmoid(gate[t, h]) for a result that another kernel has left ungated; with `per` 1
+// instead of vdim, a gate per column.
 template <typename TA>
-__global__ void gate_heads_kernel(TA* __restrict__ out, const float* __restrict__ gate, long gate_stride, int H, int vdim) {
+__global__ void gate_heads_kernel(TA* __restrict__ out, const float* __restrict__ gate, long gate_stride, int H, int vdim,
+                                  int per) {
   const int t = blockIdx.x;
   for (int e = threadIdx.x; e < H * vdim; e += blockDim.x) {
-    const float open = 1.f / (1.f + expf(-gate[(size_t)t * gate_stride + e / vdim]));
+    const float open = 1.f / (1.f + expf(-gate[(size_t)t * gate_stride + (per == 1 ? e : e / per)]));
     out[(size_t)t * H * vdim + e] = from_float<TA>(to_float(out[(size_t)t * H * vdim + e]) * open);
   }
 }
 
-extern "C" int q3_gate_heads(void* out, const float* gate, long gate_stride, int T, int H, int vdim, int act_dtype,
-                             hipStream_t stream) {
+extern "C" int q3_gate_heads(void* out, const float* gate, long gate_stride, int gate_wide, int T, int H, int vdim,
+                             int act_dtype, hipStream_t stream) {
   if (T <= 0 || H <= 0 || vdim <= 0) return Q3_ERR_BAD_ARGUMENT;
   Q3_DISPATCH_DTYPE(act_dtype, TA, hipLaunchKernelGGL(gate_heads_kernel<TA>, dim3(T), dim3(256), 0, stream, (TA*)out,
-                                                      gate, gate_stride, H, vdim));
+                                                      gate, gate_stride, H, vdim, gate_wide ? 1 : vdim));
   return q3_launch_status();
 }
 
@@ -237,19 +429,25 @@ extern "C" int q3_softcap_prepare(const float* rows, long row_stride, const floa
   return q3_launch_status();
 }
 
+// `run_k` null: no runs. `score_bias` null: a softmax.
 extern "C" int q3_softcap_attention(const void* q, const void* k_cache, const void* v_cache, const int* block_table,
                                     int table_width, const int* seq_index, const int* positions, float scale, float cap,
-                                    int window, const float* gate, long gate_stride, void* out, int T, int H, int G,
-                                    int dim, int vdim, int page, int v_transposed, const float* sink, int act_dtype,
-                                    hipStream_t stream) {
+                                    int window, const float* gate, long gate_stride, int gate_wide, void* out, int T,
+                                    int H, int G, int dim, int vdim, int page, int v_transposed, const float* sink,
+                                    const void* run_k, const void* run_v, const int* run_table, int run_width, int pool,
+                                    const float* score_bias, int act_dtype, hipStream_t stream) {
   if (T <= 0 || H <= 0 || G <= 0 || H % G || dim <= 0 || vdim <= 0 || page <= 0 || table_width <= 0 || window < 0 ||
       H > 65535)
     return Q3_ERR_BAD_ARGUMENT;
+  if (run_k && (!run_v || !run_table || run_width <= 0 || pool <= 0 || window <= 0 || !v_transposed))
+    return Q3_ERR_BAD_ARGUMENT;
+  if (score_bias && (sink || run_k)) return Q3_ERR_BAD_ARGUMENT;
   if (dim > Q3_CAP_DIM_MOST || vdim > 64 * Q3_CAP_VSLICES) return Q3_ERR_UNSUPPORTED;
+  const RunPlaces runs{const_cast<void*>(run_k), const_cast<void*>(run_v), run_table, run_width, pool};
   Q3_DISPATCH_DTYPE(act_dtype, TA,
                     hipLaunchKernelGGL(softcap_attention_kernel<TA>, dim3(T, H), dim3(64), 0, stream, (const TA*)q,
                                        (const TA*)k_cache, (const TA*)v_cache, block_table, table_width, seq_index,
-                                       positions, scale, cap, window, gate, gate_stride, (TA*)out, H, G, dim, vdim,
-                                       page, v_transposed, sink));
+                                       positions, scale, cap, window, gate, gate_stride, gate_wide, (TA*)out, H, G, dim,
+                                       vdim, page, v_transposed, sink, runs, score_bias));
   return q3_launch_status();
 }

@@ -55,6 +55,10 @@ __all__ = [
     "headnorm_prepare",
     "channel_delta",
     "softcap_attention",
+    "turn_prepare",
+    "mlstm_scan",
+    "mlstm_state_numbers",
+    "soft_cap",
     "scaled_sum",
     "linear",
     "linear_plain",
@@ -1153,6 +1157,124 @@ def headnorm_prepare(rows, heads, kv_heads, dim, vdim, q_weight, k_weight, eps, 
     return q
 
 
+def _runs_args(runs, kv_heads, page, dim, vdim, dtype):
+    """The arguments of a kernel that sees runs of tokens beside tokens: `runs` = (keys (pages, G, page,
+    dim), values (pages, G, vdim, page), int32 block table (B, W), tokens per run), or None."""
+    if runs is None:
+        return None, None, None, 0, 0
+    k, v, table, pool = runs
+    _dev(k, v, table)
+    _need(k.dim() == 4 and k.shape[1:] == (kv_heads, page, dim) and v.dim() == 4 and v.shape[1:] == (kv_heads, vdim, page)
+          and k.shape[0] == v.shape[0] and k.dtype == dtype and v.dtype == dtype, "the runs' caches are shaped like the tokens'")
+    _need(table.dtype == torch.int32 and table.dim() == 2 and int(pool) > 0, "runs come with an int32 block table and a length")
+    return _ptr(k), _ptr(v), _ptr(table), table.shape[1], int(pool)
+
+
+def turn_prepare(rows, bias, heads, kv_heads, dim, vdim, inv_freq, factor, positions, seq_index, out_dtype, block_table,
+                 k_cache, v_cache, values_are_keys=False, runs=None, cu_seqlens_q=None, kv_lens=None, max_q_len=0):
+    """Queries, keys and values of a step from the float32 rows of their joint product, without norms.
+
+    rows float32 (T, n) laid out [q: heads dim | k: kv_heads dim | v: kv_heads vdim | ...], rows possibly
+    apart; bias float32 over q, k and v is added (None: none). With `values_are_keys` there is no v: a
+    token's value is its key before it turns (dim == vdim). The first 2 len(inv_freq) numbers of every
+    head of q and k turn by position * inv_freq[i], i and i + len(inv_freq) together, cos and sin
+    multiplied by `factor`. Returns q (T, heads, dim) of `out_dtype`; keys (pages, kv_heads, page, dim)
+    and values (pages, kv_heads, vdim, page) receive the tokens at their positions.
+
+    `runs` (see `_runs_args`): every run of tokens that this step completes also leaves the means of its
+    keys and values, as the cache holds them; `cu_seqlens_q`, `kv_lens` and `max_q_len` then say what the
+    step brings. A step of single tokens does it in the same kernel."""
+    _dev(bias, inv_freq, positions, seq_index, block_table, k_cache, v_cache)
+    _need(rows.is_cuda and rows.dim() == 2 and rows.dtype == torch.float32 and rows.stride(1) == 1, "rows must be float32 (T, n)")
+    T = rows.shape[0]
+    own_values = 0 if values_are_keys else kv_heads * vdim
+    n = heads * dim + kv_heads * dim + own_values
+    _need(kv_heads > 0 and heads % kv_heads == 0 and rows.shape[1] >= n, "rows hold q, k and v; kv_heads divides heads")
+    _need(not values_are_keys or dim == vdim, "values that are keys have their size")
+    if bias is not None:
+        _f32(bias, (n,), "bias")
+    half = 0
+    if inv_freq is not None:
+        half = inv_freq.shape[0]
+        _f32(inv_freq, (half,), "inv_freq")
+    _need(2 * half <= dim and half <= 256 and out_dtype in _DT, "the rotation fits the head and 512 numbers")
+    _need(positions.dtype == torch.int32 and positions.shape == (T,) and seq_index.dtype == torch.int32
+          and seq_index.shape == (T,), "positions and seq_index must be int32 (T,)")
+    _need(block_table.dtype == torch.int32 and block_table.dim() == 2 and k_cache.dim() == 4, "an int32 block table (B, W)")
+    page = k_cache.shape[2]
+    _need(k_cache.shape[1:] == (kv_heads, page, dim) and v_cache.dim() == 4 and v_cache.shape[1:] == (kv_heads, vdim, page)
+          and k_cache.dtype == out_dtype and v_cache.dtype == out_dtype,
+          "keys (pages, kv_heads, page, dim) and values (pages, kv_heads, vdim, page) of out_dtype")
+    run_args = _runs_args(runs, kv_heads, page, dim, vdim, out_dtype)
+    single = False
+    if runs is not None:
+        _dev(cu_seqlens_q, kv_lens)
+        B = kv_lens.shape[0]
+        _need(kv_lens.dtype == torch.int32 and cu_seqlens_q.dtype == torch.int32 and cu_seqlens_q.shape == (B + 1,)
+              and max_q_len > 0 and block_table.shape[0] >= B and runs[2].shape[0] >= B,
+              "runs need int32 cu_seqlens_q (B + 1,), kv_lens (B,), block tables of B rows and max_q_len")
+        single = max_q_len == 1
+    q = torch.empty((T, heads, dim), dtype=out_dtype, device=rows.device)
+    if T:
+        lib = library("softcap")
+        _check(lib.q3_turn_prepare(
+            _ptr(rows), ctypes.c_long(rows.stride(0)), _ptr(bias), _ptr(inv_freq), half, ctypes.c_float(factor),
+            _ptr(positions), _ptr(seq_index), _ptr(block_table), block_table.shape[1], _ptr(k_cache), _ptr(v_cache), page,
+            _ptr(q), T, heads, kv_heads, dim, vdim, 1 if values_are_keys else 0,
+            *(run_args if single else (None, None, None, 0, 0)), _DT[out_dtype], _stream()), "turn_prepare")
+        if runs is not None and not single:
+            _check(lib.q3_pool_runs(
+                _ptr(k_cache), _ptr(v_cache), _ptr(block_table), block_table.shape[1], _ptr(cu_seqlens_q), _ptr(kv_lens),
+                *run_args, B, int(max_q_len), kv_heads, dim, vdim, page, _DT[out_dtype], _stream()), "pool_runs")
+    return q
+
+
+def mlstm_state_numbers(heads, dim, vdim):
+    """Float32 numbers of one request's matrix memory: per head S (dim, vdim), and for every 64 columns of it
+    copies of the vector n (dim) and of the maximum m."""
+    return heads * dim * vdim + heads * (-(-vdim // 64)) * (dim + 1)
+
+
+def mlstm_scan(rows, heads, dim, vdim, gate_cap, i_bias, f_bias, norm_weight, eps, denominator_eps, state, slots,
+               cu_seqlens_q, out_dtype, max_q_len=1):
+    """The matrix memory of mLSTM over a packed step, float32.
+
+    rows float32 (T, n), rows possibly apart, laid out [q: heads dim | k: heads dim | v: heads vdim | gate:
+    heads vdim | z_i: heads | z_f: heads]; i_bias and f_bias float32 (heads,). q is multiplied by
+    dim^(-1/2); i = cap tanh((z_i + b_i) / cap), f = logsigmoid(cap tanh((z_f + b_f) / cap)) with cap =
+    `gate_cap`; per head, with m' = max(f + m, i),
+
+        S <- exp(f + m - m') S + exp(i - m') k v^T;   n <- exp(f + m - m') n + exp(i - m') k;
+        o = S^T q / (max(|n . q|, exp(-m')) + denominator_eps);
+
+    o is divided by the root mean square of the head's vdim numbers (`eps` inside the root), multiplied by
+    `norm_weight` (heads vdim) and by sigmoid(gate). state float32 (slots, `mlstm_state_numbers`): S, n and
+    m, zeros for a fresh sequence, continued and brought up to date. Returns (T, heads vdim) of `out_dtype`.
+    `max_q_len`: the rows of the step's longest sequence; from `CHUNKED_FROM` on the sequences are worked
+    through in chunks of 64 rows, all chunks at once, instead of row by row."""
+    stride = _rows_view(rows, "rows")
+    T = rows.shape[0]
+    _need(rows.dtype == torch.float32 and rows.shape[1] >= 2 * heads * (dim + vdim + 1),
+          "rows must be float32 (T, 2 heads (dim + vdim + 1)) or wider")
+    _need(0 < dim <= 512 and vdim > 0 and heads > 0 and gate_cap > 0, "keys of up to 512 numbers and a positive cap")
+    for t, n, what in ((i_bias, heads, "i_bias"), (f_bias, heads, "f_bias"), (norm_weight, heads * vdim, "norm_weight")):
+        _f32(t, (n,), what)
+    _need(out_dtype in _DT, "out_dtype must be bfloat16 or float32")
+    B = _sequences(slots, cu_seqlens_q, state, mlstm_state_numbers(heads, dim, vdim), "mlstm_scan")
+    out = torch.empty((T, heads * vdim), dtype=out_dtype, device=rows.device)
+    if T:
+        lib = library("mlstm")
+        chunked = 1 if max_q_len >= CHUNKED_FROM else 0
+        lib.q3_mlstm_workspace.restype = ctypes.c_long
+        work = torch.empty(lib.q3_mlstm_workspace(T, B, heads, dim, vdim, chunked), dtype=torch.uint8, device=rows.device)
+        _check(lib.q3_mlstm_scan(
+            _ptr(rows), ctypes.c_long(stride), _ptr(i_bias), _ptr(f_bias), ctypes.c_float(gate_cap), _ptr(norm_weight),
+            ctypes.c_float(eps), ctypes.c_float(denominator_eps), _ptr(state), ctypes.c_long(state.stride(0)), _ptr(slots),
+            _ptr(cu_seqlens_q), _ptr(out), _ptr(work), T, B, int(max_q_len), heads, dim, vdim, chunked, _DT[out_dtype],
+            _stream()), "mlstm_scan")
+    return out
+
+
 def channel_delta(conv, b_logits, a_logits, gate, dt_bias, a_log, norm_weight, eps, unit_eps, state, slots, cu_seqlens_q,
                   heads, kv_heads, dim, vdim, out_dtype):
     """The gated delta rule with a decay per head and key channel over a packed step, float32.
@@ -1196,16 +1318,20 @@ def channel_delta(conv, b_logits, a_logits, gate, dt_bias, a_log, norm_weight, e
 
 def softcap_attention(q, k_cache, v_cache, block_table, cu_seqlens_q, kv_lens, seq_index, positions, max_q_len,
                       max_kv_len, scale, softcap, window=0, gate=None, values_transposed=False, min_q_len=1,
-                      max_kv_len_of_many=None, sink=None):
+                      max_kv_len_of_many=None, sink=None, runs=None, sigmoid_bias=None):
     """Causal softmax attention over a paged cache whose keys and values differ in size.
 
     q (T, heads, dim); keys (pages, kv_heads, page, dim), values (pages, kv_heads, page, vdim); the
     token at row t of sequence seq_index[t] sits at positions[t] and sees the keys at positions
     j <= positions[t] (with `window` > 0 only the last `window` of them). score = (q . k) scale, then
     softcap * tanh(score / softcap) if softcap > 0; softmax in float32. `gate` float32 (T, heads),
-    rows possibly apart: head h's result is multiplied by sigmoid(gate[t, h]). `sink` float32 (heads,):
-    head h's softmax has exp(sink[h]) as one more term of its denominator, a key that is always seen, is
-    not scaled and has no value. Returns (T, heads vdim).
+    rows possibly apart: head h's result is multiplied by sigmoid(gate[t, h]); or (T, heads vdim), a gate
+    per column. `sink` float32 (heads,): head h's softmax has exp(sink[h]) as one more term of its
+    denominator, a key that is always seen, is not scaled and has no value. Returns (T, heads vdim).
+
+    `runs` (see `_runs_args`; with a window and transposed values): the token at position i also sees one
+    key and value per run of tokens that ends at i - window or before, in the same softmax.
+    `sigmoid_bias` float32 (heads,): no softmax; a key counts with sigmoid(score + sigmoid_bias[h]).
 
     With `values_transposed` the values are (pages, kv_heads, vdim, page), and bfloat16 with equal key
     and value sizes of 64 or 128 then runs on the matrix cores, through the kernels of
@@ -1229,14 +1355,24 @@ def softcap_attention(q, k_cache, v_cache, block_table, cu_seqlens_q, kv_lens, s
     stride = 0
     if gate is not None:
         stride = _rows_view(gate, "gate")
-        _need(gate.shape == (T, H) and gate.dtype == torch.float32, "gate must be float32 (T, heads)")
+        _need(gate.shape in ((T, H), (T, H * vdim)) and gate.dtype == torch.float32,
+              "gate must be float32 (T, heads) or (T, heads vdim)")
+    wide = 1 if gate is not None and gate.shape[1] != H else 0
+    run_args = _runs_args(runs, G, page, dim, vdim, q.dtype)
+    _need(runs is None or (window > 0 and values_transposed and max_kv_len // runs[3] <= runs[2].shape[1] * page),
+          "runs stand behind a window, with transposed values and a table that covers them")
+    if sigmoid_bias is not None:
+        _f32(sigmoid_bias, (H,), "sigmoid_bias")
+        _dev(sigmoid_bias)
+        _need(sink is None and runs is None and softcap == 0 and window == 0,
+              "sigmoid weights take no sink, no runs, no cap and no window")
     if T and values_transposed and dim == vdim and q.dtype == torch.bfloat16 \
             and library("attention").q3_paged_attention_fast_path(H, G, dim, page, _DT[q.dtype]):
         out = paged_attention(q, H, k_cache, v_cache, block_table, cu_seqlens_q, kv_lens, max_q_len, max_kv_len, scale,
                               window=window, min_q_len=min_q_len, max_kv_len_of_many=max_kv_len_of_many, softcap=softcap,
-                              sink=sink)
+                              sink=sink, runs=runs, sigmoid_bias=sigmoid_bias)
         if gate is not None:
-            _check(library("softcap").q3_gate_heads(_ptr(out), _ptr(gate), ctypes.c_long(stride), T, H, vdim,
+            _check(library("softcap").q3_gate_heads(_ptr(out), _ptr(gate), ctypes.c_long(stride), wide, T, H, vdim,
                                                     _DT[q.dtype], _stream()), "gate_heads")
         return out
     out = torch.empty((T, H * vdim), dtype=q.dtype, device=q.device)
@@ -1244,9 +1380,19 @@ def softcap_attention(q, k_cache, v_cache, block_table, cu_seqlens_q, kv_lens, s
         _check(library("softcap").q3_softcap_attention(
             _ptr(q), _ptr(k_cache), _ptr(v_cache), _ptr(block_table), block_table.shape[1], _ptr(seq_index),
             _ptr(positions), ctypes.c_float(scale), ctypes.c_float(softcap), int(window), _ptr(gate),
-            ctypes.c_long(stride), _ptr(out), T, H, G, dim, vdim, page, 1 if values_transposed else 0, _ptr(sink),
-            _DT[q.dtype], _stream()), "softcap_attention")
+            ctypes.c_long(stride), wide, _ptr(out), T, H, G, dim, vdim, page, 1 if values_transposed else 0, _ptr(sink),
+            *run_args, _ptr(sigmoid_bias), _DT[q.dtype], _stream()), "softcap_attention")
     return out
+
+
+def soft_cap(x, cap):
+    """cap * tanh(x / cap), elementwise in float32, in place; returns x."""
+    _dev(x)
+    _need(x.dtype == torch.float32 and cap > 0, "x must be float32, the cap positive")
+    if x.numel():
+        _check(library("elementwise").q3_soft_cap(_ptr(x), ctypes.c_long(x.numel()), ctypes.c_float(cap), _stream()),
+               "soft_cap")
+    return x
 
 
 def scaled_sum(a, alpha, b, beta):
@@ -1346,11 +1492,14 @@ def qk_norm_rope_store(qkv, num_q_heads, num_kv_heads, head_dim, positions, seq_
 
 def paged_attention(q, num_q_heads, k_cache, v_cache, block_table, cu_seqlens_q, kv_lens,
                     max_q_len, max_kv_len, scale, window=0, out=None, min_q_len=1, max_kv_len_of_many=None, softcap=0.0,
-                    sink=None):
+                    sink=None, runs=None, sigmoid_bias=None):
     """Causal softmax attention of packed query rows over paged keys and values.
     `softcap` > 0: a score s enters the softmax as softcap * tanh(s * scale / softcap); that form
     exists for the sizes the matrix cores take (a second build of the same kernels) and no other.
     `sink` float32 (Hq,): exp(sink[h]) joins the denominator of head h's softmax (no key, no value).
+    `runs` (keys, values, block table, tokens per run; see `_runs_args`) with a window: a row at position p
+    also sees one key and value per run that ends at p - window or before. `sigmoid_bias` float32 (Hq,): no
+    softmax, a key counts with sigmoid(s * scale + sigmoid_bias[h]). These two are builds of their own as well.
 
     q is (T, Hq, D) seen through a row stride (a view of the qkv buffer is
     fine). Keys are cached as (pages, Hkv, page, D), values as
@@ -1394,22 +1543,41 @@ def paged_attention(q, num_q_heads, k_cache, v_cache, block_table, cu_seqlens_q,
         out = torch.empty((T, Hq * D), dtype=q.dtype, device=q.device)
     _need(out.shape == (T, Hq * D) and out.dtype == q.dtype, "out must be (T, Hq D)")
     if T and B:
-        lib = library("attention_capped" if softcap > 0 else "attention")
-        if softcap > 0:
+        kinds = [kind for kind, on in (("capped", softcap > 0), ("pooled", runs is not None),
+                                       ("sigmoid", sigmoid_bias is not None)) if on]
+        _need(len(kinds) <= 1, "capped scores, runs and sigmoid weights exclude each other")
+        lib = library("_".join(["attention"] + kinds))
+        if kinds:
             _need(lib.q3_paged_attention_fast_path(Hq, Hkv, D, page, _DT[q.dtype]) and q.stride(0) % 8 == 0,
-                  "capped scores need bfloat16, a head size of 64 or 128 and pages of a power of two from 16")
+                  "capped scores, runs and sigmoid weights need bfloat16, a head size of 64 or 128 and pages of a power "
+                  "of two from 16")
+        if softcap > 0:
             lib.q3_set_score_cap.restype = None
             lib.q3_set_score_cap(ctypes.c_float(softcap))
+        visible = int(max_kv_len)                      # keys that a row may see, for how they are shared out
+        longest = visible if max_kv_len_of_many is None else int(max_kv_len_of_many)
+        if runs is not None:
+            _need(window > 0 and runs[2].shape[0] >= B and max_kv_len // runs[3] <= runs[2].shape[1] * page,
+                  "runs stand behind a window, with a block table that covers them")
+            k_ptr, v_ptr, t_ptr, width, pool = _runs_args(runs, Hkv, page, D, D, q.dtype)
+            lib.q3_set_runs.restype = None
+            lib.q3_set_runs(k_ptr, v_ptr, t_ptr, width, runs[0].shape[0], pool)
+            visible = min(visible, window + visible // pool)
+            longest = min(longest, window + longest // pool)
+        if sigmoid_bias is not None:
+            _need(sink is None and window == 0, "sigmoid weights take no sink and no window")
+            _f32(sigmoid_bias, (Hq,), "sigmoid_bias")
+            lib.q3_set_sigmoid_bias.restype = None
+            lib.q3_set_sigmoid_bias(_ptr(sigmoid_bias))
         splits, workspace, prompt_splits, prompt_workspace = 1, None, 1, None
         if lib.q3_paged_attention_fast_path(Hq, Hkv, D, page, _DT[q.dtype]):
             if min_q_len * (Hq // Hkv) <= 16:
-                splits = _splits(B, Hkv, max_kv_len)   # few rows per sequence: the keys go over several blocks
+                splits = _splits(B, Hkv, visible)   # few rows per sequence: the keys go over several blocks
                 if splits > 1:
                     lib.q3_paged_attention_workspace.restype = ctypes.c_long
                     n = lib.q3_paged_attention_workspace(B, Hkv, D, splits)
                     workspace = torch.empty((n,), dtype=torch.float32, device=q.device)
             if max_q_len * (Hq // Hkv) > 16:           # few long sequences over many keys: likewise
-                longest = max_kv_len if max_kv_len_of_many is None else max_kv_len_of_many
                 prompt_splits = lib.q3_paged_attention_prompt_splits(T, Hq, Hkv, int(longest))
                 if prompt_splits > 1:
                     prompt_workspace = torch.empty((T * Hq * prompt_splits * (D + 2),), dtype=torch.float32,

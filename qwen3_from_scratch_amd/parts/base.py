@@ -249,30 +249,42 @@ class CacheNeed:
     different widths), all tokens kept (window == 0) or the last `window`. state: a tensor of
     fixed `state_shape` and `state_dtype` per request. A mixer may need neither, either or
     both. Mixers whose needs are equal share page numbers: one block table serves them all.
+
+    runs: tensors that grow by one element per complete run of `run_length` tokens, paged like the
+    others (a page holds page_size elements, so page_size * run_length tokens) with a block table of
+    their own, and never given back while the request lives: what a mixer keeps of tokens that have
+    left its window, say. The mixer finds them as `LayerCacheView.runs` and `run_table`; element r
+    stands for tokens r * run_length .. (r + 1) * run_length - 1.
     """
 
     paged: tuple = ()
     window: int = 0
     state_shape: tuple = ()
     state_dtype: torch.dtype = torch.float32
+    runs: tuple = ()
+    run_length: int = 0
 
     def __post_init__(self):
         object.__setattr__(self, "paged", tuple(self.paged))
+        object.__setattr__(self, "runs", tuple(self.runs))
+        if bool(self.runs) != (self.run_length > 0):
+            raise ValueError("tensors per run come with a positive run_length, and only they do")
         object.__setattr__(self, "state_shape", tuple(self.state_shape))
-        names = [t.name for t in self.paged]
-        if len(set(names)) != len(names):
-            raise ValueError("paged tensors of one mixer need different names, found %r" % (names,))
+        for tensors in (self.paged, self.runs):
+            names = [t.name for t in tensors]
+            if len(set(names)) != len(names):
+                raise ValueError("paged tensors of one mixer need different names, found %r" % (names,))
 
     @property
     def has_state(self):
         return len(self.state_shape) > 0
 
     def bytes_per_token(self, act_dtype):
-        """Bytes that one token adds to one layer's pages."""
-        total = 0
-        for t in self.paged:
-            total += t.numbers_per_token() * torch.empty((), dtype=t.dtype or act_dtype).element_size()
-        return total
+        """Bytes that one token adds to one layer's pages (its share of a run's rounded up)."""
+        def size(tensors):
+            return sum(t.numbers_per_token() * torch.empty((), dtype=t.dtype or act_dtype).element_size() for t in tensors)
+
+        return size(self.paged) + (-(-size(self.runs) // self.run_length) if self.runs else 0)
 
     def bytes_of_state(self):
         if not self.has_state:

@@ -51,7 +51,7 @@ class SwiGLU(Part):
 
     @property
     def takes_unscaled(self):
-        return self.activation == "silu" and self.gate_up is not None and self.gate_up.fuses
+        return self.gate_up is not None and self.gate_up.fuses
 
     def forward(self, x, batch=None, sink=None):
         if self.activation == "silu":

@@ -7,6 +7,19 @@ from .. import ops
 from .base import UnscaledRows
 
 
+def joined_rows(matrices, multiple=16):
+    """Matrices of one inner size as one, below each other, filled up with rows of zeros to a multiple
+    of `multiple` rows: one product for all of them, in a size that every product kernel takes."""
+    rows = sum(m.shape[0] for m in matrices)
+    out = torch.zeros((-(-rows // multiple) * multiple, matrices[0].shape[1]), dtype=matrices[0].dtype,
+                      device=matrices[0].device)
+    at = 0
+    for m in matrices:
+        out[at:at + m.shape[0]].copy_(m)
+        at += m.shape[0]
+    return out
+
+
 class LinearWeight:
     """y = x @ W^T, no bias. W (N, K) is kept row-major for products with many
     rows (the vendor library's) and for float32; when the precision asks for

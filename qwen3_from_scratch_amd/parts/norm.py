@@ -19,22 +19,27 @@ class RMSNorm(Part):
     (src/qwen3_from_scratch/models/norm.py:18-22,51-53). It reads the float32
     residual stream and can fold the pending addition `x += delta` into the
     same pass; the sum, the mean and the products are float32 and the result
-    is rounded once."""
+    is rounded once. `offset`: a constant that the stored weight lacks (1 for a
+    weight stored around zero); the sum is formed in float32 and kept so."""
 
     graph_safe = True
 
-    def __init__(self, prefix, precision, device, size, eps, leaf="weight"):
+    def __init__(self, prefix, precision, device, size, eps, leaf="weight", offset=0.0):
         super().__init__(prefix, precision, device)
         self.size = size
         self.eps = float(eps)
         self.leaf = leaf            # the tensor's name below the prefix; "" if it is the prefix itself
+        self.offset = float(offset)
         self.weight = None
 
     def tensors(self):
-        return {self._name(self.leaf): TensorShape((self.size,), "scale")}
+        return {self._name(self.leaf): TensorShape((self.size,), "scale" if self.offset == 0.0 else "bias")}
 
     def load(self, fetch):
-        self.weight = fetch(self._name(self.leaf))
+        if self.offset == 0.0:
+            self.weight = fetch(self._name(self.leaf))
+        else:
+            self.weight = (fetch(self._name(self.leaf), torch.float32) + self.offset).contiguous()
 
     def forward(self, x, delta=None, rows=None):
         """Normalised rows in the activation dtype. With `delta`, x += delta

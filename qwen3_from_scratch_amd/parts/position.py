@@ -6,6 +6,8 @@ for a rotation table (`rotation_table`) and applies it to queries and keys in
 its own fused kernel. Either hook may be a no-op.
 """
 
+import math
+
 import torch
 
 from .. import ops
@@ -13,16 +15,75 @@ from ..config.registry import register_part
 from .base import Part
 
 
-def rotation_frequencies(dims, base, device):
-    """f_i = base^(-2i / dims), i < dims / 2, formed in double precision on the host and rounded
-    once to float32: what a mixer that carries its rotation among its own parameters hands to its
-    kernels, which form the angle as a float32 product of position and frequency. dims 0: None."""
-    if not dims:
-        return None
+def plain_frequencies(dims, base):
+    """f_i = base^(-2i / dims), i < dims / 2, in double precision."""
+    return [float(base) ** (-2.0 * i / dims) for i in range(dims // 2)]
+
+
+def ramped_frequencies(dims, base, factor, original, fast, slow):
+    """Frequencies blended for contexts longer than the `original` one by the pair's number: with
+    pair(turns) = dims * ln(original / (2 pi turns)) / (2 ln base), lo = max(floor(pair(fast)), 0),
+    hi = min(ceil(pair(slow)), dims - 1) and ramp_i = clamp((i - lo) / max(hi - lo, 0.001), 0, 1),
+    pair i turns by f_i / factor * ramp_i + f_i * (1 - ramp_i). Returns them and the factor on cos
+    and sin, 0.1 ln(factor) + 1."""
+    def pair(turns):
+        return dims * math.log(original / (2.0 * math.pi * turns)) / (2.0 * math.log(base))
+
+    lo, hi = max(math.floor(pair(fast)), 0), min(math.ceil(pair(slow)), dims - 1)
+    blended = []
+    for i, f in enumerate(plain_frequencies(dims, base)):
+        ramp = min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0)
+        blended.append(f / factor * ramp + f * (1.0 - ramp))
+    return blended, 0.1 * math.log(factor) + 1.0
+
+
+def banded_frequencies(dims, base, factor, original, low, high):
+    """Frequencies stretched for contexts longer than the `original` one by their wavelength
+    l = 2 pi / f: kept where l < original / high, divided by `factor` where l > original / low, and
+    between the two (1 - s) f / factor + s f with s = (original / l - low) / (high - low)."""
+    stretched = []
+    for f in plain_frequencies(dims, base):
+        length = 2.0 * math.pi / f
+        if length < original / high:
+            stretched.append(f)
+        elif length > original / low:
+            stretched.append(f / factor)
+        else:
+            share = (original / length - low) / (high - low)
+            stretched.append((1.0 - share) * f / factor + share * f)
+    return stretched
+
+
+def scaled_frequencies(dims, base, scaling=None):
+    """(frequencies in double precision, factor on cos and sin) of a rotation with `scaling`: None;
+    ("ramp", factor, original, fast, slow) for `ramped_frequencies`; or ("bands", factor, original,
+    low, high) for `banded_frequencies`."""
+    if not scaling:
+        return plain_frequencies(dims, base), 1.0
+    kind, numbers = scaling[0], [float(v) for v in scaling[1:]]
+    if kind == "ramp":
+        return ramped_frequencies(dims, base, *numbers)
+    if kind == "bands":
+        return banded_frequencies(dims, base, *numbers), 1.0
+    raise ValueError("a rotation's scaling is 'ramp' or 'bands', not %r" % (kind,))
+
+
+def scaled_rotation(dims, base, device, scaling=None):
+    """What a mixer that carries its rotation among its own parameters hands to its kernels, which
+    form the angle as a float32 product of position and frequency: the frequencies of
+    `scaled_frequencies`, formed in double precision on the host and rounded once to float32 (None for
+    dims 0), and the factor on cos and sin."""
     if dims % 2 or dims < 0:
         raise ValueError("a rotation turns an even number of numbers, not %d" % dims)
-    freqs = [float(base) ** (-2.0 * i / dims) for i in range(dims // 2)]
-    return torch.tensor(freqs, dtype=torch.float64).to(torch.float32).to(device)
+    if not dims:
+        return None, 1.0
+    freqs, factor = scaled_frequencies(dims, base, scaling)
+    return torch.tensor(freqs, dtype=torch.float64).to(torch.float32).to(device), factor
+
+
+def rotation_frequencies(dims, base, device):
+    """The frequencies of an unscaled rotation, f_i = base^(-2i / dims) (see `scaled_rotation`)."""
+    return scaled_rotation(dims, base, device)[0]
 
 
 @register_part("position", "none")
@@ -75,12 +136,8 @@ class RotaryPairs(NoPosition):
     kernels, so there is no table and no last position.
 
     `scaling` = (factor, original, fast, slow) blends the frequencies for contexts longer than
-    the `original` one: with pair(turns) = dims * ln(original / (2 pi turns)) / (2 ln base),
-    lo = max(floor(pair(fast)), 0), hi = min(ceil(pair(slow)), dims - 1) and
-    ramp_i = clamp((i - lo) / max(hi - lo, 0.001), 0, 1), pair i turns by
-    f_i / factor * ramp_i + f_i * (1 - ramp_i), and cos and sin are multiplied by
-    0.1 ln(factor) + 1. The frequencies are formed in double precision on the host and rounded
-    once."""
+    the `original` one (`ramped_frequencies`). The frequencies are formed in double precision on
+    the host and rounded once."""
 
     max_positions = None
 
@@ -94,23 +151,7 @@ class RotaryPairs(NoPosition):
         self.factor = 1.0
 
     def host_frequencies(self):
-        import math
-
-        dims, base = self.dims, self.base
-        freqs = [base ** (-2.0 * i / dims) for i in range(dims // 2)]
-        if self.scaling is None:
-            return freqs, 1.0
-        factor, original, fast, slow = self.scaling
-
-        def pair(turns):
-            return dims * math.log(original / (2.0 * math.pi * turns)) / (2.0 * math.log(base))
-
-        lo, hi = max(math.floor(pair(fast)), 0), min(math.ceil(pair(slow)), dims - 1)
-        blended = []
-        for i, f in enumerate(freqs):
-            ramp = min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0)
-            blended.append(f / factor * ramp + f * (1.0 - ramp))
-        return blended, 0.1 * math.log(factor) + 1.0
+        return scaled_frequencies(self.dims, self.base, ("ramp",) + self.scaling if self.scaling else None)
 
     def load(self, fetch):
         freqs, self.factor = self.host_frequencies()

@@ -606,7 +606,7 @@ def channel_delta(conv, b_logits, a_logits, gate, dt_bias, a_log, norm_weight, e
 
 def softcap_attention(q, k_cache, v_cache, block_table, cu_seqlens_q, kv_lens, seq_index, positions, max_q_len,
                       max_kv_len, scale, softcap, window=0, gate=None, values_transposed=False, min_q_len=1,
-                      max_kv_len_of_many=None, sink=None):
+                      max_kv_len_of_many=None, sink=None, runs=None, sigmoid_bias=None):
     T, H, dim = q.shape
     if values_transposed:
         v_cache = v_cache.transpose(2, 3)
@@ -627,8 +627,21 @@ def softcap_attention(q, k_cache, v_cache, block_table, cu_seqlens_q, kv_lens, s
         hidden = kpos > qpos
         if window > 0:
             hidden = hidden | (qpos - kpos >= window)
+        if runs is not None and L // runs[3]:              # the runs' means stand before the tokens
+            rk, rv, table, pool = runs
+            many = L // pool
+            at = table[b, :-(-many // page)].long()
+            RK = rk[at].float().permute(1, 0, 2, 3).reshape(G, -1, dim)[:, :many]
+            RV = rv[at].float().permute(1, 0, 3, 2).reshape(G, -1, vdim)[:, :many]
+            K, V = torch.cat((RK, K), dim=1), torch.cat((RV, V), dim=1)
+            ends = (torch.arange(many, device=q.device)[None, :] + 1) * pool - 1
+            hidden = torch.cat((ends > qpos - window, hidden), dim=1)
         for h in range(H):
             s = (q[q0:q1, h].float() @ K[h // (H // G)].T) * scale
+            if sigmoid_bias is not None:
+                w = torch.sigmoid(s + sigmoid_bias[h].float()).masked_fill(hidden, 0.0)
+                res[q0:q1, h] = w @ V[h // (H // G)].nan_to_num(0.0)
+                continue
             if softcap > 0:
                 s = softcap * torch.tanh(s / softcap)
             s = s.masked_fill(hidden, float("-inf"))
@@ -638,8 +651,84 @@ def softcap_attention(q, k_cache, v_cache, block_table, cu_seqlens_q, kv_lens, s
             else:
                 res[q0:q1, h] = torch.softmax(s, dim=-1) @ V[h // (H // G)]
     if gate is not None:
-        res = res * torch.sigmoid(gate.float())[:, :, None]
+        res = res * torch.sigmoid(gate.float()).reshape(T, H, -1)
     return res.reshape(T, H * vdim).to(q.dtype)
+
+
+def turn_prepare(rows, bias, heads, kv_heads, dim, vdim, inv_freq, factor, positions, seq_index, out_dtype, block_table,
+                 k_cache, v_cache, values_are_keys=False, runs=None, cu_seqlens_q=None, kv_lens=None, max_q_len=0):
+    T = rows.shape[0]
+    nq, nk = heads * dim, kv_heads * dim
+    n = nq + nk + (0 if values_are_keys else kv_heads * vdim)
+    z = rows[:, :n].float()
+    if bias is not None:
+        z = z + bias.float()
+    q, k = z[:, :nq].reshape(T, heads, dim), z[:, nq:nq + nk].reshape(T, kv_heads, dim)
+    v = k if values_are_keys else z[:, nq + nk:].reshape(T, kv_heads, vdim)
+
+    def turn(x):
+        if inv_freq is None:
+            return x
+        half = inv_freq.shape[0]
+        turned = _turn(x, positions, inv_freq, False)
+        turned[..., :2 * half] *= factor
+        return turned
+
+    page, pos = k_cache.shape[2], positions.long()
+    pages = block_table[seq_index.long(), pos // page].long()
+    k_cache[pages, :, pos % page] = turn(k).to(k_cache.dtype)
+    v_cache[pages, :, :, pos % page] = v.to(v_cache.dtype)
+    if runs is not None:
+        rk, rv, table, pool = runs
+        cu, kvl = cu_seqlens_q.tolist(), kv_lens.tolist()
+        for b, L in enumerate(kvl):
+            for r in range((L - (cu[b + 1] - cu[b])) // pool, L // pool):
+                at = torch.arange(r * pool, (r + 1) * pool, device=rows.device)
+                of = block_table[b, at // page].long()
+                place = (table[b, r // page].long(), slice(None), r % page)
+                rk[place] = k_cache[of, :, at % page].float().mean(dim=0).to(rk.dtype)
+                rv[table[b, r // page].long(), :, :, r % page] = v_cache[of, :, :, at % page].float().mean(dim=0).to(rv.dtype)
+    return turn(q).to(out_dtype).contiguous()
+
+
+def mlstm_state_numbers(heads, dim, vdim):
+    return heads * dim * vdim + heads * (-(-vdim // 64)) * (dim + 1)
+
+
+def mlstm_scan(rows, heads, dim, vdim, gate_cap, i_bias, f_bias, norm_weight, eps, denominator_eps, state, slots,
+               cu_seqlens_q, out_dtype, max_q_len=1):
+    T, hd, hv, tiles = rows.shape[0], heads * dim, heads * vdim, -(-vdim // 64)
+    z = rows.float()
+    q = z[:, :hd].reshape(T, heads, dim) * dim ** -0.5
+    k = z[:, hd:2 * hd].reshape(T, heads, dim)
+    v = z[:, 2 * hd:2 * hd + hv].reshape(T, heads, vdim)
+    gate = z[:, 2 * hd + hv:2 * hd + 2 * hv]
+    base = 2 * hd + 2 * hv
+    gi = gate_cap * torch.tanh((z[:, base:base + heads] + i_bias) / gate_cap)
+    gf = torch.nn.functional.logsigmoid(gate_cap * torch.tanh((z[:, base + heads:base + 2 * heads] + f_bias) / gate_cap))
+    o = torch.empty((T, heads, vdim), dtype=torch.float32, device=rows.device)
+    for first, last, slot in _sequences(cu_seqlens_q, slots):
+        if last == first:
+            continue
+        S = state[slot, :hd * vdim].reshape(heads, dim, vdim).clone()
+        n = state[slot, hd * vdim:hd * vdim + heads * tiles * dim].reshape(heads, tiles, dim)[:, 0].clone()
+        m = state[slot, hd * vdim + heads * tiles * dim:].reshape(heads, tiles)[:, 0].clone()
+        for t in range(first, last):
+            new = torch.maximum(gf[t] + m, gi[t])
+            keep, enter = torch.exp(gf[t] + m - new), torch.exp(gi[t] - new)
+            S = keep[:, None, None] * S + enter[:, None, None] * k[t][:, :, None] * v[t][:, None, :]
+            n = keep[:, None] * n + enter[:, None] * k[t]
+            m = new
+            below = torch.maximum((n * q[t]).sum(dim=-1).abs(), torch.exp(-m)) + denominator_eps
+            o[t] = torch.einsum("hdv,hd->hv", S, q[t]) / below[:, None]
+        state[slot] = torch.cat((S.reshape(-1), n[:, None].expand(heads, tiles, dim).reshape(-1),
+                                 m[:, None].expand(heads, tiles).reshape(-1)))
+    o = o * torch.rsqrt((o * o).mean(dim=-1, keepdim=True) + eps)
+    return (o.reshape(T, hv) * norm_weight * torch.sigmoid(gate)).to(out_dtype)
+
+
+def soft_cap(x, cap):
+    return x.copy_(cap * torch.tanh(x / cap))
 
 
 def scaled_sum(a, alpha, b, beta):
@@ -650,4 +739,5 @@ ALL = ("gated_act", "GATE_KINDS", "layernorm_addend", "moe_glu_experts", "glu_cl
        "paged_attention", "decode_attention_takes", "linear", "linear_swiglu", "tile_weight", "sample",
        "rmsnorm_addend", "gelu", "GELU_KINDS", "latent_prepare", "headwise_linear", "rotate_heads", "latent_attention",
        "moe_route", "moe_experts", "embed_streams", "hyper_norm", "causal_conv", "mamba2_scan", "gated_rmsnorm",
-       "block_gates", "rglru_scan", "retention_scan", "softcap_prepare", "softcap_attention", "scaled_sum")
+       "block_gates", "rglru_scan", "retention_scan", "softcap_prepare", "softcap_attention", "scaled_sum",
+       "turn_prepare", "mlstm_scan", "mlstm_state_numbers", "soft_cap")
