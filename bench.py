@@ -2,7 +2,7 @@
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch B] [--layers L]
                     [--shape 8b|14b|32b|0.6b] [--prompt P] [--context C]
-                    [--workload decode|continuous|served|prefix|products|kodisun|surasun|dufinex|fidevik]
+                    [--workload decode|continuous|served|prefix|products|kodisun|surasun|dufinex|fidevik|zedotar]
 
 Random bfloat16 weights, uniform-random prompts of 2,048 tokens, greedy decoding
 through the engine's own step loop (scheduler, step function, sampling). A
@@ -825,6 +825,147 @@ def fidevik(args, sync):
     return 0
 
 
+ZEDOTAR_SHAPES = {
+    # (width, feed-forward inner size, window, tokens a run, mixers)
+    "base": (2048, 6144, 512, 16, ("attention", "attention_2", "mlstm", "mlstm")),
+    "wide": (4096, 12288, 1024, 16, ("mlstm", "attention", "attention_2")),
+}
+
+
+def zedotar_layers(W, ff, window, pool, kinds):
+    """Layers of real proportions: both attentions in heads of 128, four query heads a key head, half of
+    each head turned; the matrix memory in heads of 128 with values of 256, as the retention it stands
+    beside."""
+    half = {"dims": 64, "base": 500000.0}
+    mixers = {
+        "attention": {"heads": W // 128, "kv_heads": W // 512, "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+                      "mask": {"size": window, "pool": pool}, "rot": half},
+        "attention_2": {"heads": W // 128, "kv_heads": W // 512, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "conv": 4,
+                        "rot": half},
+        "mlstm": {"heads": W // 256, "dim": 128, "vdim": 256, "gate_cap": 15.0},
+    }
+    return [{"type": kind, "mixer": mixers[kind], "mlp": {"kind": "dense", "ff": ff}} for kind in kinds]
+
+
+def zedotar(args, sync):
+    """Prefill and decode throughput of the Zedotar design at sizes that resemble a real model's layers
+    (random weights, a few layers, a vocabulary of 32,768), beside the Surasun design, the closest of the
+    others (attention with a gate through the same kernels, recurrences with a matrix per head), at the
+    same width, layer count and feed-forward inner size: a layer of attention beside retention (heads as
+    the matrix memory's) where this one has attention, and Mamba-2 where it has the matrix memory. Both
+    go through the engine's own loop: one prompt in one step, then greedy decoding at batch 8 and 64
+    behind prompts of 1,024 tokens. `frac` prices a prompt's multiply-adds (the products, the recurrences'
+    updates and reads, the attentions' visible pairs) against the bfloat16 matrix peak, and a decode
+    step's bytes (the weights once, the states read and written, the visible keys and values) against
+    the HBM peak."""
+    import torch
+
+    from qwen3_from_scratch_amd.config.surasun_config import SurasunConfig
+    from qwen3_from_scratch_amd.config.zedotar_config import ZedotarConfig
+    from qwen3_from_scratch_amd.engine import SyncEngine, random_model
+
+    vocab, prompt_len, decode_prompt, context = 32768, args.prefill_tokens, 1024, 4096
+    results = {}
+    for shape in ([args.zedotar_shape] if args.zedotar_shape != "all" else sorted(ZEDOTAR_SHAPES)):
+        W, ff, window, pool, kinds = ZEDOTAR_SHAPES[shape]
+        if args.layers:
+            kinds = (kinds * args.layers)[:args.layers]
+        listed = zedotar_layers(W, ff, window, pool, kinds)
+        new = ZedotarConfig.from_dict({"architecture": "Zedotar", "vocab": vocab, "width": W, "norm": {"eps": 1e-5},
+                                       "logit_softcap": 30.0, "layers": listed})
+        other = SurasunConfig.from_dict({"architecture": "Surasun", "vocab": vocab, "width": W, "norm": {"eps": 1e-5},
+                                         "residual_mult": 1.0,
+                                         "layers": surasun_layers(W, ff, [("mamba2" if k == "mlstm" else "parallel", True)
+                                                                          for k in kinds])})
+
+        def visible(i):
+            """Keys that position i of a windowed layer sees: its tokens and the runs behind them."""
+            return min(i + 1, window) + max(0, i - window + 1) // pool
+
+        for name, config in (("zedotar", new), ("surasun", other)):
+            if args.zedotar_only and name != args.zedotar_only:
+                continue
+            model = random_model(config, dtype=args.dtype, device="cuda:0", seed=0, std=0.02)
+            gen = torch.Generator().manual_seed(1)
+            entry = {}
+            matrices = sum(t[0] * t[1] for key, t in model.tensors().items()
+                           if len(t) == 2 and key not in ("embed", "head") and ".hc" not in key and not key.endswith("conv"))
+            # per token: multiply-adds of the recurrences, floats of state; over a prompt: pairs times their numbers;
+            # of a decode step at a context: numbers of keys and values that are seen
+            scans = state = prompt_pairs = 0
+            seen = decode_prompt + args.warmup + args.steps // 2
+            read = 0
+            every = prompt_len * (prompt_len + 1) // 2
+            for layer in config.to_dict()["layers"]:
+                m, kind = layer["mixer"], layer["type"]
+                if kind == "mlstm":
+                    scans += 3 * m["heads"] * m["dim"] * m["vdim"]
+                    state += m["heads"] * m["dim"] * (m["vdim"] + 1)
+                elif kind == "mamba2":
+                    scans += 3 * m["heads"] * m["state"] * m["vdim"]
+                    state += m["heads"] * m["state"] * m["vdim"] + 3 * (m["heads"] * m["vdim"] + 2 * m["state"])
+                elif kind == "parallel":
+                    scans += 3 * m["right"]["heads"] * m["right"]["dim"] * m["right"]["vdim"]
+                    state += m["right"]["heads"] * m["right"]["dim"] * m["right"]["vdim"]
+                    prompt_pairs += every * m["left"]["heads"] * (m["left"]["dim"] + m["left"]["vdim"])
+                    read += seen * m["left"]["kv_heads"] * (m["left"]["dim"] + m["left"]["vdim"])
+                else:
+                    windowed = kind == "attention"
+                    prompt_pairs += (sum(visible(i) for i in range(prompt_len)) if windowed else every) * m["heads"] * 256
+                    read += (visible(seen) if windowed else seen) * m["kv_heads"] * 256
+                    state += 0 if windowed else 3 * (m["heads"] + m["kv_heads"]) * 128
+            if "prefill" in args.phases:
+                room = prompt_len + 64
+                engine = SyncEngine(model=model, path="", dtype=args.dtype, device="cuda:0", max_len=room, block_size=BLOCK,
+                                    num_blocks=-(-room // BLOCK), max_num_seqs=1, max_num_tokens=prompt_len,
+                                    chunked_prefill_size=prompt_len, enable_prefix_cache=False)
+                timings = []
+                for _ in range(4):
+                    engine.add_request(torch.randint(0, vocab, (prompt_len,), generator=gen).tolist(),
+                                       engine.default_params(1, temperature=0.0, ignore_eos=True))
+                    sync()
+                    t0 = time.perf_counter()
+                    engine.step()
+                    sync()
+                    timings.append(time.perf_counter() - t0)
+                    while engine.scheduler.has_work():
+                        engine.step()
+                seconds = sorted(timings[1:])[1]
+                flops = 2.0 * prompt_len * (matrices + scans) + 2.0 * vocab * W + 2.0 * prompt_pairs
+                entry["prefill"] = {"tokens": prompt_len, "tokens_per_s": round(prompt_len / seconds, 1),
+                                    "ms": round(seconds * 1e3, 3), "frac": round(flops / seconds / PEAK_FLOPS[args.dtype], 4)}
+                del engine
+            for batch in ((8, 64) if "decode" in args.phases else ()):
+                engine = SyncEngine(model=model, path="", dtype=args.dtype, device="cuda:0", max_len=context,
+                                    block_size=BLOCK, num_blocks=batch * (context // BLOCK), max_num_seqs=batch,
+                                    max_num_tokens=max(2048, batch), chunked_prefill_size=2048, enable_prefix_cache=False)
+                params = engine.default_params(context - decode_prompt - 1, temperature=0.0, ignore_eos=True)
+                requests = [engine.add_request(torch.randint(0, vocab, (decode_prompt,), generator=gen).tolist(), params)
+                            for _ in range(batch)]
+                while any(r.is_prefill for r in requests) or len(engine.scheduler.waiting):
+                    engine.step()
+                for _ in range(args.warmup):
+                    engine.step()
+                sync()
+                t0 = time.perf_counter()
+                for _ in range(args.steps):
+                    engine.step()
+                sync()
+                step_s = (time.perf_counter() - t0) / args.steps
+                need = 2 * (matrices + vocab * W) + batch * (8 * state + 2 * read)
+                entry["decode_b%d" % batch] = {"tokens_per_s": round(batch / step_s, 1), "ms_per_step": round(step_s * 1e3, 3),
+                                               "frac_hbm": round(need / step_s / PEAK_HBM, 4)}
+                del engine
+            results.setdefault(shape, {})[name] = entry
+            del model
+            torch.cuda.empty_cache()
+        results[shape]["sizes"] = {"width": W, "ff": ff, "window": window, "pool": pool, "layers": list(kinds), "vocab": vocab}
+    print(json.dumps({"metric": "Zedotar beside Surasun at equal size: prefill and decode tokens/s",
+                      "unit": "tokens/s", "n_gpus": 1, "higher_is_better": True, "dtype": "bf16", "data": "synthetic",
+                      "steps": args.steps, "warmup": args.warmup, "shapes": results}))
+    return 0
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -836,13 +977,14 @@ def main():
     ap.add_argument("--shape", default="8b", choices=sorted(SHAPES))
     ap.add_argument("--prompt", type=int, default=2048, help="tokens every request holds when decoding starts")
     ap.add_argument("--context", type=int, default=8192, help="tokens of cache per request")
-    ap.add_argument("--workload", default="decode", choices=["decode", "continuous", "served", "prefix", "products", "kodisun", "surasun", "dufinex", "fidevik"],
+    ap.add_argument("--workload", default="decode", choices=["decode", "continuous", "served", "prefix", "products", "kodisun", "surasun", "dufinex", "fidevik",
+                                                                 "zedotar"],
                     help="continuous: 64 requests at once, prompts of 128 to 4,096 tokens, 64 to 512 generated "
                          "tokens each, prompts in portions of 512 (its own JSON line; --steps and --warmup unused); "
                          "prefix: 64 requests that share their first 2,048 tokens, with the prefix index on and off; "
                          "products: a layer's four products by the chosen kernel and by each tile shape of the "
-                         "hand-written one; kodisun, surasun: that design beside the dense decoder at equal size; dufinex: "
-                         "that design beside Surasun at equal size")
+                         "hand-written one; kodisun, surasun: that design beside the dense decoder at equal size; dufinex, "
+                         "zedotar: that design beside Surasun at equal size; fidevik: beside Kodisun")
     ap.add_argument("--kodisun-shape", default="all", choices=["all"] + sorted(KODISUN_SHAPES))
     ap.add_argument("--kodisun-only", default="", choices=["", "kodisun", "qwen3_dense"], help="one of the two models")
     ap.add_argument("--surasun-shape", default="all", choices=["all"] + sorted(SURASUN_SHAPES))
@@ -851,8 +993,10 @@ def main():
     ap.add_argument("--dufinex-only", default="", choices=["", "dufinex", "surasun"], help="one of the two models")
     ap.add_argument("--fidevik-shape", default="all", choices=["all"] + sorted(FIDEVIK_SHAPES))
     ap.add_argument("--fidevik-only", default="", choices=["", "fidevik", "kodisun"], help="one of the two models")
+    ap.add_argument("--zedotar-shape", default="all", choices=["all"] + sorted(ZEDOTAR_SHAPES))
+    ap.add_argument("--zedotar-only", default="", choices=["", "zedotar", "surasun"], help="one of the two models")
     ap.add_argument("--phases", default="prefill,decode",
-                    help="of --workload kodisun, surasun, dufinex or fidevik: prefill, decode or both")
+                    help="of --workload kodisun, surasun, dufinex, fidevik or zedotar: prefill, decode or both")
     ap.add_argument("--single-copy", action="store_true",
                     help="hold the matrices once (no tile-ordered copy for steps of few rows): half the weights' memory, slower decoding")
     ap.add_argument("--no-points", action="store_true", help="skip the batch-1 and batch-64 points")
@@ -888,6 +1032,10 @@ def main():
         torch.cuda.set_device(0)
         args.steps, args.warmup = min(args.steps, 32), min(args.warmup, 8)
         return fidevik(args, torch.cuda.synchronize)
+    if args.workload == "zedotar":
+        torch.cuda.set_device(0)
+        args.steps, args.warmup = min(args.steps, 32), min(args.warmup, 8)
+        return zedotar(args, torch.cuda.synchronize)
     shape_name, raw = SHAPES[args.shape]
     raw = dict(raw)
     prompt_len, context = args.prompt, args.context

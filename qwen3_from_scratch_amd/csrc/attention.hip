@@ -224,6 +224,33 @@ static inline float make_score_scale(float scale) { return scale * 1.44269504088
 // maximum stands -bias log2(e), which never moves, so that the argument is formed as an exponent is
 // elsewhere; wherever results are joined every weight is one. `q3_set_sigmoid_bias` names the
 // biases (one per query head) of the launches that follow in the calling thread.
+// The builds with Q3_POOLED or Q3_SIGMOID also multiply a result by sigmoid(gate) on its way out, where
+// its row is final: `gate` float32, rows `stride` apart, a number per head or (`wide`) one per column;
+// null: no gate. `q3_set_gate` names the gate of the launches that follow in the calling thread.
+#if defined(Q3_POOLED) || defined(Q3_SIGMOID)
+#define Q3_GATED 1
+struct OutGate {
+  const float* gate;
+  long stride;
+  int wide;
+};
+static thread_local OutGate g_gate{};
+extern "C" void q3_set_gate(const float* gate, long stride, int wide) { g_gate = OutGate{gate, stride, wide}; }
+#define Q3_GATE_PARAM , OutGate gate
+#define Q3_GATE_ARG , g_gate
+// the factor of column d of head `head` (of D) of row `row`
+__device__ __forceinline__ float open_gate(const OutGate& g, int row, int head, int D, int d) {
+  if (g.gate == nullptr) return 1.f;
+  const float z = g.gate[(size_t)row * g.stride + (g.wide ? head * D + d : head)];
+  return __builtin_amdgcn_rcpf(1.f + fast_exp2(-1.4426950408889634f * z));
+}
+#define Q3_OPEN(row, head, D, d) *open_gate(gate, row, head, D, d)
+#else
+#define Q3_GATE_PARAM
+#define Q3_GATE_ARG
+#define Q3_OPEN(row, head, D, d)
+#endif
+
 #ifdef Q3_SIGMOID
 #define Q3_BIAS_PARAM , const float* __restrict__ score_bias
 #define Q3_BIAS_ARG , g_score_bias
@@ -546,6 +573,61 @@ __device__ __forceinline__ void attend_tiles_ahead(const Pack16 (&qreg)[QB][D / 
   }
 }
 
+#ifdef Q3_POOLED
+// Both sources of a wavefront's rows as one sequence of tiles: of tiles first, first + step, ... below
+// last, those before `run_tiles` are runs', the others tokens' from tile `tile_lo` on. As in
+// attend_tiles_ahead a tile's keys and values are asked for a whole tile before they are used and its
+// table entries two tiles before.
+template <int D>
+__device__ __forceinline__ void attend_both(const Pack16 (&qreg)[1][D / 32], const bf16_t* __restrict__ k_cache,
+                                            const bf16_t* __restrict__ v_cache, int num_pages,
+                                            const int* __restrict__ bt_row, int bt_stride, const RunSource& runs,
+                                            const int* __restrict__ run_row, int Hkv, int g_kv, int page, int first,
+                                            int last, int step, int run_tiles, int tile_lo, int kv_len,
+                                            const int (&row_pos)[1], int window, score_scale_t scale_log2,
+                                            f32x4_t (&acc)[1][D / 16], float (&m_run)[1], float (&l_run)[1]) {
+  if (first >= last) return;
+  const int run_pos = runs_seen(row_pos[0], window, runs.pool) - 1, run_count = kv_len / runs.pool;
+  auto key_of = [&](int s) { return (s < run_tiles ? s : tile_lo + s - run_tiles) * FAST_TILE; };
+  auto pages_of = [&](int s) {
+    return s < run_tiles ? tile_pages(run_row, runs.stride, page, key_of(s)) : tile_pages(bt_row, bt_stride, page, key_of(s));
+  };
+  auto addr_of = [&](const TilePages& p, int s) {
+    const bool run = s < run_tiles;
+    return tile_addr_of(p, run ? runs.k : k_cache, run ? runs.v : v_cache, run ? runs.num_pages : num_pages, Hkv, g_kv, page,
+                        D, key_of(s));
+  };
+  Pack16 a_cur[2][D / 32], v_cur[D / 16], a_nxt[2][D / 32], v_nxt[D / 16];
+  {
+    const TileAddr t = addr_of(pages_of(first), first);
+    load_keys<D>(a_cur, t);
+    load_values<D>(v_cur, t, page);
+  }
+  TilePages p_nxt = pages_of(first + step);
+  for (int s = first; s < last; s += step) {
+    const bool more = s + step < last;
+    if (more) {
+      const TileAddr t = addr_of(p_nxt, s + step);
+      load_keys<D>(a_nxt, t);
+      load_values<D>(v_nxt, t, page);
+      p_nxt = pages_of(s + 2 * step);
+    }
+    const bool run = s < run_tiles;
+    int pos[1] = {run ? run_pos : row_pos[0]};
+    attend_tile<D, 1>(qreg, a_cur, v_cur, key_of(s), run ? run_count : kv_len, pos, run ? 0 : window, scale_log2, acc, m_run,
+                      l_run);
+    if (more) {
+#pragma unroll
+      for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+        for (int i = 0; i < D / 32; ++i) a_cur[kb][i] = a_nxt[kb][i];
+#pragma unroll
+      for (int nb = 0; nb < D / 16; ++nb) v_cur[nb] = v_nxt[nb];
+    }
+  }
+}
+#endif
+
 // ---- sequences with few rows (q_len * G <= 16): decoding ---------------------
 // grid (splits, Hkv, B), 256 threads. The four wavefronts of a block take the
 // tiles of the block's share of the keys in turn and are merged through shared
@@ -702,7 +784,7 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(
     const bf16_t* __restrict__ v_cache, int num_pages, const int* __restrict__ block_table, int bt_stride,
     const int* __restrict__ cu_q, const int* __restrict__ kv_lens, int Hq, int Hkv, int page, score_scale_t scale_log2,
     int window, int splits, float* __restrict__ ws_acc, float* __restrict__ ws_ml, DecodePrep prep,
-    const float* __restrict__ sink Q3_BIAS_PARAM Q3_RUNS_PARAM) {
+    const float* __restrict__ sink Q3_BIAS_PARAM Q3_RUNS_PARAM Q3_GATE_PARAM) {
   const int b = blockIdx.z, g_kv = blockIdx.y, split = blockIdx.x;
   const int G = Hq / Hkv;
   // a step of single tokens (PREP): sequence b's token is row b, and nothing is read to know it
@@ -785,15 +867,17 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(
   const int all_tiles = run_tiles + max(tile_hi - tile_lo, 0);
   const int per_split = (all_tiles + splits - 1) / splits;
   const int s0 = min(split * per_split, all_tiles), s1 = min(s0 + per_split, all_tiles);
-  const int t0 = tile_lo + max(s0 - run_tiles, 0), t1 = tile_lo + max(s1 - run_tiles, 0);
+  (void)t_first;
 #else
   const int per_split = (max(tile_hi - tile_lo, 0) + splits - 1) / splits;
   const int t0 = tile_lo + split * per_split;
   const int t1 = min(tile_hi, t0 + per_split);
 #endif
+#ifndef Q3_POOLED
   // the first tile's keys are on their way while the query rows are prepared
   if constexpr (!ahead)
     t_first = first_tile_keys<D>(a_first, k_cache, v_cache, num_pages, bt_row, Hkv, g_kv, page, t0 + wave, t1, kv_seen);
+#endif
   float m_new = -INFINITY;  // in the last wavefront: the new key's score for this lane's row
   if constexpr (PREP) {
     prepare_query<D, W>(qreg[0], static_cast<const W*>(prep.q_weight), prep.eps, table_row, grp);
@@ -829,6 +913,10 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(
 #else
   float m_run[1] = {-INFINITY}, l_run[1] = {0.f};
 #endif
+#ifdef Q3_POOLED
+  attend_both<D>(qreg, k_cache, v_cache, num_pages, bt_row, bt_stride, runs, runs.table + (size_t)b * runs.stride, Hkv, g_kv,
+                 page, s0 + wave, s1, 4, run_tiles, tile_lo, kv_seen, row_pos, win, scale_log2, acc, m_run, l_run);
+#else
   if constexpr (ahead)
     attend_tiles_ahead<D, 1>(qreg, a_first, v_first, p_second, k_cache, v_cache, num_pages, bt_row, bt_stride, Hkv,
                              g_kv, page, ahead_first, tile_hi, ahead_step, kv_seen, row_pos, win, scale_log2, acc,
@@ -836,20 +924,9 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(
   else
     attend_tiles<D, 1>(qreg, a_first, t_first, k_cache, v_cache, num_pages, bt_row, Hkv, g_kv, page, t0 + wave, t1, 4,
                        kv_seen, row_pos, win, scale_log2, acc, m_run, l_run);
+#endif
 #ifdef Q3_SIGMOID
   m_run[0] = 0.f;
-#endif
-#ifdef Q3_POOLED
-  {
-    int run_pos[1];
-    run_pos[0] = runs_seen(row_pos[0], window, runs.pool) - 1;
-    const int* run_row = runs.table + (size_t)b * runs.stride;
-    const int run_first = s0 + wave, run_last = min(s1, run_tiles), run_count = kv_len / runs.pool;
-    t_first = first_tile_keys<D>(a_first, runs.k, runs.v, runs.num_pages, run_row, Hkv, g_kv, page, run_first, run_last,
-                                 run_count);
-    attend_tiles<D, 1>(qreg, a_first, t_first, runs.k, runs.v, runs.num_pages, run_row, Hkv, g_kv, page, run_first,
-                       run_last, 4, run_count, run_pos, 0, scale_log2, acc, m_run, l_run);
-  }
 #endif
 
   // this lane's sum covers its own keys only
@@ -897,7 +974,7 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(
     for (int d = dd; d < D; d += 16) {
       float o = sh_acc[0][r][d] + sh_acc[1][r][d] + sh_acc[2][r][d] + sh_acc[3][r][d];
       if (PREP && w5 > 0.f) o += sh_v[d] * w5;
-      out[(size_t)token * Hq * D + (size_t)head * D + d] = float_to_bf16(o * inv);
+      out[(size_t)token * Hq * D + (size_t)head * D + d] = float_to_bf16(o * inv Q3_OPEN(token, head, D, d));
     }
   } else {
     const size_t slot = (((size_t)b * Hkv + g_kv) * splits + split) * 16 + r;
@@ -927,7 +1004,7 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(
 template <int D>
 __global__ __launch_bounds__(256) void attn_decode_reduce_kernel(
     bf16_t* __restrict__ out, const int* __restrict__ cu_q, int Hq, int Hkv, int splits,
-    const float* __restrict__ ws_acc, const float* __restrict__ ws_ml, const float* __restrict__ sink) {
+    const float* __restrict__ ws_acc, const float* __restrict__ ws_ml, const float* __restrict__ sink Q3_GATE_PARAM) {
   __shared__ float sh_w[16][MAX_SPLITS];
   __shared__ float4 sh_part[256];
   const int b = blockIdx.y, g_kv = blockIdx.x;
@@ -1012,8 +1089,8 @@ __global__ __launch_bounds__(256) void attn_decode_reduce_kernel(
         uint2 u;
         bf16_t e[4];
       } pk;
-      pk.e[0] = float_to_bf16(o.x); pk.e[1] = float_to_bf16(o.y);
-      pk.e[2] = float_to_bf16(o.z); pk.e[3] = float_to_bf16(o.w);
+      pk.e[0] = float_to_bf16(o.x Q3_OPEN(token, head, D, d)); pk.e[1] = float_to_bf16(o.y Q3_OPEN(token, head, D, d + 1));
+      pk.e[2] = float_to_bf16(o.z Q3_OPEN(token, head, D, d + 2)); pk.e[3] = float_to_bf16(o.w Q3_OPEN(token, head, D, d + 3));
       *reinterpret_cast<uint2*>(out + (size_t)token * Hq * D + (size_t)head * D + d) = pk.u;
     }
   }
@@ -1156,7 +1233,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
     const bf16_t* __restrict__ v_cache, int num_pages, const int* __restrict__ block_table, int bt_stride,
     const int* __restrict__ cu_q, const int* __restrict__ kv_lens, int Hq, int Hkv, int page, score_scale_t scale_log2,
     int window, int tokens_per_block, int key_splits, float* __restrict__ part_acc, float* __restrict__ part_ml,
-    const float* __restrict__ sink Q3_BIAS_PARAM Q3_RUNS_PARAM) {
+    const float* __restrict__ sink Q3_BIAS_PARAM Q3_RUNS_PARAM Q3_GATE_PARAM) {
   typedef PrefillSmem<D, TILE> SM;
   constexpr int KB4 = TILE / 16;  // 16-key blocks per tile
   __shared__ __attribute__((aligned(16))) unsigned char smem[STAGES * SM::STAGE];
@@ -1609,7 +1686,8 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
         bf16_t e[4];
       } pk;
 #pragma unroll
-      for (int j = 0; j < 4; ++j) pk.e[j] = float_to_bf16(acc[qb][nb][j] * inv);
+      for (int j = 0; j < 4; ++j)
+        pk.e[j] = float_to_bf16(acc[qb][nb][j] * inv Q3_OPEN(row_tok[qb], row_head[qb], D, 16 * nb + 4 * grp + j));
       *reinterpret_cast<uint2*>(o + 16 * nb) = pk.u;
     }
   }
@@ -1623,7 +1701,7 @@ __global__ __launch_bounds__(256) void attn_prefill_merge_kernel(bf16_t* __restr
                                                                  const int* __restrict__ cu_q, int Hq, int Hkv,
                                                                  int key_splits, const float* __restrict__ part_acc,
                                                                  const float* __restrict__ part_ml,
-                                                                 const float* __restrict__ sink) {
+                                                                 const float* __restrict__ sink Q3_GATE_PARAM) {
   const int b = blockIdx.y;
   const int q0 = cu_q[b], q_len = cu_q[b + 1] - q0;
   if (q_len * (Hq / Hkv) <= 16) return;
@@ -1656,8 +1734,10 @@ __global__ __launch_bounds__(256) void attn_prefill_merge_kernel(bf16_t* __restr
       uint2 u;
       bf16_t e[4];
     } pk;
-    pk.e[0] = float_to_bf16(o.x * inv); pk.e[1] = float_to_bf16(o.y * inv);
-    pk.e[2] = float_to_bf16(o.z * inv); pk.e[3] = float_to_bf16(o.w * inv);
+    const int token = q0 + first;
+    (void)token;
+    pk.e[0] = float_to_bf16(o.x * inv Q3_OPEN(token, row, D, d)); pk.e[1] = float_to_bf16(o.y * inv Q3_OPEN(token, row, D, d + 1));
+    pk.e[2] = float_to_bf16(o.z * inv Q3_OPEN(token, row, D, d + 2)); pk.e[3] = float_to_bf16(o.w * inv Q3_OPEN(token, row, D, d + 3));
     *reinterpret_cast<uint2*>(out + ((size_t)(q0 + first) * Hq + row) * D + d) = pk.u;
   }
 }
@@ -1700,19 +1780,21 @@ static int launch_fast(const void* q, int q_stride, void* out, const void* k_cac
   if (window != 0 || g_score_bias == nullptr || sink != nullptr) return Q3_ERR_BAD_ARGUMENT;
 #endif
   if (min_q_len * G <= 16) {
+#ifndef Q3_POOLED
     if (window == 0)
       hipLaunchKernelGGL((attn_decode_kernel<D, false, float, true>), dim3(splits, Hkv, B), dim3(256), 0, stream,
                          (const bf16_t*)q, q_stride, (bf16_t*)out, (const bf16_t*)k_cache, (const bf16_t*)v_cache,
                          num_pages, block_table, bt_stride, cu_q, kv_lens, Hq, Hkv, page, scale_log2, window, splits,
-                         ws_acc, ws_ml, DecodePrep{}, sink Q3_BIAS_ARG Q3_RUNS_ARG);
+                         ws_acc, ws_ml, DecodePrep{}, sink Q3_BIAS_ARG Q3_RUNS_ARG Q3_GATE_ARG);
     else
+#endif
       hipLaunchKernelGGL((attn_decode_kernel<D, false, float, false>), dim3(splits, Hkv, B), dim3(256), 0, stream,
                          (const bf16_t*)q, q_stride, (bf16_t*)out, (const bf16_t*)k_cache, (const bf16_t*)v_cache,
                          num_pages, block_table, bt_stride, cu_q, kv_lens, Hq, Hkv, page, scale_log2, window, splits,
-                         ws_acc, ws_ml, DecodePrep{}, sink Q3_BIAS_ARG Q3_RUNS_ARG);
+                         ws_acc, ws_ml, DecodePrep{}, sink Q3_BIAS_ARG Q3_RUNS_ARG Q3_GATE_ARG);
     if (splits > 1)
       hipLaunchKernelGGL(attn_decode_reduce_kernel<D>, dim3(Hkv, B), dim3(256), 0, stream, (bf16_t*)out, cu_q, Hq,
-                         Hkv, splits, ws_acc, ws_ml, sink);
+                         Hkv, splits, ws_acc, ws_ml, sink Q3_GATE_ARG);
   }
   if (max_q_len * G > 16) {
     const int tokens_per_block = prompt_tokens_per_block(total_tokens, G, Hkv, key_splits);
@@ -1723,10 +1805,10 @@ static int launch_fast(const void* q, int q_stride, void* out, const void* k_cac
     hipLaunchKernelGGL((attn_prefill_kernel<D, PF_TILE, PF_STAGES>), dim3(Hkv, tiles * key_splits, B), dim3(256), 0,
                        stream, (const bf16_t*)q, q_stride, (bf16_t*)out, (const bf16_t*)k_cache,
                        (const bf16_t*)v_cache, num_pages, block_table, bt_stride, cu_q, kv_lens, Hq, Hkv, page,
-                       scale_log2, window, tokens_per_block, key_splits, part_acc, part_ml, sink Q3_BIAS_ARG Q3_RUNS_ARG);
+                       scale_log2, window, tokens_per_block, key_splits, part_acc, part_ml, sink Q3_BIAS_ARG Q3_RUNS_ARG Q3_GATE_ARG);
     if (key_splits > 1)
       hipLaunchKernelGGL(attn_prefill_merge_kernel<D>, dim3(max_q_len, B), dim3(256), 0, stream,
-                         (bf16_t*)out, cu_q, Hq, Hkv, key_splits, part_acc, part_ml, sink);
+                         (bf16_t*)out, cu_q, Hq, Hkv, key_splits, part_acc, part_ml, sink Q3_GATE_ARG);
   }
   return q3_launch_status();
 }

@@ -219,22 +219,27 @@ __global__ void __launch_bounds__(256) mlstm_chunk_sums_kernel(const float* __re
   const int tile = rest / d_tiles, i0 = rest % d_tiles * 64, j0 = tile * 64;
   const size_t row0 = (size_t)start + c * Q3_CHUNK;
   const size_t chunk = (size_t)mlstm_chunks_before(cu, b) + c;
-  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), col = lane & 15, grp = lane >> 4;
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), col = lane & 15,
+            grp = lane >> 4;
+  // rows past the chunk's end have weight zero and are read from the last that exists, as are columns past the
+  // head's, whose results nobody keeps: no load waits behind a branch
+  const float *k0 = sh.k(rows, row0, h), *v0 = sh.v(rows, row0, h);
+  const int stride = (int)sh.row_stride, k_col = min(i0 + lane, sh.d - 1), v_col = min(j0 + lane, sh.dv - 1);
   float gk[16], gv[16];
 #pragma unroll
   for (int u = 0; u < 16; ++u) {
-    const int s = (tid >> 6) + 4 * u, e = tid & 63;
-    gk[u] = (s < len && i0 + e < sh.d) ? sh.k(rows, row0 + s, h)[i0 + e] : 0.f;
-    gv[u] = (s < len && j0 + e < sh.dv) ? sh.v(rows, row0 + s, h)[j0 + e] : 0.f;
+    const int s = min(wave + 4 * u, len - 1) * stride;
+    gk[u] = (k0 + s)[k_col];
+    gv[u] = (v0 + s)[v_col];
   }
   if (tid < Q3_CHUNK)
     weight[tid] = tid < len ? expf((float)(lift[(row0 + tid) * sh.H + h] - top[(row0 + len - 1) * sh.H + h])) : 0.f;
   __syncthreads();
 #pragma unroll
   for (int u = 0; u < 16; ++u) {
-    const int s = (tid >> 6) + 4 * u, e = tid & 63;
-    kw[s * ML_LDB + e] = gk[u] * weight[s];
-    vt[s * ML_LDB + e] = gv[u];
+    const int s = wave + 4 * u;
+    kw[s * ML_LDB + lane] = gk[u] * weight[s];
+    vt[s * ML_LDB + lane] = gv[u];
   }
   __syncthreads();
   mat4_t acc[4];
@@ -311,60 +316,85 @@ __global__ void __launch_bounds__(256) mlstm_chunk_scan_kernel(float* __restrict
   }
 }
 
-// grid (chunks of the longest sequence, H, B), 256 threads: the chunk's results of one head, a wavefront 16 of
-// its rows. First the weights W[t][s] = (q_t . k_s) exp(a_s - g_t), s <= t, into shared memory, and the
-// denominators from their sums and q . n0; then, 64 columns at a time, exp(m0 - g_t) q S0 + W v over the
-// denominator into `raw` (T, H dv); last every row over its root mean square, times `norm` and sigmoid(gate).
-template <typename TA>
+// grid (chunks of the longest sequence, H * tiles, B), 256 threads: the chunk's results in 64 columns of one
+// head, a wavefront 16 of its rows. First the weights W[t][s] = (q_t . k_s) exp(a_s - g_t), s <= t, into shared
+// memory, and the denominators from their sums and q . n0; then exp(m0 - g_t) q S0 + W v over the denominator.
+// A slice of 64 of the inner size is asked for while the one before it is worked on. With one tile a head's row
+// is whole here and leaves over its root mean square, times `norm` and sigmoid(gate), into `out`; with more it
+// goes to `raw` (T, H dv), and mlstm_finish_kernel follows.
+template <typename TA, bool FINISH>
 __global__ void __launch_bounds__(256) mlstm_chunk_output_kernel(
     const float* __restrict__ rows, MlstmShape sh, float* __restrict__ state, const int* __restrict__ slots,
     const int* __restrict__ cu, const double* __restrict__ sum_f, const double* __restrict__ lift,
     const double* __restrict__ top, const float* __restrict__ sums, const float* __restrict__ before,
-    const float* __restrict__ norm, float* raw, TA* __restrict__ out) {
+    const float* __restrict__ norm, float* __restrict__ raw, TA* __restrict__ out) {
   __shared__ __attribute__((aligned(16))) float W[Q3_CHUNK * ML_LDA];
   __shared__ __attribute__((aligned(16))) float qs[Q3_CHUNK * ML_LDA];
   __shared__ __attribute__((aligned(16))) float other[Q3_CHUNK * ML_LDB];
   __shared__ float ns[64];
   __shared__ double lifts[Q3_CHUNK];
-  const int b = blockIdx.z, h = blockIdx.y, c = blockIdx.x;
+  const int b = blockIdx.z, h = blockIdx.y / sh.tiles, tile = blockIdx.y % sh.tiles, c = blockIdx.x;
   const int start = cu[b], count = cu[b + 1] - start, len = min(count - c * Q3_CHUNK, Q3_CHUNK);
   if (len <= 0) return;
-  const int d = sh.d, dv = sh.dv;
+  const int d = sh.d, dv = sh.dv, j0 = 64 * tile;
   const size_t row0 = (size_t)start + c * Q3_CHUNK;
   const size_t at = ((size_t)mlstm_chunks_before(cu, b) + c) * sh.H + h;
-  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), col = lane & 15, grp = lane >> 4;
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), col = lane & 15,
+            grp = lane >> 4;
   const float* S0 = sums + at * ((size_t)d * dv + d);
   const float* n0 = S0 + (size_t)d * dv;
   const double m0 = (double)before[at];
   if (tid < Q3_CHUNK) lifts[tid] = tid < len ? lift[(row0 + tid) * sh.H + h] : 0.0;
 
-  // 64 numbers from column e0 of q (scaled) into qs, and of k into `other`
-  auto load_rows = [&](int e0, bool with_k) {
-    float gq[16], gk[16];
+  // What a thread brings of a slice: number `lane` of rows wave + 4 u: q (scaled) and k from column e0 on, S0
+  // from row e0 on, v. Nothing branches: rows past the chunk's end and columns past the head's are read from
+  // the last one that exists. Such rows of q make results that nobody keeps, such rows of k and v have weight
+  // zero, and columns of q and k past the head's count as zero.
+  float ga[16], gb[16];
+  const float *q0 = sh.q(rows, row0, h), *k0 = sh.k(rows, row0, h), *v0 = sh.v(rows, row0, h);
+  const int stride = (int)sh.row_stride, v_col = min(j0 + lane, dv - 1);
+  auto ask_q = [&](int e0) {
+    const int e = min(e0 + lane, d - 1);
 #pragma unroll
-    for (int u = 0; u < 16; ++u) {
-      const int s = (tid >> 6) + 4 * u, e = e0 + (tid & 63);
-      const bool in = s < len && e < d;
-      gq[u] = in ? sh.q(rows, row0 + s, h)[e] * sh.q_scale : 0.f;
-      gk[u] = (in && with_k) ? sh.k(rows, row0 + s, h)[e] : 0.f;
-    }
+    for (int u = 0; u < 16; ++u) ga[u] = (q0 + min(wave + 4 * u, len - 1) * stride)[e];
+  };
+  auto ask_k = [&](int e0) {
+    const int e = min(e0 + lane, d - 1);
 #pragma unroll
-    for (int u = 0; u < 16; ++u) {
-      const int s = (tid >> 6) + 4 * u, e = tid & 63;
-      qs[s * ML_LDA + e] = gq[u];
-      if (with_k) other[s * ML_LDA + e] = gk[u];
-    }
+    for (int u = 0; u < 16; ++u) gb[u] = (k0 + min(wave + 4 * u, len - 1) * stride)[e];
+  };
+  auto ask_S = [&](int e0) {
+#pragma unroll
+    for (int u = 0; u < 16; ++u) gb[u] = (S0 + (size_t)min(e0 + wave + 4 * u, d - 1) * dv)[v_col];
+  };
+  auto ask_v = [&]() {
+#pragma unroll
+    for (int u = 0; u < 16; ++u) gb[u] = (v0 + min(wave + 4 * u, len - 1) * stride)[v_col];
+  };
+  auto put = [&](float (&from)[16], float* to, int apart, float scale) {
+#pragma unroll
+    for (int u = 0; u < 16; ++u) to[(wave + 4 * u) * apart + lane] = scale == 0.f ? 0.f : from[u] * scale;
   };
 
   mat4_t acc[4];
 #pragma unroll
   for (int x = 0; x < 4; ++x) acc[x] = mat4_t{0.f, 0.f, 0.f, 0.f};
   float dot_n = 0.f;                    // row 16 wave + col's q . n0, the numbers 4 i + grp of it
+  ask_q(0);
+  ask_k(0);
   for (int e0 = 0; e0 < d; e0 += 64) {
     __syncthreads();
-    load_rows(e0, true);
+    put(ga, qs, ML_LDA, e0 + lane < d ? sh.q_scale : 0.f);
+    put(gb, other, ML_LDA, e0 + lane < d ? 1.f : 0.f);
     if (tid < 64) ns[tid] = e0 + tid < d ? n0[e0 + tid] : 0.f;
     __syncthreads();
+    if (e0 + 64 < d) {
+      ask_q(e0 + 64);
+      ask_k(e0 + 64);
+    } else {
+      if (d > 64) ask_q(0);             // the first slice of the product with S0; a single slice is still in place
+      ask_S(0);
+    }
 #pragma unroll
     for (int i = 0; i < 64; i += 4) {
       const float a = qs[(16 * wave + col) * ML_LDA + i + grp];
@@ -377,7 +407,7 @@ __global__ void __launch_bounds__(256) mlstm_chunk_output_kernel(
   }
   dot_n += __shfl_xor(dot_n, 16, 64);
   dot_n += __shfl_xor(dot_n, 32, 64);
-  float carry[4], under[4], squares[4];
+  float carry[4], under[4];
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
     const int t = 16 * wave + 4 * grp + r;
@@ -397,90 +427,75 @@ __global__ void __launch_bounds__(256) mlstm_chunk_output_kernel(
     carry[r] = real ? expf((float)(m0 - g)) : 0.f;
     const float den = sum + carry[r] * __shfl(dot_n, 4 * grp + r, 64);
     under[r] = 1.f / (fmaxf(fabsf(den), real ? expf((float)(-(b_t + g))) : 1.f) + sh.small);
-    squares[r] = 0.f;
   }
-  for (int tile = 0; tile < sh.tiles; ++tile) {
-    const int j0 = 64 * tile;
 #pragma unroll
-    for (int x = 0; x < 4; ++x) acc[x] = mat4_t{0.f, 0.f, 0.f, 0.f};
-    for (int e0 = 0; e0 < d; e0 += 64) {
-      __syncthreads();
-      if (d > 64) load_rows(e0, false);          // otherwise q is still there
-      {
-        float gs[16];
-#pragma unroll
-        for (int u = 0; u < 16; ++u) {
-          const int i = e0 + (tid >> 6) + 4 * u, j = j0 + (tid & 63);
-          gs[u] = (i < d && j < dv) ? S0[(size_t)i * dv + j] : 0.f;
-        }
-#pragma unroll
-        for (int u = 0; u < 16; ++u) other[((tid >> 6) + 4 * u) * ML_LDB + (tid & 63)] = gs[u];
-      }
-      __syncthreads();
-#pragma unroll
-      for (int i = 0; i < 64; i += 4) {
-        const float a = qs[(16 * wave + col) * ML_LDA + i + grp];
-#pragma unroll
-        for (int x = 0; x < 4; ++x)
-          acc[x] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, other[(i + grp) * ML_LDB + 16 * x + col], acc[x], 0, 0, 0);
-      }
+  for (int x = 0; x < 4; ++x) acc[x] = mat4_t{0.f, 0.f, 0.f, 0.f};
+  for (int e0 = 0; e0 < d; e0 += 64) {
+    __syncthreads();
+    if (d > 64) put(ga, qs, ML_LDA, e0 + lane < d ? sh.q_scale : 0.f);
+    put(gb, other, ML_LDB, 1.f);
+    __syncthreads();
+    if (e0 + 64 < d) {
+      ask_q(e0 + 64);
+      ask_S(e0 + 64);
+    } else {
+      ask_v();
     }
 #pragma unroll
-    for (int x = 0; x < 4; ++x)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) acc[x][r] *= carry[r];
-    __syncthreads();
-    {
-      float gv[16];
-#pragma unroll
-      for (int u = 0; u < 16; ++u) {
-        const int s = (tid >> 6) + 4 * u, j = j0 + (tid & 63);
-        gv[u] = (s < len && j < dv) ? sh.v(rows, row0 + s, h)[j] : 0.f;
-      }
-#pragma unroll
-      for (int u = 0; u < 16; ++u) other[((tid >> 6) + 4 * u) * ML_LDB + (tid & 63)] = gv[u];
-    }
-    __syncthreads();
-    for (int s = 0; s < 16 * (wave + 1); s += 4) {
-      const float a = W[(16 * wave + col) * ML_LDA + s + grp];
+    for (int i = 0; i < 64; i += 4) {
+      const float a = qs[(16 * wave + col) * ML_LDA + i + grp];
 #pragma unroll
       for (int x = 0; x < 4; ++x)
-        acc[x] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, other[(s + grp) * ML_LDB + 16 * x + col], acc[x], 0, 0, 0);
-    }
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int t = 16 * wave + 4 * grp + r;
-#pragma unroll
-      for (int x = 0; x < 4; ++x) {
-        const int j = j0 + 16 * x + col;
-        const float o = acc[x][r] * under[r];
-        if (t < len && j < dv) {
-          squares[r] += o * o;
-          raw[((row0 + t) * sh.H + h) * dv + j] = o;
-        }
-      }
+        acc[x] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, other[(i + grp) * ML_LDB + 16 * x + col], acc[x], 0, 0, 0);
     }
   }
-  // every thread reads again what it has written itself
+#pragma unroll
+  for (int x = 0; x < 4; ++x)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) acc[x][r] *= carry[r];
+  __syncthreads();
+  put(gb, other, ML_LDB, 1.f);
+  __syncthreads();
+  for (int s = 0; s < 16 * (wave + 1); s += 4) {
+    const float a = W[(16 * wave + col) * ML_LDA + s + grp];
+#pragma unroll
+    for (int x = 0; x < 4; ++x)
+      acc[x] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, other[(s + grp) * ML_LDB + 16 * x + col], acc[x], 0, 0, 0);
+  }
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
     const int t = 16 * wave + 4 * grp + r;
-    float sq = squares[r];
+    const float* gate = sh.gate(rows, row0 + (t < len ? t : 0), h);
+    float inv = 1.f;
+    if (FINISH) {
+      float sq = 0.f;
 #pragma unroll
-    for (int off = 1; off < 16; off <<= 1) sq += __shfl_xor(sq, off, 64);
-    const float inv = rsqrtf(sq / (float)dv + sh.eps);
-    if (t >= len) continue;
-    const float* gate = sh.gate(rows, row0 + t, h);
-    for (int j = col; j < dv; j += 16) {
-      const size_t place = ((row0 + t) * sh.H + h) * dv + j;
-      out[place] = from_float<TA>(raw[place] * inv * norm[h * dv + j] * gate_sigmoid(gate[j]));
+      for (int x = 0; x < 4; ++x) {
+        const float o = 16 * x + col < dv ? acc[x][r] * under[r] : 0.f;
+        sq += o * o;
+      }
+#pragma unroll
+      for (int off = 1; off < 16; off <<= 1) sq += __shfl_xor(sq, off, 64);
+      inv = rsqrtf(sq / (float)dv + sh.eps);
+    }
+#pragma unroll
+    for (int x = 0; x < 4; ++x) {
+      const int j = j0 + 16 * x + col;
+      if (t < len && j < dv) {
+        const size_t place = ((row0 + t) * sh.H + h) * dv + j;
+        const float o = acc[x][r] * under[r];
+        if (FINISH)
+          out[place] = from_float<TA>(o * inv * norm[h * dv + j] * gate_sigmoid(gate[j]));
+        else
+          raw[place] = o;
+      }
     }
   }
   // the m after the sequence's last row: as the scan has it
-  if ((c + 1) * Q3_CHUNK >= count && tid < sh.tiles) {
+  if ((c + 1) * Q3_CHUNK >= count && tid == 0) {
     const size_t last = row0 + len - 1;
     const double B = sum_f[last * sh.H + h];
-    *sh.m(state + (size_t)slots[b] * sh.state_stride, h, tid) = (float)fmax(m0 + B, top[last * sh.H + h] + B);
+    *sh.m(state + (size_t)slots[b] * sh.state_stride, h, tile) = (float)fmax(m0 + B, top[last * sh.H + h] + B);
   }
 }
 
@@ -514,7 +529,7 @@ extern "C" int q3_mlstm_scan(const float* rows, long row_stride, const float* i_
   if (T <= 0 || B <= 0 || max_q_len <= 0 || !mlstm_shape(sh, H, d, dv, row_stride, state_stride, cap, small, eps))
     return Q3_ERR_BAD_ARGUMENT;
   const long d_tiles = (d + 63) / 64;
-  if (d > 512 || B > 65535 || (long)H * sh.tiles * d_tiles > 65535 || sh.tiles > 256) return Q3_ERR_UNSUPPORTED;
+  if (d > 512 || row_stride > (1 << 24) || B > 65535 || (long)H * sh.tiles * d_tiles > 65535 || sh.tiles > 256) return Q3_ERR_UNSUPPORTED;
   if (!chunked) {
     float* raw = (float*)workspace;
     const dim3 grid(H * sh.tiles, B);
@@ -550,8 +565,16 @@ extern "C" int q3_mlstm_scan(const float* rows, long row_stride, const float* i_
                      cu, lift, top, sums);
   hipLaunchKernelGGL(mlstm_chunk_scan_kernel, dim3((unsigned)((size + 255) / 256), H, B), dim3(256), 0, stream, sums, sh,
                      state, slots, cu, sum_f, top, before);
+  if (sh.tiles == 1) {
+    Q3_DISPATCH_DTYPE(act_dtype, TA,
+                      hipLaunchKernelGGL((mlstm_chunk_output_kernel<TA, true>), dim3(chunks, H, B), dim3(256), 0, stream,
+                                         rows, sh, state, slots, cu, sum_f, lift, top, sums, before, norm, raw, (TA*)out));
+    return q3_launch_status();
+  }
+  hipLaunchKernelGGL((mlstm_chunk_output_kernel<float, false>), dim3(chunks, H * sh.tiles, B), dim3(256), 0, stream, rows,
+                     sh, state, slots, cu, sum_f, lift, top, sums, before, norm, raw, (float*)nullptr);
   Q3_DISPATCH_DTYPE(act_dtype, TA,
-                    hipLaunchKernelGGL(mlstm_chunk_output_kernel<TA>, dim3(chunks, H, B), dim3(256), 0, stream, rows, sh,
-                                       state, slots, cu, sum_f, lift, top, sums, before, norm, raw, (TA*)out));
+                    hipLaunchKernelGGL(mlstm_finish_kernel<TA>, dim3(T, H), dim3(64), 0, stream, raw, rows, sh, norm,
+                                       (TA*)out));
   return q3_launch_status();
 }

@@ -69,8 +69,8 @@ __global__ void softcap_prepare_kernel(const float* __restrict__ rows, long row_
   }
 }
 
-// Queries, keys and values without norms, turned by the position, i and i + half together. One block
-// per token, a wavefront per head in turn. The row is [q: H dim | k: G dim | v: G vdim | ...] float32,
+// Queries, keys and values without norms, turned by the position, i and i + half together. grid (T,
+// shares): a token's heads (queries', then keys') go over the wavefronts of its blocks in turn. The row is [q: H dim | k: G dim | v: G vdim | ...] float32,
 // `bias` covers q, k and v (null: none); with `values_are_keys` there is no v and a token's value is
 // its key before it turns. The first 2 * half numbers of every head of q and k turn by position *
 // inv_freq[i], cos and sin multiplied by `factor`; they are formed once per token, in shared memory. q
@@ -100,7 +100,8 @@ __global__ void __launch_bounds__(256) turn_prepare_kernel(
     int H, int G, int dim, int vdim, int values_are_keys, RunPlaces runs) {
   __shared__ float cs[Q3_TURN_HALF_MOST], sn[Q3_TURN_HALF_MOST];
   const int t = blockIdx.x;
-  const int wave = threadIdx.x / Q3_WAVE, lane = threadIdx.x % Q3_WAVE, waves = blockDim.x / Q3_WAVE;
+  const int lane = threadIdx.x % Q3_WAVE, waves = blockDim.x / Q3_WAVE * gridDim.y;
+  const int wave = blockIdx.y * (blockDim.x / Q3_WAVE) + threadIdx.x / Q3_WAVE;
   const float* row = rows + (size_t)t * row_stride;
   const int nq = H * dim, nk = G * dim;
   const int pos = positions[t];
@@ -133,7 +134,8 @@ __global__ void __launch_bounds__(256) turn_prepare_kernel(
     for (int e = lane; e < dim; e += Q3_WAVE) q_out[(size_t)t * nq + h * dim + e] = from_float<TA>(turned(x, add, e));
   }
   if (pg < 0) return;
-  for (int g = wave; g < G; g += waves) {
+  int g = wave - H % waves;                    // the wavefront after the last query head's takes the first key head
+  for (g = g < 0 ? g + waves : g; g < G; g += waves) {
     const float* x = row + nq + g * dim;
     const float* add = bias ? bias + nq + g * dim : nullptr;
     for (int e = lane; e < dim; e += Q3_WAVE) {
@@ -178,8 +180,11 @@ extern "C" int q3_turn_prepare(const float* rows, long row_stride, const float* 
   if (run_k && (!run_v || !run_table || run_width <= 0 || pool <= 0)) return Q3_ERR_BAD_ARGUMENT;
   if (half > Q3_TURN_HALF_MOST) return Q3_ERR_UNSUPPORTED;
   const RunPlaces runs{run_k, run_v, run_table, run_width, pool};
+  // few tokens: a wavefront per head; many: the tokens fill the chip, and share their cosines among more heads
+  const int most = (H + G + 3) / 4;
+  const int shares = T >= 1024 ? 1 : (T >= 256 ? (most < 2 ? most : 2) : (most < 64 ? most : 64));
   Q3_DISPATCH_DTYPE(act_dtype, TA,
-                    hipLaunchKernelGGL(turn_prepare_kernel<TA>, dim3(T), dim3(256), 0, stream, rows, row_stride, bias,
+                    hipLaunchKernelGGL(turn_prepare_kernel<TA>, dim3(T, shares), dim3(256), 0, stream, rows, row_stride, bias,
                                        inv_freq, half, factor, positions, seq_index, block_table, table_width,
                                        (TA*)k_cache, (TA*)v_cache, page, (TA*)q_out, H, G, dim, vdim, values_are_keys,
                                        runs));

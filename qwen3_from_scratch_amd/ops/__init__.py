@@ -1370,8 +1370,9 @@ def softcap_attention(q, k_cache, v_cache, block_table, cu_seqlens_q, kv_lens, s
             and library("attention").q3_paged_attention_fast_path(H, G, dim, page, _DT[q.dtype]):
         out = paged_attention(q, H, k_cache, v_cache, block_table, cu_seqlens_q, kv_lens, max_q_len, max_kv_len, scale,
                               window=window, min_q_len=min_q_len, max_kv_len_of_many=max_kv_len_of_many, softcap=softcap,
-                              sink=sink, runs=runs, sigmoid_bias=sigmoid_bias)
-        if gate is not None:
+                              sink=sink, runs=runs, sigmoid_bias=sigmoid_bias,
+                              gate=gate if runs is not None or sigmoid_bias is not None else None)
+        if gate is not None and runs is None and sigmoid_bias is None:
             _check(library("softcap").q3_gate_heads(_ptr(out), _ptr(gate), ctypes.c_long(stride), wide, T, H, vdim,
                                                     _DT[q.dtype], _stream()), "gate_heads")
         return out
@@ -1492,14 +1493,16 @@ def qk_norm_rope_store(qkv, num_q_heads, num_kv_heads, head_dim, positions, seq_
 
 def paged_attention(q, num_q_heads, k_cache, v_cache, block_table, cu_seqlens_q, kv_lens,
                     max_q_len, max_kv_len, scale, window=0, out=None, min_q_len=1, max_kv_len_of_many=None, softcap=0.0,
-                    sink=None, runs=None, sigmoid_bias=None):
+                    sink=None, runs=None, sigmoid_bias=None, gate=None):
     """Causal softmax attention of packed query rows over paged keys and values.
     `softcap` > 0: a score s enters the softmax as softcap * tanh(s * scale / softcap); that form
     exists for the sizes the matrix cores take (a second build of the same kernels) and no other.
     `sink` float32 (Hq,): exp(sink[h]) joins the denominator of head h's softmax (no key, no value).
     `runs` (keys, values, block table, tokens per run; see `_runs_args`) with a window: a row at position p
     also sees one key and value per run that ends at p - window or before. `sigmoid_bias` float32 (Hq,): no
-    softmax, a key counts with sigmoid(s * scale + sigmoid_bias[h]). These two are builds of their own as well.
+    softmax, a key counts with sigmoid(s * scale + sigmoid_bias[h]). These two are builds of their own as well,
+    and they alone take `gate` float32 (T, Hq) or (T, Hq D), rows possibly apart, whose sigmoid multiplies the
+    result where it is written.
 
     q is (T, Hq, D) seen through a row stride (a view of the qkv buffer is
     fine). Keys are cached as (pages, Hkv, page, D), values as
@@ -1569,6 +1572,14 @@ def paged_attention(q, num_q_heads, k_cache, v_cache, block_table, cu_seqlens_q,
             _f32(sigmoid_bias, (Hq,), "sigmoid_bias")
             lib.q3_set_sigmoid_bias.restype = None
             lib.q3_set_sigmoid_bias(_ptr(sigmoid_bias))
+        _need(gate is None or runs is not None or sigmoid_bias is not None, "a gate comes with runs or sigmoid weights only")
+        if runs is not None or sigmoid_bias is not None:
+            gate_stride = 0
+            if gate is not None:
+                gate_stride = _rows_view(gate, "gate")
+                _need(gate.shape in ((T, Hq), (T, Hq * D)) and gate.dtype == torch.float32, "gate must be float32 (T, Hq) or (T, Hq D)")
+            lib.q3_set_gate.restype = None
+            lib.q3_set_gate(_ptr(gate), ctypes.c_long(gate_stride), 1 if gate is not None and gate.shape[1] != Hq else 0)
         splits, workspace, prompt_splits, prompt_workspace = 1, None, 1, None
         if lib.q3_paged_attention_fast_path(Hq, Hkv, D, page, _DT[q.dtype]):
             if min_q_len * (Hq // Hkv) <= 16:
