@@ -87,9 +87,27 @@ struct RunPlaces {
   int width, pool;
 };
 
+// The sum of one number of a head over tokens first .. last - 1, in their order, from a paged cache: token j's
+// stands at element `offset + (j % page) * apart` of its page's head. Sixteen loads are asked for before the
+// first is used, none behind a branch (past the end the last token's are read again and not counted).
 template <typename TA>
-__device__ inline float rounded(float v) {
-  return to_float(from_float<TA>(v));
+__device__ inline float sum_over_tokens(const TA* cache, const int* __restrict__ table, int first, int last, int page, int G,
+                                        int g, size_t head_size, size_t offset, int apart) {
+  float sum = 0.f;
+  for (int j0 = first; j0 < last; j0 += 16) {
+    int pages[16];
+    TA got[16];
+#pragma unroll
+    for (int u = 0; u < 16; ++u) pages[u] = table[min(j0 + u, last - 1) / page];
+#pragma unroll
+    for (int u = 0; u < 16; ++u) {
+      const int slot = min(j0 + u, last - 1) % page;
+      got[u] = cache[((size_t)max(pages[u], 0) * G + g) * head_size + offset + (size_t)slot * apart];
+    }
+#pragma unroll
+    for (int u = 0; u < 16; ++u) sum += (j0 + u < last && pages[u] >= 0) ? to_float(got[u]) : 0.f;
+  }
+  return sum;
 }
 
 template <typename TA>
@@ -142,12 +160,8 @@ __global__ void __launch_bounds__(256) turn_prepare_kernel(
       const TA key = from_float<TA>(turned(x, add, e));
       k_cache[(((size_t)pg * G + g) * page + off) * dim + e] = key;
       if (run_page >= 0) {
-        float sum = 0.f;
-        for (int j = pos - runs.pool + 1; j < pos; ++j) {
-          const int from = table[j / page];
-          sum += from < 0 ? 0.f : to_float(k_cache[(((size_t)from * G + g) * page + j % page) * dim + e]);
-        }
-        sum += to_float(key);
+        const float sum = sum_over_tokens<TA>(k_cache, table, pos - runs.pool + 1, pos, page, G, g, (size_t)page * dim, e, dim) +
+                          to_float(key);
         ((TA*)runs.k)[(((size_t)run_page * G + g) * page + run_off) * dim + e] = from_float<TA>(sum / (float)runs.pool);
       }
     }
@@ -157,12 +171,9 @@ __global__ void __launch_bounds__(256) turn_prepare_kernel(
       const TA value = from_float<TA>(y[e] + (add_v ? add_v[e] : 0.f));
       v_cache[(((size_t)pg * G + g) * vdim + e) * page + off] = value;
       if (run_page >= 0) {
-        float sum = 0.f;
-        for (int j = pos - runs.pool + 1; j < pos; ++j) {
-          const int from = table[j / page];
-          sum += from < 0 ? 0.f : to_float(v_cache[(((size_t)from * G + g) * vdim + e) * page + j % page]);
-        }
-        sum += to_float(value);
+        const float sum = sum_over_tokens<TA>(v_cache, table, pos - runs.pool + 1, pos, page, G, g, (size_t)page * vdim,
+                                              (size_t)e * page, 1) +
+                          to_float(value);
         ((TA*)runs.v)[(((size_t)run_page * G + g) * vdim + e) * page + run_off] = from_float<TA>(sum / (float)runs.pool);
       }
     }
@@ -212,13 +223,9 @@ __global__ void __launch_bounds__(256) pool_runs_kernel(const TA* __restrict__ k
   for (int e = threadIdx.x; e < dim + vdim; e += blockDim.x) {
     const bool key = e < dim;
     const int c = key ? e : e - dim;
-    float sum = 0.f;
-    for (int j = r * pool; j < (r + 1) * pool; ++j) {
-      const int pg = j / page < table_width ? table[j / page] : -1;
-      if (pg < 0) continue;
-      const size_t head = (size_t)pg * G + g;
-      sum += key ? to_float(k_cache[(head * page + j % page) * dim + c]) : to_float(v_cache[(head * vdim + c) * page + j % page]);
-    }
+    const float sum = key ? sum_over_tokens<TA>(k_cache, table, r * pool, (r + 1) * pool, page, G, g, (size_t)page * dim, c, dim)
+                          : sum_over_tokens<TA>(v_cache, table, r * pool, (r + 1) * pool, page, G, g, (size_t)page * vdim,
+                                                (size_t)c * page, 1);
     const size_t head = (size_t)run_page * G + g;
     const TA mean = from_float<TA>(sum / (float)pool);
     if (key)
