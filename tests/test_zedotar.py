@@ -107,6 +107,11 @@ ODD = _model(53, 40, [
 # the matrix memory alone, over several tiles of columns and slices of rows
 MEMORY = _model(97, 64, [_layer(_mlstm(2, 130, 150, cap=8.0), 96), _layer(_mlstm(4, 16, 64), 48)], cap=12.0)
 CONFIGS = {"mixed": MIXED, "cores": CORES, "odd": ODD, "memory": MEMORY}
+# in bfloat16 heads of two or three numbers, whose root mean square is divided out, move by more than any bound
+# on rounding; the same layers with more numbers in them
+ROUNDED = {"odd": dict(ODD, layers=[
+    _layer(_attention(3, 1, 10, 14, size=9, pool=1, rot=_rot(4)), 18), _layer(_mlstm(1, 13, 70, cap=2.0), 22),
+    _layer(_sigmoid(1, 1, 26, 1), None), _layer(_attention(2, 2, 6, 30, size=5), 10), _layer(_attention(1, 1, 7, 23), 14)])}
 
 
 def _write(folder, data, seed=5, std=0.2, keep=3.0, apart=2.0):
@@ -131,9 +136,12 @@ def folder(request, tmp_path_factory):
 
 @pytest.fixture(scope="module", params=sorted(CONFIGS))
 def folders(request, tmp_path_factory):
-    """{dtype: folder}: smaller weights for bfloat16, so that rounding alone stays well inside the bound."""
+    """{dtype: folder}: for bfloat16 smaller weights, and sigmoid weights that are small for all but a few keys (sums
+    that hundreds of keys enter undivided make every later rounding count), so that rounding alone stays well
+    inside the bound."""
     return {"float32": _write(tmp_path_factory.mktemp(request.param), CONFIGS[request.param]),
-            "bfloat16": _write(tmp_path_factory.mktemp(request.param + "_bf16"), CONFIGS[request.param], std=0.1)}
+            "bfloat16": _write(tmp_path_factory.mktemp(request.param + "_bf16"), ROUNDED.get(request.param, CONFIGS[request.param]),
+                               std=0.05, apart=4.0)}
 
 
 def _truth(folder, requests, dtype=torch.float64):
@@ -679,7 +687,7 @@ def test_memory_kernels_against_plain(dtype, H, d, dv, cap):
         state = torch.zeros((5, ops.mlstm_state_numbers(H, d, dv)), dtype=torch.float32).cuda()
         slots = torch.tensor([3, 0, 4], dtype=torch.int32).cuda()
         at = [0, 0, 0]
-        for cut in ([64, 9, 1], [1, 1, 1], [8, 2, 63], [63, 0, 65], [1, 1, 0], [60, 54, 1], [3, 0, 0]):
+        for cut in ([64, 9, 1], [1, 1, 1], [8, 2, 63], [63, 0, 65], [1, 1, 0], [60, 54, 0], [3, 0, 0]):
             rows = torch.cat([data[b][0][at[b]:at[b] + n] for b, n in enumerate(cut)]).cuda()
             cu = torch.tensor([0] + list(np.cumsum(cut)), dtype=torch.int32).cuda()
             got = ops.mlstm_scan(rows, H, d, dv, cap, ib, fb, norm, 1e-5, 1e-6, state, slots, cu, dtype, max_q_len=max(cut))
@@ -755,35 +763,49 @@ def test_long_decoding_and_first_tokens(folders):
         assert _off(run_trace(runner, steps), want, dtype) <= 1.0
 
 
-@pytest.mark.gpu
-@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-def test_a_far_key_and_a_far_run_carry_the_last_row(tmp_path, dtype):
-    """A prompt of 600 tokens in which one early token returns at the end, with queries made from the keys'
-    matrices and no rotation: the last rows lean on that token's key (sigmoid attention) and on its run's mean
-    (pooled attention), hundreds of positions back, in a whole prompt, in portions, and decoded."""
-    layers = [_layer(_attention(4, 2, 64, 64, size=40, pool=4, scale=0.6), 96), _layer(_sigmoid(4, 2, 64, 1, scale=0.6), 64)]
-    data = _model(131, 128, layers, cap=20.0)
-    folder = _write(tmp_path / "m", data, std=0.1, apart=9.0)
+def _far_model(folder, kind):
+    """One layer of either attention. Queries are the keys' negatives, and the embedding of one token (`asks`) is
+    another's (`holds`) negative: a query of the one stands on the keys of the other. Nothing turns. A prompt in
+    which a whole run of the one that holds stands early and the one that asks near the end."""
+    layer = (_attention(4, 2, 64, 64, size=40, pool=4, scale=0.25) if kind == "attention" else _sigmoid(4, 2, 64, 1, scale=0.25))
+    data = _model(131, 128, [_layer(layer, 96)], cap=20.0)
+    folder = _write(folder, data, std=0.1, apart=9.0)
     path = os.path.join(folder, "model.safetensors")
     tensors = load_file(path)
-    for i in range(2):
-        p = "l%d.mix." % i
-        k = tensors[p + "k"].view(2, 64, -1)
-        tensors[p + "q"] = k.repeat_interleave(2, dim=0).reshape(256, -1).contiguous()
-        tensors[p + "q.b"] = torch.zeros_like(tensors[p + "q.b"])
-        tensors[p + "k.b"] = torch.zeros_like(tensors[p + "k.b"])
-        if i:
-            tensors[p + "q.conv"] = torch.ones_like(tensors[p + "q.conv"])
-            tensors[p + "k.conv"] = torch.ones_like(tensors[p + "k.conv"])
+    p = "l0.mix."
+    k = tensors[p + "k"].view(2, 64, -1)
+    tensors[p + "q"] = -k.repeat_interleave(2, dim=0).reshape(256, -1).contiguous()
+    for name in ("q.b", "k.b"):
+        tensors[p + name] = torch.zeros_like(tensors[p + name])
+    if kind != "attention":
+        for name in ("q.conv", "k.conv"):
+            tensors[p + name] = torch.ones_like(tensors[p + name])
+    asks, holds = data["vocab"] - 1, data["vocab"] - 2
+    tensors["embed"][asks] = -tensors["embed"][holds]
     save_file(tensors, path, metadata={"format": "pt"})
-    rare = data["vocab"] - 1
-    tokens = [t if t != rare else 0 for t in random_tokens(600, data["vocab"], 31)]
-    tokens[37] = tokens[-2] = rare
-    config, w, want = _truth(folder, {"far": tokens})
-    cut = list(tokens)
-    cut[37] = 3
-    other = plain.logits_of_sequence(config, w, cut)
-    assert float((other[-2] - want["far"][-2]).abs().max()) > 0.15 * float(want["far"][-2].std())
+    tokens = [min(t, holds - 1) for t in random_tokens(600, data["vocab"], 31)]
+    tokens[36:40] = [holds] * 4
+    tokens[-2] = asks
+    return folder, tokens
+
+
+@pytest.mark.parametrize("kind", ["attention", "attention_2"])
+def test_the_far_model_leans_on_its_far_run(tmp_path, kind):
+    """The truth of the test below: without the early run the row that asks is another one."""
+    folder, tokens = _far_model(tmp_path / "m", kind)
+    _, _, want = _truth(folder, {"far": tokens, "cut": tokens[:36] + [3, 5, 7, 11] + tokens[40:]})
+    a, b = want["far"][-2], want["cut"][-2]
+    assert float((a - b).pow(2).mean().sqrt()) > 0.3 * float(a.std())
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("kind", ["attention", "attention_2"])
+def test_a_far_run_carries_the_last_row(tmp_path, dtype, kind):
+    """The row that asks leans on a run's mean (pooled attention) or on keys (sigmoid attention) hundreds of
+    positions back, in a whole prompt, in portions, and decoded."""
+    folder, tokens = _far_model(tmp_path / "m", kind)
+    _, _, want = _truth(folder, {"far": tokens})
     for steps in (trace_whole({"far": tokens}), trace_tail_decoded({"far": tokens}, tail=4),
                   trace_portions({"far": tokens}, sizes=(130, 37, 2, 261, 64, 3))):
         runner = load_runner(folder, dtype=dtype, device="cuda", page_size=16, max_tokens=608, max_requests=1)
