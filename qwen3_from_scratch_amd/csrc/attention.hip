@@ -778,8 +778,15 @@ __device__ __forceinline__ void store_new_key_value(const bf16_t* row, int Hq, i
   }
 }
 
+// (with two sources the kernel would take a few registers more than leave room for two blocks a CU, which
+// takes a third longer from two splits on)
+#ifdef Q3_POOLED
+#define Q3_DECODE_WAVES __attribute__((amdgpu_waves_per_eu(2)))
+#else
+#define Q3_DECODE_WAVES
+#endif
 template <int D, bool PREP, typename W, bool AHEAD>
-__global__ __launch_bounds__(256) void attn_decode_kernel(
+__global__ __launch_bounds__(256) Q3_DECODE_WAVES void attn_decode_kernel(
     const bf16_t* __restrict__ q, int q_stride, bf16_t* __restrict__ out, const bf16_t* __restrict__ k_cache,
     const bf16_t* __restrict__ v_cache, int num_pages, const int* __restrict__ block_table, int bt_stride,
     const int* __restrict__ cu_q, const int* __restrict__ kv_lens, int Hq, int Hkv, int page, score_scale_t scale_log2,
