@@ -1,5 +1,6 @@
 // Embedding row gather and the gated activations (SwiGLU and its gelu forms).
 #include "common.h"
+#include "gates.h"
 
 // out[t, :] = float(table[ids[t], :]) * scale. An id outside the table gives a row of
 // zeros (the host refuses such ids before launching; this only keeps the
@@ -36,16 +37,8 @@ extern "C" int q3_soft_cap(float* x, long n, float cap, hipStream_t stream) {
 }
 
 // out[t, j] = act(gate[t, j]) * up[t, j] for rows that interleave the two:
-// gate_up[t, 2j] = gate[t, j], gate_up[t, 2j + 1] = up[t, j]. ACT 0: silu(g) = g / (1 + exp(-g));
-// 1: the tanh form of gelu, 0.5 g (1 + tanh(sqrt(2/pi) (g + 0.044715 g^3))); 2: the exact gelu,
-// 0.5 g (1 + erf(g / sqrt 2)). Evaluated in float32 and rounded once.
-template <int ACT>
-__device__ inline float gate_value(float g) {
-  if (ACT == 0) return g / (1.f + expf(-g));
-  if (ACT == 1) return 0.5f * g * (1.f + tanhf(0.79788456080286536f * (g + 0.044715f * g * g * g)));
-  return 0.5f * g * (1.f + erff(g * 0.70710678118654752f));
-}
-
+// gate_up[t, 2j] = gate[t, j], gate_up[t, 2j + 1] = up[t, j]; the activations ACT are gate_value's.
+// Evaluated in float32 and rounded once.
 template <typename T, int ACT>
 __global__ void swiglu_kernel(const T* __restrict__ gate_up, T* __restrict__ out, int I) {
   const int t = blockIdx.y;

@@ -1,5 +1,6 @@
 // out = x @ weight^T with float32 accumulation: x (M, K), weight (N, K), out (M, N).
 #include "common.h"
+#include "gates.h"
 
 // ---------------------------------------------------------------------------
 // float32: plain fused multiply-adds, no matrix-core mode of reduced precision.
@@ -139,7 +140,10 @@ union Pack16 {
 // * `row_sums`: the rows of x are such weighted, unscaled rows. The block adds the partial sums
 //   (`sums_rows` slabs of 16 rows) in a fixed order and multiplies row m of the product by
 //   rsqrt(sum_m * inv_width + eps) before any other epilogue: (x / rms) @ W^T = (x @ W^T) / rms.
-enum { EPI_PLAIN = 0, EPI_SWIGLU = 1, EPI_RESIDUAL = 2 };
+// EPI_GELU: as EPI_SWIGLU with the tanh form of gelu in silu's place.
+enum { EPI_PLAIN = 0, EPI_SWIGLU = 1, EPI_RESIDUAL = 2, EPI_GELU = 3 };
+#define EPI_IS_GATED(EPI) ((EPI) == EPI_SWIGLU || (EPI) == EPI_GELU)
+#define EPI_GATE_ACT(EPI) ((EPI) == EPI_GELU ? 1 : 0)
 
 struct SkinnyFusion {
   const float* row_sums;
@@ -182,7 +186,7 @@ __global__ __launch_bounds__(1024) void gemm_skinny_kernel(const bf16_t* __restr
   if constexpr (GROUPS) {
     M = min(16, M - row0);
     x += (size_t)row0 * K;
-    out += (size_t)row0 * (EPI == EPI_SWIGLU ? N / 2 : N);
+    out += (size_t)row0 * (EPI_IS_GATED(EPI) ? N / 2 : N);
     if (EPI == EPI_RESIDUAL) fu.residual += (size_t)row0 * N;
   }
   const int slab = blockIdx.x * sw + wave / kw;
@@ -307,14 +311,14 @@ __global__ __launch_bounds__(1024) void gemm_skinny_kernel(const bf16_t* __restr
     return;
   }
   if (col >= M) return;
-  if constexpr (EPI == EPI_SWIGLU) {
+  if constexpr (EPI_IS_GATED(EPI)) {
     OUT* o = out + (size_t)col * (N / 2) + n / 2;  // n is even: pairs (n, n + 1) and (n + 2, n + 3)
 #pragma unroll
     for (int j = 0; j < 2; ++j) {
       if (n + 2 * j + 1 < N) {
         // the separate kernel sees gate and up rounded to the activation dtype: do the same
         const float g = to_float(from_float<OUT>(acc[2 * j])), u = to_float(from_float<OUT>(acc[2 * j + 1]));
-        o[j] = from_float<OUT>(g / (1.f + expf(-g)) * u);
+        o[j] = from_float<OUT>(gate_value<EPI_GATE_ACT(EPI)>(g) * u);
       }
     }
     return;
@@ -356,7 +360,7 @@ __global__ __launch_bounds__(512, 4) void gemm_skinny_pair_kernel(const bf16_t* 
                                                                const bf16_t* __restrict__ w, OUT* __restrict__ out,
                                                                int M, int N, int K, int kw, int k_per_wave,
                                                                SkinnyFusion fu) {
-  static_assert(EPI == EPI_PLAIN || EPI == EPI_SWIGLU, "plain and SwiGLU epilogues");
+  static_assert(EPI == EPI_PLAIN || EPI_IS_GATED(EPI), "plain and gated epilogues");
   extern __shared__ float red[];  // [waves][2][64][4], then [waves][16] for the rows' sums
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int col = lane & 15, grp = lane >> 4;
@@ -446,13 +450,13 @@ __global__ __launch_bounds__(512, 4) void gemm_skinny_pair_kernel(const bf16_t* 
   for (int h = 0; h < 2; ++h) {
     if (h == 1 && !second) break;
     const int n = (slab0 + h) * 16 + 4 * grp;
-    if constexpr (EPI == EPI_SWIGLU) {
+    if constexpr (EPI_IS_GATED(EPI)) {
       OUT* o = out + (size_t)col * (N / 2) + n / 2;
 #pragma unroll
       for (int j = 0; j < 2; ++j) {
         if (n + 2 * j + 1 < N) {
           const float g = to_float(from_float<OUT>(acc[h][2 * j])), u = to_float(from_float<OUT>(acc[h][2 * j + 1]));
-          o[j] = from_float<OUT>(g / (1.f + expf(-g)) * u);
+          o[j] = from_float<OUT>(gate_value<EPI_GATE_ACT(EPI)>(g) * u);
         }
       }
     } else {
@@ -495,7 +499,7 @@ static int launch_skinny(const void* x, const void* w, void* out, int M, int N, 
   int k_per_wave = (K + kw - 1) / kw;
   k_per_wave = (k_per_wave + step - 1) / step * step;
   const int groups = (M + 15) / 16;   // of 16 rows of x: one, or a few for a small weight (q3_linear_tiled)
-  if constexpr (TILED && (EPI == EPI_PLAIN || EPI == EPI_SWIGLU)) {
+  if constexpr (TILED && (EPI == EPI_PLAIN || EPI_IS_GATED(EPI))) {
     if (slabs >= SKINNY_PAIR_SLABS && sw == 1 && M > 8 && groups == 1) {
       const size_t pair_smem = (size_t)kw * (2 * 64 * 4 + 16) * sizeof(float);
       hipLaunchKernelGGL((gemm_skinny_pair_kernel<OUT, EPI, SCALED>), dim3((slabs + 1) / 2), dim3(64 * kw), pair_smem,
@@ -629,7 +633,7 @@ extern "C" int q3_linear_swiglu(const void* x, const void* weight, void* out, in
 
 // The same products from the tile-ordered copy of the weight (see gemm_skinny_kernel):
 // x (M, K) bfloat16, K a multiple of 32. `epilogue`: 0 output (M, N) in `out_dtype`;
-// 1 the activation (output (M, N / 2) bfloat16); 2 the residual addition and the next norm's
+// 1 (or 3) the activation, silu (or the tanh form of gelu) (output (M, N / 2) bfloat16); 2 the residual addition and the next norm's
 // preparation (N a multiple of 16; `residual` (M, N) float32 updated in place, `norm_weight`
 // (N,) of `norm_w_dtype`, output (M, N) bfloat16 = residual * norm_weight, `sums_out`
 // (N / 16, sums_stride) float32). `row_sums` (sums_rows, sums_stride) float32, if not null, says that
@@ -662,6 +666,11 @@ extern "C" int q3_linear_tiled(const void* x, const void* weight_tiled, void* ou
     if (N % 2 || out_dtype != Q3_BF16) return Q3_ERR_BAD_ARGUMENT;
     return row_sums ? launch_skinny<bf16_t, EPI_SWIGLU, true, true>(x, weight_tiled, out, M, N, K, stream, fu)
                     : launch_skinny<bf16_t, EPI_SWIGLU, true>(x, weight_tiled, out, M, N, K, stream, fu);
+  }
+  if (epilogue == EPI_GELU) {
+    if (N % 2 || out_dtype != Q3_BF16) return Q3_ERR_BAD_ARGUMENT;
+    return row_sums ? launch_skinny<bf16_t, EPI_GELU, true, true>(x, weight_tiled, out, M, N, K, stream, fu)
+                    : launch_skinny<bf16_t, EPI_GELU, true>(x, weight_tiled, out, M, N, K, stream, fu);
   }
   if (epilogue == EPI_RESIDUAL) {
     if (row_sums || N % 16 || out_dtype != Q3_BF16 || !residual || !norm_weight || !sums_out ||

@@ -50,6 +50,7 @@
 #pragma once
 
 #include "common.h"
+#include "gates.h"
 
 namespace tiles {
 
@@ -61,7 +62,8 @@ union Frag {
   bf16x8_t v;
 };
 
-enum { EPI_PLAIN = 0, EPI_SWIGLU = 1 };
+// EPI_GELU (store_tile alone): as EPI_SWIGLU with the tanh form of gelu in silu's place.
+enum { EPI_PLAIN = 0, EPI_SWIGLU = 1, EPI_GELU = 2 };
 
 constexpr int BK = 64;          // k per step: two matrix instructions deep
 constexpr int ROW_BYTES = 128;  // a row of a slice
@@ -150,7 +152,7 @@ __device__ inline void store_tile(const f32x4_t (&acc)[MI][NJ], OUT* __restrict_
       const int n = n_base + 16 * j + 4 * grp;
       if (n >= N) continue;
       const f32x4_t c = acc[i][j] * r;
-      if constexpr (EPI == EPI_SWIGLU) {
+      if constexpr (EPI != EPI_PLAIN) {
         // rows of w interleave gate and up (row 2 i gate, row 2 i + 1 up); both are rounded to
         // the activation type first, as a separate activation kernel would have read them
         OUT* o = out + (size_t)m * (N / 2) + n / 2;
@@ -158,7 +160,7 @@ __device__ inline void store_tile(const f32x4_t (&acc)[MI][NJ], OUT* __restrict_
         for (int p = 0; p < 2; ++p) {
           if (n + 2 * p + 1 < N) {
             const float g = to_float(from_float<OUT>(c[2 * p])), u = to_float(from_float<OUT>(c[2 * p + 1]));
-            o[p] = from_float<OUT>(g / (1.f + expf(-g)) * u);
+            o[p] = from_float<OUT>(gate_value<EPI == EPI_GELU ? 1 : 0>(g) * u);
           }
         }
       } else {

@@ -650,7 +650,7 @@ extern "C" int q3_tiles_residual(const void* x, const void* w, int M, int N, int
 
 // A product of 17 to 96 rows (and a gate/up product of 9 to 16) by the weight-streaming kernel of gemm_stream.h, from the tile-ordered copy `wt` of
 // the weight (N, K): out (M, N) in `out_dtype` (`epilogue` 0) or, the weight's rows interleaving gate and up,
-// out (M, N / 2) bfloat16 = silu(gate) * up (`epilogue` 1). With `sums` the rows of x still lack their norm's
+// out (M, N / 2) bfloat16 = silu(gate) * up (`epilogue` 1) or gelu(gate) * up, its tanh form (2). With `sums` the rows of x still lack their norm's
 // division, as for q3_tiles_scaled. Returns Q3_DECLINED, and has done nothing, where another kernel is the way:
 // the caller has asked for the library's or the tiled kernel's products alone, the tuner is on (it times those),
 // the size is not the kernel's, the weight is so small that other kernels serve these rows better, or its slabs
@@ -684,13 +684,13 @@ extern "C" int q3_stream_product(const void* x, const void* wt, void* out, int M
                                  int epilogue, const float* sums, int chunks, int sums_stride, float eps, int width,
                                  void* stream_) {
   if (!x || !wt || !out || M < 1 || N < 1 || K < 1) return Q3_ERR_BAD_ARGUMENT;
-  const bool swiglu = epilogue == tiles::EPI_SWIGLU;
-  if (!swiglu && epilogue != tiles::EPI_PLAIN) return Q3_ERR_BAD_ARGUMENT;
-  if (swiglu ? out_dtype != Q3_BF16 : (out_dtype != Q3_BF16 && out_dtype != Q3_F32)) return Q3_ERR_BAD_ARGUMENT;
+  const bool gated = epilogue == tiles::EPI_SWIGLU || epilogue == tiles::EPI_GELU;
+  if (!gated && epilogue != tiles::EPI_PLAIN) return Q3_ERR_BAD_ARGUMENT;
+  if (gated ? out_dtype != Q3_BF16 : (out_dtype != Q3_BF16 && out_dtype != Q3_F32)) return Q3_ERR_BAD_ARGUMENT;
   if (sums && (chunks < 1 || sums_stride < M || width != K)) return Q3_ERR_BAD_ARGUMENT;
   hipStream_t stream = (hipStream_t)stream_;
   std::lock_guard<std::mutex> hold(g_lock);
-  const int ws = stream_plan_locked(M, N, K, swiglu);
+  const int ws = stream_plan_locked(M, N, K, gated);
   if (!ws) return Q3_DECLINED;
   tiles::RowScale scale;
   if (sums) {
@@ -700,7 +700,9 @@ extern "C" int q3_stream_product(const void* x, const void* wt, void* out, int M
     scale.eps = eps;
     scale.inv_width = 1.f / (float)width;
   }
-  if (swiglu) return stream::launch<bf16_t, tiles::EPI_SWIGLU>(ws, x, wt, out, M, N, K, stream, scale);
+  if (epilogue == tiles::EPI_SWIGLU)
+    return stream::launch<bf16_t, tiles::EPI_SWIGLU>(ws, x, wt, out, M, N, K, stream, scale);
+  if (epilogue == tiles::EPI_GELU) return stream::launch<bf16_t, tiles::EPI_GELU>(ws, x, wt, out, M, N, K, stream, scale);
   if (out_dtype == Q3_F32) return stream::launch<float, tiles::EPI_PLAIN>(ws, x, wt, out, M, N, K, stream, scale);
   return stream::launch<bf16_t, tiles::EPI_PLAIN>(ws, x, wt, out, M, N, K, stream, scale);
 }

@@ -1786,8 +1786,9 @@ def stream_plan(M, N, K, swiglu=False):
     return int(ws) if ws else None
 
 
-def _stream_product(x, weight, tiled, out, swiglu, unscaled, what):
-    """The product by the weight-streaming kernel, if it takes it: True if `out` is written."""
+def _stream_product(x, weight, tiled, out, swiglu, unscaled, what, kind="silu"):
+    """The product by the weight-streaming kernel, if it takes it: True if `out` is written. `swiglu`: a gated
+    unit in its epilogue, with the activation `kind` ("silu" or "gelu_tanh")."""
     M, K = x.shape
     N = weight.shape[0]
     least = STREAM_ROWS_LEAST if swiglu else FEW_ROWS + 1
@@ -1802,8 +1803,8 @@ def _stream_product(x, weight, tiled, out, swiglu, unscaled, what):
         _need(width == K, "the rows' width must be the product's inner size")
         chunks, stride = sums.shape
     status = _matmul().q3_stream_product(
-        _ptr(x), _ptr(tiled), _ptr(out), M, N, K, _DT[out.dtype], 1 if swiglu else 0, _ptr(sums), chunks, stride,
-        ctypes.c_float(eps), int(width), _stream())
+        _ptr(x), _ptr(tiled), _ptr(out), M, N, K, _DT[out.dtype], (1 + GATE_KINDS[kind]) if swiglu else 0, _ptr(sums),
+        chunks, stride, ctypes.c_float(eps), int(width), _stream())
     if status == _DECLINED:
         return False
     _check(status, what)
@@ -1884,11 +1885,18 @@ def linear_plain(x, weight, out):
     return out
 
 
-def linear_swiglu(x, weight, tiled=None, unscaled=None):
-    """swiglu(x @ weight^T) for a weight whose rows interleave gate and up (row 2i gate's, row
-    2i + 1 up's): (M, K) x (2I, K) -> (M, I). With few bfloat16 rows the activation is the
-    product kernel's epilogue; otherwise it is the product followed by `swiglu`.
-    `unscaled`: as for `linear`."""
+_FEW_ROW_EPILOGUES = {"silu": 1, "gelu_tanh": 3}      # the few-row kernel's codes of its gated epilogues
+
+
+def linear_swiglu(x, weight, tiled=None, unscaled=None, kind="silu"):
+    """act(gate) * up of x @ weight^T for a weight whose rows interleave gate and up (row 2i gate's, row
+    2i + 1 up's): (M, K) x (2I, K) -> (M, I); `kind` names the activation (`GATE_KINDS`). With few
+    bfloat16 rows the activation is the product kernel's epilogue (silu in every kernel for up to 128 rows, the
+    tanh form of gelu in the few-row and the weight-streaming kernel, the exact gelu nowhere); otherwise
+    it is the product followed by `gated_act`, with the same bits. `unscaled`: as for `linear`."""
+    _need(kind in GATE_KINDS, "kind is one of %s" % ", ".join(sorted(GATE_KINDS)))
+    if kind == "gelu_erf":
+        return gated_act(linear(x, weight, tiled=tiled, unscaled=unscaled), kind)
     _dev(x, weight)
     _need(x.dim() == 2 and weight.dim() == 2 and x.shape[1] == weight.shape[1] and weight.shape[0] % 2 == 0,
           "x (M, K) and weight (2I, K)")
@@ -1900,20 +1908,22 @@ def linear_swiglu(x, weight, tiled=None, unscaled=None):
         if unscaled is not None:
             _need(unscaled[0].dim() == 2 and unscaled[0].shape[1] == sums_stride(M), "row sums (P, M rounded up to 16)")
         out = torch.empty((M, N // 2), dtype=x.dtype, device=x.device)
-        if _stream_product(x, weight, tiled, out, True, unscaled, "linear_swiglu"):
+        if _stream_product(x, weight, tiled, out, True, unscaled, "linear_swiglu", kind):
             return out
     if M and x.dtype == torch.bfloat16 and _tiled_ok(tiled, weight, M):
         out = torch.empty((M, N // 2), dtype=x.dtype, device=x.device)
         sums, sums_rows, eps, width, stride = _row_sums_args(unscaled, M, K)
         _check(library("gemm").q3_linear_tiled(
-            _ptr(x), _ptr(tiled), _ptr(out), M, N, K, 1, 1, sums, sums_rows, eps, width,
+            _ptr(x), _ptr(tiled), _ptr(out), M, N, K, 1, _FEW_ROW_EPILOGUES[kind], sums, sums_rows, eps, width,
             None, None, 0, None, stride, _stream()), "linear_swiglu")
         return out
     if M and x.dtype == torch.bfloat16 and tiled is not None and FEW_ROWS < M <= STREAM_ROWS_MOST \
             and (unscaled is None or fused_rows_take(weight, M)):
         out = torch.empty((M, N // 2), dtype=x.dtype, device=x.device)
-        if _stream_product(x, weight, tiled, out, True, unscaled, "linear_swiglu"):
+        if _stream_product(x, weight, tiled, out, True, unscaled, "linear_swiglu", kind):
             return out
+    if kind != "silu":
+        return gated_act(linear(x, weight, tiled=tiled, unscaled=unscaled), kind)
     if unscaled is not None and x.dtype == torch.bfloat16 and fused_rows_take(weight, M):
         out = torch.empty((M, N // 2), dtype=x.dtype, device=x.device)
         return _tiles_scaled(x, weight, out, unscaled, True, "linear_swiglu")

@@ -16,8 +16,8 @@ class SwiGLU(Part):
     that one product feeds the activation, which for few rows is the product
     kernel's epilogue (the reference's fused variant concatenates them,
     feedback.py:52-54). `activation`: what the gate passes, "silu" or one of the other kinds of
-    `ops.GATE_KINDS` (the tanh form of gelu, the exact gelu), which run as the plain product and an
-    activation kernel behind it."""
+    `ops.GATE_KINDS` (the tanh form of gelu, the exact gelu); where a product's kernel does not carry it,
+    it is an activation kernel behind the product (`ops.linear_swiglu`)."""
 
     graph_safe = True
     feeds_sink = True
@@ -54,10 +54,7 @@ class SwiGLU(Part):
         return self.gate_up is not None and self.gate_up.fuses
 
     def forward(self, x, batch=None, sink=None):
-        if self.activation == "silu":
-            h = self.gate_up.forward_swiglu(x)
-        else:
-            h = ops.gated_act(self.gate_up.forward(x), self.activation)
+        h = self.gate_up.forward_swiglu(x, self.activation)
         return self.down.forward(h) if sink is None else self.down.forward_into(h, sink)
 
 

@@ -39,11 +39,11 @@ class LinearWeight:
             return ops.linear(x.values, self.weight, out_dtype=out_dtype, tiled=self.tiled, unscaled=x.scale_args())
         return ops.linear(x, self.weight, out_dtype=out_dtype, tiled=self.tiled)
 
-    def forward_swiglu(self, x):
-        """swiglu(x @ W^T) for a W whose rows interleave gate and up."""
+    def forward_swiglu(self, x, kind="silu"):
+        """act(gate) * up of x @ W^T for a W whose rows interleave gate and up; `kind` names the activation."""
         if isinstance(x, UnscaledRows):
-            return ops.linear_swiglu(x.values, self.weight, tiled=self.tiled, unscaled=x.scale_args())
-        return ops.linear_swiglu(x, self.weight, tiled=self.tiled)
+            return ops.linear_swiglu(x.values, self.weight, tiled=self.tiled, unscaled=x.scale_args(), kind=kind)
+        return ops.linear_swiglu(x, self.weight, tiled=self.tiled, kind=kind)
 
     @property
     def fuses(self):

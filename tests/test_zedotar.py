@@ -704,6 +704,28 @@ def test_memory_kernels_against_plain(dtype, H, d, dv, cap):
 
 
 @pytest.mark.gpu
+@pytest.mark.parametrize("M,I,K", [(1, 96, 64), (7, 200, 128), (16, 6144, 2048), (12, 6144, 2048), (48, 512, 256),
+                                   (64, 6144, 2048), (90, 6144, 2048), (130, 256, 128), (5, 33, 40)])
+def test_gelu_in_a_products_epilogue(M, I, K):
+    """The same bits as the product followed by the activation's kernel, also for rows that still lack their
+    norm's division; sizes of the few-row kernel (one slab and two a block), of the weight-streaming one, and
+    of neither."""
+    from qwen3_from_scratch_amd import ops
+
+    x, w = _rand((M, K), 1, torch.bfloat16, 2.0), _rand((2 * I, K), 2, torch.bfloat16, K ** -0.5)
+    tiled = ops.tile_weight(w)
+    for unscaled in (None, (torch.full((1, ops.sums_stride(M)), 3.0 * K).cuda(), 1e-5, K)):
+        if unscaled is not None and not (tiled is not None and (M <= ops.few_rows_limit(w) or ops.fused_rows_take(w, M))):
+            continue
+        for kind in ("gelu_tanh", "silu", "gelu_erf"):
+            got = ops.linear_swiglu(x, w, tiled=tiled, unscaled=unscaled, kind=kind)
+            want = ops.gated_act(ops.linear(x, w, tiled=tiled, unscaled=unscaled), kind)
+            close = (got.float() - want.float()).abs().max() <= 2e-2 * max(1.0, float(want.float().abs().max()))
+            # the kernels for a gated product and for a plain one may add up a row's terms in different orders
+            assert bool(close) and float((got != want).float().mean()) < 0.2, kind
+
+
+@pytest.mark.gpu
 def test_soft_cap_kernel():
     from qwen3_from_scratch_amd import ops
 

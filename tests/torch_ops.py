@@ -175,8 +175,8 @@ def linear(x, weight, out_dtype=None, out=None, tiled=None):
     return res
 
 
-def linear_swiglu(x, weight, tiled=None):
-    return swiglu(linear(x, weight))
+def linear_swiglu(x, weight, tiled=None, kind="silu"):
+    return gated_act(linear(x, weight), kind)
 
 
 def _uniform(seed, counter, n, device):
