@@ -836,7 +836,7 @@ def zedotar_layers(W, ff, window, pool, kinds):
     """Layers of real proportions: both attentions in heads of 128, four query heads a key head, half of
     each head turned; the matrix memory in heads of 128 with values of 256, as the retention it stands
     beside."""
-    half = {"dims": 64, "base": 500000.0}
+    half = {"dims": 64, "base": 10000.0}
     mixers = {
         "attention": {"heads": W // 128, "kv_heads": W // 512, "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
                       "mask": {"size": window, "pool": pool}, "rot": half},
@@ -872,7 +872,7 @@ def zedotar(args, sync):
             kinds = (kinds * args.layers)[:args.layers]
         listed = zedotar_layers(W, ff, window, pool, kinds)
         new = ZedotarConfig.from_dict({"architecture": "Zedotar", "vocab": vocab, "width": W, "norm": {"eps": 1e-5},
-                                       "logit_softcap": 30.0, "layers": listed})
+                                       "logit_softcap": 50.0, "layers": listed})
         other = SurasunConfig.from_dict({"architecture": "Surasun", "vocab": vocab, "width": W, "norm": {"eps": 1e-5},
                                          "residual_mult": 1.0,
                                          "layers": surasun_layers(W, ff, [("mamba2" if k == "mlstm" else "parallel", True)
