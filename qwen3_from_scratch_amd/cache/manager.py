@@ -6,7 +6,8 @@ window of them form another, and so on. A group has a page pool of
 its own and, per request, one block table that serves all its layers: page p of
 a group exists once in each of the group's layers' planes. A request's pages
 go back to the pool when it ends, and, in a windowed group, as soon as every
-position a page covers lies behind the window. Tensors that grow by one element
+position a page covers lies behind the window; pages of first tokens that stay visible are kept. A group
+whose layers see chunks of the sequence gives a chunk's pages back when the next chunk begins. Tensors that grow by one element
 per complete run of tokens form groups of their own, whose pages count runs. Mixers that keep a state of
 fixed size get one slot per live request, the same slot number in all such
 groups; it is handed out at admission and taken back when the request ends.
@@ -41,9 +42,22 @@ from .pages import OutOfPages, PagePool
 class _Group:
     tensors: tuple                       # the PagedTensors that every layer of the group keeps
     window: int
+    chunk: int
+    keep_first: int
     every: int                           # tokens that one element stands for: 1, or a run's length
     planes: list
     pool: PagePool
+
+    @property
+    def gives_back(self):
+        """Whether pages go back while the request lives."""
+        return self.window > 0 or self.chunk > 0
+
+    def first_needed(self, length):
+        """The first position, the kept first tokens aside, that a query at `length` or behind it can see."""
+        if self.chunk > 0:
+            return length - length % self.chunk
+        return max(0, length - self.window + 1) if self.window > 0 else 0
 
 
 @dataclass
@@ -92,10 +106,10 @@ class CacheManager:
         for plane, need in enumerate(needs):
             g = r = s = -1
             if need is not None and need.paged:
-                g = self._join_group((tuple(need.paged), need.window, 1), plane, num_pages)
+                g = self._join_group((tuple(need.paged), need.window, need.chunk, need.keep_first, 1), plane, num_pages)
             if need is not None and need.runs:
                 every = int(need.run_length)
-                r = self._join_group((tuple(need.runs), 0, every), plane,
+                r = self._join_group((tuple(need.runs), 0, 0, 0, every), plane,
                                      min(num_pages, -(-num_pages // every) + max_requests))
             if need is not None and need.has_state:
                 key = (tuple(need.state_shape), need.state_dtype)
@@ -114,7 +128,7 @@ class CacheManager:
         self._admissions = 0
         self.fresh_slots = []     # slots handed out since the storage last cleared them
         self.prefix_cache = bool(prefix_cache) and bool(self.groups) and not self.state_groups \
-            and all(g.window <= 0 and g.every == 1 for g in self.groups)
+            and all(not g.gives_back and g.every == 1 for g in self.groups)
         self._nodes = {}                  # node id -> _Node
         self._index = {}                  # (parent id, tokens of the block) -> node id
         self._idle = OrderedDict()        # nodes without holders, the one left longest ago first
@@ -122,9 +136,9 @@ class CacheManager:
         self.prefix_hits = 0              # tokens that requests did not have to compute
 
     def _join_group(self, key, plane, num_pages):
-        """The number of the group that keeps (tensors, window, tokens per element), made if it is new."""
+        """The number of the group that keeps (tensors, window, chunk, first tokens, tokens per element), made if it is new."""
         for i, grp in enumerate(self.groups):
-            if (grp.tensors, grp.window, grp.every) == key:
+            if (grp.tensors, grp.window, grp.chunk, grp.keep_first, grp.every) == key:
                 grp.planes.append(plane)
                 return i
         self.groups.append(_Group(*key, planes=[plane], pool=PagePool(num_pages)))
@@ -205,21 +219,20 @@ class CacheManager:
         held.reserved = max(held.reserved, new_tokens)
 
     def commit(self, request_id, new_tokens):
-        """The step wrote `new_tokens` more positions. Pages of windowed groups
-        that no later query can see are given back."""
+        """The step wrote `new_tokens` more positions. Pages of windowed and chunked
+        groups that no later query can see are given back."""
         held = self._requests[request_id]
         if new_tokens > held.reserved:
             raise RuntimeError("commit of %d tokens, only %d reserved" % (new_tokens, held.reserved))
         held.length += new_tokens
         held.reserved = 0
         for g, grp in enumerate(self.groups):
-            if grp.window <= 0:
+            if not grp.gives_back:
                 continue
-            # the next query sits at position >= length and sees keys > its position - window
-            first_needed = held.length - grp.window + 1
-            dead_blocks = max(0, first_needed) // self.page_size
+            dead_blocks = grp.first_needed(held.length) // self.page_size
+            kept_blocks = -(-grp.keep_first // self.page_size)
             table = held.tables[g]
-            for b in range(min(dead_blocks, len(table))):
+            for b in range(kept_blocks, min(dead_blocks, len(table))):
                 if table[b] >= 0:
                     grp.pool.give(table[b])
                     table[b] = -1

@@ -224,10 +224,10 @@ static inline float make_score_scale(float scale) { return scale * 1.44269504088
 // maximum stands -bias log2(e), which never moves, so that the argument is formed as an exponent is
 // elsewhere; wherever results are joined every weight is one. `q3_set_sigmoid_bias` names the
 // biases (one per query head) of the launches that follow in the calling thread.
-// The builds with Q3_POOLED or Q3_SIGMOID also multiply a result by sigmoid(gate) on its way out, where
+// The builds with Q3_POOLED, Q3_SIGMOID or Q3_SPAN also multiply a result by sigmoid(gate) on its way out, where
 // its row is final: `gate` float32, rows `stride` apart, a number per head or (`wide`) one per column;
 // null: no gate. `q3_set_gate` names the gate of the launches that follow in the calling thread.
-#if defined(Q3_POOLED) || defined(Q3_SIGMOID)
+#if defined(Q3_POOLED) || defined(Q3_SIGMOID) || defined(Q3_SPAN)
 #define Q3_GATED 1
 struct OutGate {
   const float* gate;
@@ -292,6 +292,53 @@ __device__ __forceinline__ int runs_seen(int pos, int window, int pool) {
 #define Q3_RUNS_ARG
 #endif
 
+// Which keys before its own position a row sees. Ordinarily `window` says it: all of them (0) or fewer than
+// `window` behind. A build with Q3_SPAN (attention_span.hip) has a `Span` in the window's place: a row at
+// position p sees keys from p - window + 1 on, or, with `chunk`, from the start of its own stretch of `chunk`
+// positions (counted from the sequence's first) on, and besides, in either case, the keys before `keep`.
+// The tiles of those first keys come ahead of the others; what a page given back or an earlier chunk holds is
+// never asked for. `q3_set_span` names the span of the launches that follow in the calling thread, and the
+// values' size, which may differ from the keys' there.
+#ifdef Q3_SPAN
+struct Span {
+  int window, chunk, keep;
+};
+typedef Span span_t;
+__device__ __forceinline__ int span_begin(const Span& s, int pos) {
+  if (s.chunk > 0) return pos - pos % s.chunk;
+  return s.window > 0 ? max(0, pos - s.window + 1) : 0;
+}
+// a row's own: from which key on it sees, and which first keys besides
+struct RowSpan {
+  int lo, keep;
+};
+typedef RowSpan row_span_t;
+template <int N>
+struct RowSpans {
+  int lo[N], keep;
+};
+template <int N>
+using row_spans_t = RowSpans<N>;
+template <int N>
+__device__ __forceinline__ RowSpan span_of(const RowSpans<N>& s, int i) { return RowSpan{s.lo[i], s.keep}; }
+__device__ __forceinline__ bool span_hides(const RowSpan& s, int pos, int key) { return key < s.lo && key >= s.keep; }
+static thread_local int g_span_chunk = 0, g_span_keep = 0, g_span_value_dim = 0;
+extern "C" void q3_set_span(int chunk, int keep, int value_dim) {
+  g_span_chunk = chunk;
+  g_span_keep = keep;
+  g_span_value_dim = value_dim;
+}
+static inline Span make_span(int window) { return Span{window, g_span_chunk, g_span_keep}; }
+#else
+typedef int span_t;
+typedef int row_span_t;
+template <int N>
+using row_spans_t = int;
+__device__ __forceinline__ int span_of(int window, int i) { return window; }
+__device__ __forceinline__ bool span_hides(int window, int pos, int key) { return window > 0 && pos - key >= window; }
+static inline int make_span(int window) { return window; }
+#endif
+
 // The softmax update of one block of 16 rows for one 32-key tile. s: this lane's
 // eight raw scores (two key blocks of four). Scores enter scaled by scale_log2
 // only inside the exponent: p = 2^(s * scale - m), with m the running maximum of
@@ -300,7 +347,7 @@ __device__ __forceinline__ int runs_seen(int pos, int window, int pool) {
 // operand and rescales the accumulators only if some row's maximum moved.
 template <int NB>
 __device__ __forceinline__ Pack16 softmax_step(const f32x4_t (&s)[2], bool full, int key0, int grp, int row_pos,
-                                               int window, score_scale_t scale_log2, float& m_run, float& l_run,
+                                               row_span_t window, score_scale_t scale_log2, float& m_run, float& l_run,
                                                f32x4_t (&acc)[NB]) {
   float v[8];
 #pragma unroll
@@ -314,7 +361,7 @@ __device__ __forceinline__ Pack16 softmax_step(const f32x4_t (&s)[2], bool full,
     for (int j = 0; j < 8; ++j) {
       const int key = key0 + 16 * (j >> 2) + 4 * grp + (j & 3);
       bool seen = key <= row_pos;
-      if (window > 0 && row_pos - key >= window) seen = false;
+      if (span_hides(window, row_pos, key)) seen = false;
       if (!seen) v[j] = -INFINITY;
     }
   }
@@ -362,7 +409,7 @@ struct TileAddr {
 
 __device__ __forceinline__ TileAddr tile_addr(const bf16_t* __restrict__ k_cache, const bf16_t* __restrict__ v_cache,
                                               int num_pages, const int* __restrict__ bt_row, int Hkv, int g_kv,
-                                              int page, int D, int key0, int kv_len) {
+                                              int page, int D, int DV, int key0, int kv_len) {
   const int lane = threadIdx.x & 63;
   const int col = lane & 15, grp = lane >> 4;
   TileAddr t;
@@ -376,7 +423,7 @@ __device__ __forceinline__ TileAddr tile_addr(const bf16_t* __restrict__ k_cache
       if (pg >= 0 && pg < num_pages) {
         const int slot0 = kbase % page;
         t.k[kb] = k_cache + (((size_t)pg * Hkv + g_kv) * page + slot0 + col) * D + 8 * grp;
-        t.v[kb] = v_cache + (((size_t)pg * Hkv + g_kv) * D + col) * page + slot0 + 4 * grp;
+        t.v[kb] = v_cache + (((size_t)pg * Hkv + g_kv) * DV + col) * page + slot0 + 4 * grp;
       }
     }
   }
@@ -403,7 +450,7 @@ __device__ __forceinline__ TilePages tile_pages(const int* __restrict__ bt_row, 
 
 __device__ __forceinline__ TileAddr tile_addr_of(const TilePages& p, const bf16_t* __restrict__ k_cache,
                                                  const bf16_t* __restrict__ v_cache, int num_pages, int Hkv, int g_kv,
-                                                 int page, int D, int key0) {
+                                                 int page, int D, int DV, int key0) {
   const int lane = threadIdx.x & 63;
   const int col = lane & 15, grp = lane >> 4;
   TileAddr t;
@@ -415,7 +462,7 @@ __device__ __forceinline__ TileAddr tile_addr_of(const TilePages& p, const bf16_
     if (pg >= 0 && pg < num_pages) {
       const int slot0 = (key0 + 16 * kb) % page;
       t.k[kb] = k_cache + (((size_t)pg * Hkv + g_kv) * page + slot0 + col) * D + 8 * grp;
-      t.v[kb] = v_cache + (((size_t)pg * Hkv + g_kv) * D + col) * page + slot0 + 4 * grp;
+      t.v[kb] = v_cache + (((size_t)pg * Hkv + g_kv) * DV + col) * page + slot0 + 4 * grp;
     }
   }
   return t;
@@ -454,11 +501,11 @@ __device__ __forceinline__ void load_values(Pack16 (&vt)[D / 16], const TileAddr
     }
 }
 
-template <int D, int QB>
+template <int D, int QB, int DV = D>
 __device__ __forceinline__ void attend_tile(const Pack16 (&qreg)[QB][D / 32], const Pack16 (&a)[2][D / 32],
-                                            Pack16 (&vt)[D / 16], int key0, int kv_len,
-                                            const int (&row_pos)[QB], int window, score_scale_t scale_log2,
-                                            f32x4_t (&acc)[QB][D / 16], float (&m_run)[QB], float (&l_run)[QB]) {
+                                            Pack16 (&vt)[DV / 16], int key0, int kv_len,
+                                            const int (&row_pos)[QB], row_spans_t<QB> window, score_scale_t scale_log2,
+                                            f32x4_t (&acc)[QB][DV / 16], float (&m_run)[QB], float (&l_run)[QB]) {
   const int lane = threadIdx.x & 63;
   const int grp = lane >> 4;
   f32x4_t s[QB][2];
@@ -475,17 +522,17 @@ __device__ __forceinline__ void attend_tile(const Pack16 (&qreg)[QB][D / 32], co
   Pack16 p[QB];
 #pragma unroll
   for (int qb = 0; qb < QB; ++qb)
-    p[qb] = softmax_step<D / 16>(s[qb], false, key0, grp, row_pos[qb], window, scale_log2, m_run[qb], l_run[qb],
-                                 acc[qb]);
+    p[qb] = softmax_step<DV / 16>(s[qb], false, key0, grp, row_pos[qb], span_of(window, qb), scale_log2, m_run[qb],
+                                  l_run[qb], acc[qb]);
   if (key0 + FAST_TILE > kv_len) {  // slots past the sequence's end hold anything: zero them, 0 * NaN is NaN
 #pragma unroll
-    for (int nb = 0; nb < D / 16; ++nb)
+    for (int nb = 0; nb < DV / 16; ++nb)
 #pragma unroll
       for (int j = 0; j < 8; ++j)
         if (key0 + 16 * (j >> 2) + 4 * grp + (j & 3) >= kv_len) vt[nb].e[j] = (__bf16)0.f;
   }
 #pragma unroll
-  for (int nb = 0; nb < D / 16; ++nb)
+  for (int nb = 0; nb < DV / 16; ++nb)
 #pragma unroll
     for (int qb = 0; qb < QB; ++qb)
       acc[qb][nb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vt[nb].v, p[qb].v, acc[qb][nb], 0, 0, 0);
@@ -502,7 +549,7 @@ __device__ __forceinline__ TileAddr first_tile_keys(Pack16 (&a_cur)[2][D / 32], 
                                                     int first, int last, int kv_len) {
   TileAddr t{};
   if (first >= last) return t;
-  t = tile_addr(k_cache, v_cache, num_pages, bt_row, Hkv, g_kv, page, D, first * FAST_TILE, kv_len);
+  t = tile_addr(k_cache, v_cache, num_pages, bt_row, Hkv, g_kv, page, D, D, first * FAST_TILE, kv_len);
   load_keys<D>(a_cur, t);
   return t;
 }
@@ -512,8 +559,8 @@ __device__ __forceinline__ void attend_tiles(const Pack16 (&qreg)[QB][D / 32], P
                                              TileAddr t_cur, const bf16_t* __restrict__ k_cache,
                                              const bf16_t* __restrict__ v_cache, int num_pages,
                                              const int* __restrict__ bt_row, int Hkv, int g_kv, int page, int first,
-                                             int last, int step, int kv_len, const int (&row_pos)[QB], int window,
-                                             score_scale_t scale_log2, f32x4_t (&acc)[QB][D / 16], float (&m_run)[QB],
+                                             int last, int step, int kv_len, const int (&row_pos)[QB],
+                                             row_spans_t<QB> window, score_scale_t scale_log2, f32x4_t (&acc)[QB][D / 16], float (&m_run)[QB],
                                              float (&l_run)[QB]) {
   if (first >= last) return;
   Pack16 a_nxt[2][D / 32], vt[D / 16];
@@ -521,7 +568,7 @@ __device__ __forceinline__ void attend_tiles(const Pack16 (&qreg)[QB][D / 32], P
     load_values<D>(vt, t_cur, page);
     const bool more = t + step < last;
     if (more) {
-      t_cur = tile_addr(k_cache, v_cache, num_pages, bt_row, Hkv, g_kv, page, D, (t + step) * FAST_TILE, kv_len);
+      t_cur = tile_addr(k_cache, v_cache, num_pages, bt_row, Hkv, g_kv, page, D, D, (t + step) * FAST_TILE, kv_len);
       load_keys<D>(a_nxt, t_cur);
     }
     attend_tile<D, QB>(qreg, a_cur, vt, t * FAST_TILE, kv_len, row_pos, window, scale_log2, acc, m_run, l_run);
@@ -545,9 +592,9 @@ __device__ __forceinline__ void attend_tiles_ahead(const Pack16 (&qreg)[QB][D / 
                                                    const bf16_t* __restrict__ v_cache, int num_pages,
                                                    const int* __restrict__ bt_row, int bt_stride, int Hkv, int g_kv,
                                                    int page, int first, int last, int step, int kv_len,
-                                                   const int (&row_pos)[QB], int window, score_scale_t scale_log2,
-                                                   f32x4_t (&acc)[QB][D / 16], float (&m_run)[QB],
-                                                   float (&l_run)[QB]) {
+                                                   const int (&row_pos)[QB], row_spans_t<QB> window,
+                                                   score_scale_t scale_log2, f32x4_t (&acc)[QB][D / 16],
+                                                   float (&m_run)[QB], float (&l_run)[QB]) {
   if (first >= last) return;
   // a tile's keys and values are asked for together, a whole tile before they are used: a
   // wavefront with two or three tiles (few requests, each over a few thousand keys) then waits
@@ -556,7 +603,7 @@ __device__ __forceinline__ void attend_tiles_ahead(const Pack16 (&qreg)[QB][D / 
   for (int t = first; t < last; t += step) {
     const bool more = t + step < last;
     if (more) {
-      const TileAddr t_nxt = tile_addr_of(p_nxt, k_cache, v_cache, num_pages, Hkv, g_kv, page, D, (t + step) * FAST_TILE);
+      const TileAddr t_nxt = tile_addr_of(p_nxt, k_cache, v_cache, num_pages, Hkv, g_kv, page, D, D, (t + step) * FAST_TILE);
       load_keys<D>(a_nxt, t_nxt);
       load_values<D>(v_nxt, t_nxt, page);
       p_nxt = tile_pages(bt_row, bt_stride, page, (t + 2 * step) * FAST_TILE);
@@ -595,7 +642,7 @@ __device__ __forceinline__ void attend_both(const Pack16 (&qreg)[1][D / 32], con
   auto addr_of = [&](const TilePages& p, int s) {
     const bool run = s < run_tiles;
     return tile_addr_of(p, run ? runs.k : k_cache, run ? runs.v : v_cache, run ? runs.num_pages : num_pages, Hkv, g_kv, page,
-                        D, key_of(s));
+                        D, D, key_of(s));
   };
   Pack16 a_cur[2][D / 32], v_cur[D / 16], a_nxt[2][D / 32], v_nxt[D / 16];
   {
@@ -623,6 +670,50 @@ __device__ __forceinline__ void attend_both(const Pack16 (&qreg)[1][D / 32], con
         for (int i = 0; i < D / 32; ++i) a_cur[kb][i] = a_nxt[kb][i];
 #pragma unroll
       for (int nb = 0; nb < D / 16; ++nb) v_cur[nb] = v_nxt[nb];
+    }
+  }
+}
+#endif
+
+#ifdef Q3_SPAN
+// A wavefront's rows over a sequence of tiles of which those before `keep_tiles` are the sequence's first and
+// the others begin at tile `tile_lo`: tiles first, first + step, ... below last of it. As above a tile's keys
+// and values are asked for a whole tile before they are used and its table entries two tiles before.
+template <int D, int DV>
+__device__ __forceinline__ void attend_span(const Pack16 (&qreg)[1][D / 32], const bf16_t* __restrict__ k_cache,
+                                            const bf16_t* __restrict__ v_cache, int num_pages,
+                                            const int* __restrict__ bt_row, int bt_stride, int Hkv, int g_kv, int page,
+                                            int first, int last, int step, int keep_tiles, int tile_lo, int kv_len,
+                                            const int (&row_pos)[1], RowSpans<1> span, score_scale_t scale_log2,
+                                            f32x4_t (&acc)[1][DV / 16], float (&m_run)[1], float (&l_run)[1]) {
+  if (first >= last) return;
+  auto key_of = [&](int s) { return (s < keep_tiles ? s : tile_lo + s - keep_tiles) * FAST_TILE; };
+  auto addr_of = [&](const TilePages& p, int s) {
+    return tile_addr_of(p, k_cache, v_cache, num_pages, Hkv, g_kv, page, D, DV, key_of(s));
+  };
+  Pack16 a_cur[2][D / 32], v_cur[DV / 16], a_nxt[2][D / 32], v_nxt[DV / 16];
+  {
+    const TileAddr t = addr_of(tile_pages(bt_row, bt_stride, page, key_of(first)), first);
+    load_keys<D>(a_cur, t);
+    load_values<DV>(v_cur, t, page);
+  }
+  TilePages p_nxt = tile_pages(bt_row, bt_stride, page, key_of(first + step));
+  for (int s = first; s < last; s += step) {
+    const bool more = s + step < last;
+    if (more) {
+      const TileAddr t = addr_of(p_nxt, s + step);
+      load_keys<D>(a_nxt, t);
+      load_values<DV>(v_nxt, t, page);
+      p_nxt = tile_pages(bt_row, bt_stride, page, key_of(s + 2 * step));
+    }
+    attend_tile<D, 1, DV>(qreg, a_cur, v_cur, key_of(s), kv_len, row_pos, span, scale_log2, acc, m_run, l_run);
+    if (more) {
+#pragma unroll
+      for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+        for (int i = 0; i < D / 32; ++i) a_cur[kb][i] = a_nxt[kb][i];
+#pragma unroll
+      for (int nb = 0; nb < DV / 16; ++nb) v_cur[nb] = v_nxt[nb];
     }
   }
 }
@@ -780,17 +871,17 @@ __device__ __forceinline__ void store_new_key_value(const bf16_t* row, int Hq, i
 
 // (with two sources the kernel would take a few registers more than leave room for two blocks a CU, which
 // takes a third longer from two splits on)
-#ifdef Q3_POOLED
+#if defined(Q3_POOLED) || defined(Q3_SPAN)
 #define Q3_DECODE_WAVES __attribute__((amdgpu_waves_per_eu(2)))
 #else
 #define Q3_DECODE_WAVES
 #endif
-template <int D, bool PREP, typename W, bool AHEAD>
+template <int D, bool PREP, typename W, bool AHEAD, int DV = D>
 __global__ __launch_bounds__(256) Q3_DECODE_WAVES void attn_decode_kernel(
     const bf16_t* __restrict__ q, int q_stride, bf16_t* __restrict__ out, const bf16_t* __restrict__ k_cache,
     const bf16_t* __restrict__ v_cache, int num_pages, const int* __restrict__ block_table, int bt_stride,
     const int* __restrict__ cu_q, const int* __restrict__ kv_lens, int Hq, int Hkv, int page, score_scale_t scale_log2,
-    int window, int splits, float* __restrict__ ws_acc, float* __restrict__ ws_ml, DecodePrep prep,
+    span_t window, int splits, float* __restrict__ ws_acc, float* __restrict__ ws_ml, DecodePrep prep,
     const float* __restrict__ sink Q3_BIAS_PARAM Q3_RUNS_PARAM Q3_GATE_PARAM) {
   const int b = blockIdx.z, g_kv = blockIdx.y, split = blockIdx.x;
   const int G = Hq / Hkv;
@@ -812,7 +903,7 @@ __global__ __launch_bounds__(256) Q3_DECODE_WAVES void attn_decode_kernel(
   TilePages p_second{};
   if constexpr (ahead) {
     t_first = tile_addr_of(tile_pages(bt_row, bt_stride, page, ahead_first * FAST_TILE), k_cache, v_cache, num_pages,
-                           Hkv, g_kv, page, D, ahead_first * FAST_TILE);
+                           Hkv, g_kv, page, D, D, ahead_first * FAST_TILE);
     load_keys<D>(a_first, t_first);
     load_values<D>(v_first, t_first, page);
     p_second = tile_pages(bt_row, bt_stride, page, (ahead_first + ahead_step) * FAST_TILE);
@@ -861,14 +952,27 @@ __global__ __launch_bounds__(256) Q3_DECODE_WAVES void attn_decode_kernel(
   // with a fresh key the cache is read up to the position before it: the rows then stand one
   // position earlier for the masks, and the window, which counts the new key, is one shorter
   const int kv_seen = fresh ? kv_len - 1 : kv_len;
-  const int win = (fresh && window > 0) ? window - 1 : window;
   int row_pos[1];
   row_pos[0] = col < rows ? first_pos + col / G - (fresh ? 1 : 0) : -1;
+#ifdef Q3_SPAN
+  const RowSpans<1> win{{span_begin(window, row_pos[0])}, window.keep};
+  const int tile_lo = span_begin(window, first_pos) / FAST_TILE;
+  const int tile_hi = (kv_seen + FAST_TILE - 1) / FAST_TILE;
+#else
+  const int win = (fresh && window > 0) ? window - 1 : window;
   int tile_lo = 0;
   if (window > 0) tile_lo = max(0, first_pos - window + 1) / FAST_TILE;
   int tile_hi = (kv_seen + FAST_TILE - 1) / FAST_TILE;
   if (fresh && window == 1) tile_hi = tile_lo;  // the new key alone is visible
-#ifdef Q3_POOLED
+#endif
+#if defined(Q3_SPAN)
+  // the first keys' tiles come first in the sequence of tiles that the splits share out
+  const int keep_tiles = min((window.keep + FAST_TILE - 1) / FAST_TILE, tile_lo);
+  const int all_tiles = keep_tiles + tile_hi - tile_lo;
+  const int per_split = (all_tiles + splits - 1) / splits;
+  const int s0 = min(split * per_split, all_tiles), s1 = min(s0 + per_split, all_tiles);
+  (void)t_first;
+#elif defined(Q3_POOLED)
   // the runs' tiles come first in the sequence of tiles that the splits share out
   const int run_tiles = (runs_seen(first_pos + q_len - 1, window, runs.pool) + FAST_TILE - 1) / FAST_TILE;
   const int all_tiles = run_tiles + max(tile_hi - tile_lo, 0);
@@ -880,7 +984,7 @@ __global__ __launch_bounds__(256) Q3_DECODE_WAVES void attn_decode_kernel(
   const int t0 = tile_lo + split * per_split;
   const int t1 = min(tile_hi, t0 + per_split);
 #endif
-#ifndef Q3_POOLED
+#if !defined(Q3_POOLED) && !defined(Q3_SPAN)
   // the first tile's keys are on their way while the query rows are prepared
   if constexpr (!ahead)
     t_first = first_tile_keys<D>(a_first, k_cache, v_cache, num_pages, bt_row, Hkv, g_kv, page, t0 + wave, t1, kv_seen);
@@ -912,15 +1016,18 @@ __global__ __launch_bounds__(256) Q3_DECODE_WAVES void attn_decode_kernel(
     }
   }
 
-  f32x4_t acc[1][D / 16];
+  f32x4_t acc[1][DV / 16];
 #pragma unroll
-  for (int nb = 0; nb < D / 16; ++nb) acc[0][nb] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  for (int nb = 0; nb < DV / 16; ++nb) acc[0][nb] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #ifdef Q3_SIGMOID
   float m_run[1] = {col < rows ? -score_bias[g_kv * G + col % G] * 1.4426950408889634f : 0.f}, l_run[1] = {0.f};
 #else
   float m_run[1] = {-INFINITY}, l_run[1] = {0.f};
 #endif
-#ifdef Q3_POOLED
+#if defined(Q3_SPAN)
+  attend_span<D, DV>(qreg, k_cache, v_cache, num_pages, bt_row, bt_stride, Hkv, g_kv, page, s0 + wave, s1, 4, keep_tiles,
+                     tile_lo, kv_seen, row_pos, win, scale_log2, acc, m_run, l_run);
+#elif defined(Q3_POOLED)
   attend_both<D>(qreg, k_cache, v_cache, num_pages, bt_row, bt_stride, runs, runs.table + (size_t)b * runs.stride, Hkv, g_kv,
                  page, s0 + wave, s1, 4, run_tiles, tile_lo, kv_seen, row_pos, win, scale_log2, acc, m_run, l_run);
 #else
@@ -944,7 +1051,7 @@ __global__ __launch_bounds__(256) Q3_DECODE_WAVES void attn_decode_kernel(
   // the merge of the four wavefronts, and of the new key as a fifth contribution of one key:
   // its score is its maximum, its sum is one, its accumulator is the value itself
   __shared__ float sh_m[5][16], sh_l[4][16];
-  __shared__ float sh_acc[4][16][D + 4];
+  __shared__ float sh_acc[4][16][DV + 4];
   if (grp == 0) {
     sh_m[wave][col] = m_run[0];
     sh_l[wave][col] = l;
@@ -956,7 +1063,7 @@ __global__ __launch_bounds__(256) Q3_DECODE_WAVES void attn_decode_kernel(
   const float w_mine = m_run[0] > -INFINITY ? exp2f(m_run[0] - m_all) : 0.f;
   if (col < rows) {
 #pragma unroll
-    for (int nb = 0; nb < D / 16; ++nb)
+    for (int nb = 0; nb < DV / 16; ++nb)
 #pragma unroll
       for (int j = 0; j < 4; ++j) sh_acc[wave][col][16 * nb + 4 * grp + j] = acc[0][nb][j] * w_mine;
   }
@@ -978,17 +1085,17 @@ __global__ __launch_bounds__(256) Q3_DECODE_WAVES void attn_decode_kernel(
 #else
     const float inv = 1.f / (sink ? lr + exp2f(sink[head] * 1.4426950408889634f - mr) : lr);
 #endif
-    for (int d = dd; d < D; d += 16) {
+    for (int d = dd; d < DV; d += 16) {
       float o = sh_acc[0][r][d] + sh_acc[1][r][d] + sh_acc[2][r][d] + sh_acc[3][r][d];
       if (PREP && w5 > 0.f) o += sh_v[d] * w5;
-      out[(size_t)token * Hq * D + (size_t)head * D + d] = float_to_bf16(o * inv Q3_OPEN(token, head, D, d));
+      out[(size_t)token * Hq * DV + (size_t)head * DV + d] = float_to_bf16(o * inv Q3_OPEN(token, head, DV, d));
     }
   } else {
     const size_t slot = (((size_t)b * Hkv + g_kv) * splits + split) * 16 + r;
-    for (int d = dd; d < D; d += 16) {
+    for (int d = dd; d < DV; d += 16) {
       float o = sh_acc[0][r][d] + sh_acc[1][r][d] + sh_acc[2][r][d] + sh_acc[3][r][d];
       if (PREP && w5 > 0.f) o += sh_v[d] * w5;
-      ws_acc[slot * D + d] = o;
+      ws_acc[slot * DV + d] = o;
     }
     if (dd == 0) {
       ws_ml[slot * 2] = mr;
@@ -1136,25 +1243,28 @@ __global__ __launch_bounds__(256) void attn_decode_reduce_kernel(
 // overlap only in part. The rewrite was not kept: its gain is within what boxes differ by from 4,096 tokens on.)
 #define PF_TILE 64    // keys per tile
 #define PF_STAGES 2  // tiles in shared memory: one being worked on, the others on their way
-template <int D, int TILE>
+template <int D, int TILE, int DV = D>
 struct PrefillSmem {
   // A stage holds a tile's keys (TILE rows of D) and values (D rows of TILE), both as
   // 16-byte pieces in an order chosen so that the matrix-core operand reads spread over all
   // banks without padding (the loads that fill a stage write whole kilobytes, see below).
-  // A window is 256 bytes. Keys: a window = RPW rows of CPR pieces; piece c of row r sits at
-  // place (r % RPW) * CPR + (c ^ (window % CPR)) of window r / RPW. Values (a piece = eight
+  // A window is 256 bytes. Keys: a row has CPR places, its pieces (or the next power of two: key sizes
+  // that are none leave places empty), and a window RPW rows; piece c of row r sits at place
+  // c ^ ((r / RPW) % min(CPR, 16)) of its row. Values (a piece = eight
   // keys of one 16-key block): sixteen rows' pieces of the tile's first half of blocks are
   // followed by the same rows' pieces of its second half (two planes), so that the two 8-byte
   // reads that make one operand of the second product (four keys of block h, four of block
   // h + blocks / 2) are a fixed, short distance apart and one instruction fetches both. A
   // plane's sixteen rows are VPR windows of VRW rows of VPR pieces (q = 2 * (block in the
   // plane) + half); piece q of row d sits at place (d % VRW) * VPR + (q ^ window) of its window.
-  static constexpr int CPR = D / 8;          // 16-byte pieces per key row
-  static constexpr int RPW = 16 / CPR > 0 ? 16 / CPR : 1;   // key rows per window (D <= 128)
+  static constexpr int PIECES = D / 8;       // 16-byte pieces of a key
+  static constexpr int CPR = PIECES <= 8 ? 8 : PIECES <= 16 ? 16 : 32;   // and places of its row
+  static constexpr int RPW = CPR < 16 ? 16 / CPR : 1;       // key rows per window
+  static constexpr int SWZ = CPR < 16 ? CPR : 16;
   static constexpr int VPR = TILE / 16;      // pieces per value row in a plane
   static constexpr int VRW = 16 / VPR;       // value rows per window
-  static constexpr int K_BYTES = TILE * D * 2;
-  static constexpr int V_BYTES = D * TILE * 2;
+  static constexpr int K_BYTES = TILE * CPR * 16;
+  static constexpr int V_BYTES = DV * TILE * 2;
   static constexpr int STAGE = K_BYTES + V_BYTES;
   static constexpr int K_PIECES = K_BYTES / 16, V_PIECES = V_BYTES / 16;
 };
@@ -1163,7 +1273,7 @@ struct PrefillSmem {
 // softmax_step; the probabilities come back as the P operands of the tile's 32-key halves.
 template <int NB, int KB4>
 __device__ __forceinline__ void softmax_tile(const f32x4_t (&s)[KB4], bool full, int key0, int grp, int row_pos,
-                                             int window, score_scale_t scale_log2, float& m_run, float& l_run,
+                                             row_span_t window, score_scale_t scale_log2, float& m_run, float& l_run,
                                              f32x4_t (&acc)[NB], Pack16 (&p)[KB4 / 2]) {
   constexpr int N = 4 * KB4;
   static_assert(N % 2 == 0, "maxima are taken three at a time");
@@ -1184,7 +1294,7 @@ __device__ __forceinline__ void softmax_tile(const f32x4_t (&s)[KB4], bool full,
     for (int j = 0; j < N; ++j) {
       const int key = first_key + 16 * (j >> 2) + (j & 3);
       bool seen = key <= pos;
-      if (window > 0 && pos - key >= window) seen = false;
+      if (span_hides(window, pos, key)) seen = false;
       if (!seen) v[j] = -INFINITY;
     }
   }
@@ -1234,14 +1344,14 @@ __device__ __forceinline__ void softmax_tile(const f32x4_t (&s)[KB4], bool full,
 #endif
 }
 
-template <int D, int TILE, int STAGES>
+template <int D, int TILE, int STAGES, int DV = D>
 __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) void attn_prefill_kernel(
     const bf16_t* __restrict__ q, int q_stride, bf16_t* __restrict__ out, const bf16_t* __restrict__ k_cache,
     const bf16_t* __restrict__ v_cache, int num_pages, const int* __restrict__ block_table, int bt_stride,
     const int* __restrict__ cu_q, const int* __restrict__ kv_lens, int Hq, int Hkv, int page, score_scale_t scale_log2,
-    int window, int tokens_per_block, int key_splits, float* __restrict__ part_acc, float* __restrict__ part_ml,
+    span_t window, int tokens_per_block, int key_splits, float* __restrict__ part_acc, float* __restrict__ part_ml,
     const float* __restrict__ sink Q3_BIAS_PARAM Q3_RUNS_PARAM Q3_GATE_PARAM) {
-  typedef PrefillSmem<D, TILE> SM;
+  typedef PrefillSmem<D, TILE, DV> SM;
   constexpr int KB4 = TILE / 16;  // 16-key blocks per tile
   __shared__ __attribute__((aligned(16))) unsigned char smem[STAGES * SM::STAGE];
   __shared__ int sh_pages[PREFILL_PAGES];  // the block-table entries of the tiles in hand
@@ -1304,11 +1414,11 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
   // the same in all lanes: kept as scalars, so that what is decided by them per tile is a scalar branch
   pos_max = __builtin_amdgcn_readfirstlane(pos_max);
   pos_min = __builtin_amdgcn_readfirstlane(pos_min);
-  f32x4_t acc[2][D / 16];
+  f32x4_t acc[2][DV / 16];
 #pragma unroll
   for (int qb = 0; qb < 2; ++qb)
 #pragma unroll
-    for (int nb = 0; nb < D / 16; ++nb) acc[qb][nb] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    for (int nb = 0; nb < DV / 16; ++nb) acc[qb][nb] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #ifdef Q3_SIGMOID
   float m_run[2], l_run[2] = {0.f, 0.f};
 #pragma unroll
@@ -1321,12 +1431,38 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
   const int blk_first_tok = tile * tokens_per_block;
   const int blk_last_tok = min(q_len, blk_first_tok + tokens_per_block) - 1;
   int tile_lo = 0;
+#ifdef Q3_SPAN
+  tile_lo = span_begin(window, first_pos + blk_first_tok) / TILE;
+#else
   if (window > 0) tile_lo = max(0, first_pos + blk_first_tok - window + 1) / TILE;
+#endif
   int tile_hi = (first_pos + blk_last_tok) / TILE + 1;
   // and this wavefront's own (a wavefront whose rows do not exist has none)
   int my_lo = tile_lo, my_hi = pos_max >= 0 ? pos_max / TILE + 1 : 0;
-  if (window > 0 && pos_max >= 0) my_lo = max(0, pos_min - window + 1) / TILE;
-#ifdef Q3_POOLED
+#ifdef Q3_SPAN
+  // (where a block's span begins among the first keys, none of its wavefronts may pass them by)
+  if (pos_max >= 0 && window.keep <= tile_lo * TILE) my_lo = span_begin(window, pos_min) / TILE;
+  row_spans_t<2> row_spans;
+  row_spans.keep = window.keep;
+#pragma unroll
+  for (int qb = 0; qb < 2; ++qb) row_spans.lo[qb] = span_begin(window, max(row_pos[qb], 0));
+  const int first_seen = span_begin(window, first_pos);                 // of the portion's first row
+  const int latest_lo = span_begin(window, max(pos_max, 0));            // of the wavefront's last row
+  // the tiles of the first keys, ahead of the others in the sequence of tiles that the splits share out
+  int keep_lo = 0, keep_hi = min((window.keep + TILE - 1) / TILE, tile_lo);
+  if (key_splits > 1) {
+    const int keep_tiles = keep_hi, all = keep_tiles + tile_hi - tile_lo;
+    const int share = (all + key_splits - 1) / key_splits;
+    const int s0 = min(all, split * share), s1 = min(all, s0 + share);
+    keep_lo = min(s0, keep_tiles);
+    keep_hi = min(s1, keep_tiles);
+    const int base = tile_lo;
+    tile_lo = base + max(s0 - keep_tiles, 0);
+    tile_hi = base + max(s1 - keep_tiles, 0);
+    my_lo = max(my_lo, tile_lo);
+    my_hi = min(my_hi, tile_hi);
+  }
+#elif defined(Q3_POOLED)
   // the same of the runs, ahead of the tokens in the sequence of tiles that the splits share out
   int run_lo = 0, run_hi = (runs_seen(first_pos + blk_last_tok, window, runs.pool) + TILE - 1) / TILE;
   if (key_splits > 1) {
@@ -1367,9 +1503,9 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
   int k_row[K_TURNS], k_off[K_TURNS], v_kb[V_TURNS], v_d[V_TURNS], v_h[V_TURNS];
 #pragma unroll
   for (int j = 0; j < K_TURNS; ++j) {
-    const int place = tid + 256 * j, w = place >> 4, u = place & 15;
-    k_row[j] = w * SM::RPW + u / SM::CPR;
-    k_off[j] = 8 * ((u % SM::CPR) ^ (w % SM::CPR));
+    const int place = tid + 256 * j;
+    k_row[j] = place / SM::CPR;
+    k_off[j] = 8 * ((place % SM::CPR) ^ ((k_row[j] / SM::RPW) % SM::SWZ));
   }
 #pragma unroll
   for (int j = 0; j < V_TURNS; ++j) {
@@ -1380,7 +1516,8 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
     v_kb[j] = plane * (TILE / 32) + (q >> 1);
     v_h[j] = q & 1;
   }
-  const size_t page_elems = (size_t)page * D;  // elements of one (page, head) in either cache
+  const size_t page_elems = (size_t)page * D;  // elements of one (page, head) in the keys' cache
+  const size_t page_elems_v = (size_t)page * DV;  // and in the values'
   // What a thread keeps per load of a whole tile: where in the address tables its piece's page stands,
   // counted from the tile's first page, and the piece's byte offset within (page, head). With pages of
   // fewer keys than a tile the tile begins a page and both are fixed; with larger pages the tile lies
@@ -1413,7 +1550,16 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
 
   // (a page is given back only when every later row's window has left it, so a tile that the first row's
   // window covers from its first key on is all there)
+#ifdef Q3_SPAN
+  // (and so is a tile of first keys that stay)
+  auto plain_tile = [&](int t) {
+    return t * TILE + TILE <= kv_len && (t * TILE >= first_seen || t * TILE + TILE <= window.keep);
+  };
+#else
   auto plain_tile = [&](int t) { return t * TILE + TILE <= kv_len && (window == 0 || t * TILE > first_pos - window); };
+#endif
+  // a place that no piece belongs to is left alone (a key size that is no power of two)
+  auto piece_at = [&](int j) { return SM::PIECES == SM::CPR || k_off[j] < D; };
   auto copy_direct = [&](int t, int stage) {
     const int key0 = t * TILE;
     // this wavefront's kilobyte of each turn
@@ -1431,14 +1577,15 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
     for (int j = 0; j < V_TURNS; ++j) base[K_TURNS + j] = *reinterpret_cast<const long long*>(v_table + v_slot[j]);
     if (small_pages) {   // a tile begins a page: nothing to add to the thread's own offsets
 #pragma unroll
-      for (int j = 0; j < K_TURNS; ++j) load_to_lds(reinterpret_cast<const char*>(base[j]) + k_at[j], ks + 4096 * j);
+      for (int j = 0; j < K_TURNS; ++j)
+        if (piece_at(j)) load_to_lds(reinterpret_cast<const char*>(base[j]) + k_at[j], ks + 4096 * j);
 #pragma unroll
       for (int j = 0; j < V_TURNS; ++j)
         load_to_lds(reinterpret_cast<const char*>(base[K_TURNS + j]) + v_at[j], vs + 4096 * j);
     } else {
 #pragma unroll
       for (int j = 0; j < K_TURNS; ++j)
-        load_to_lds(reinterpret_cast<const char*>(base[j]) + (k_at[j] + k_in), ks + 4096 * j);
+        if (piece_at(j)) load_to_lds(reinterpret_cast<const char*>(base[j]) + (k_at[j] + k_in), ks + 4096 * j);
 #pragma unroll
       for (int j = 0; j < V_TURNS; ++j)
         load_to_lds(reinterpret_cast<const char*>(base[K_TURNS + j]) + (v_at[j] + v_in), vs + 4096 * j);
@@ -1452,7 +1599,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
     for (int j = 0; j < K_TURNS; ++j) {
       const int key = key0 + k_row[j];
       uint4 piece = make_uint4(0, 0, 0, 0);  // rows past the end are zero
-      if (key < kv_len) {
+      if (key < kv_len && piece_at(j)) {
         const int pg = sh_pages[(key >> page_shift) - page_base];
         if (pg >= 0 && pg < num_pages)
           piece = *reinterpret_cast<const uint4*>(k_cache + (size_t)(pg * Hkv + g_kv) * page_elems +
@@ -1468,7 +1615,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
       if (key < kv_len) {
         const int pg = sh_pages[(key >> page_shift) - page_base];
         if (pg >= 0 && pg < num_pages) {
-          piece.u = *reinterpret_cast<const uint4*>(v_cache + (size_t)(pg * Hkv + g_kv) * page_elems +
+          piece.u = *reinterpret_cast<const uint4*>(v_cache + (size_t)(pg * Hkv + g_kv) * page_elems_v +
                                                     (v_d[j] * page + (key & (page - 1))));
           if (key + 8 > kv_len) {  // slots past the end hold anything: zero them (0 * NaN is NaN)
 #pragma unroll
@@ -1488,8 +1635,8 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
   };
   // the operand reads' addresses: this lane's window and swizzle for the key rows 16 kb4 + col
   // and for the value rows 16 nb + col
-  const int k_lane = (col / SM::RPW) * 256 + (col % SM::RPW) * SM::CPR * 16;
-  const int k_swz = (col / SM::RPW) % SM::CPR;
+  const int k_lane = col * SM::CPR * 16;
+  const int k_swz = (col / SM::RPW) % SM::SWZ;
   const int v_lane = (col / SM::VRW) * 256 + (col % SM::VRW) * SM::VPR * 16 + 8 * (grp & 1);
   const int v_swz = (col / SM::VRW) % SM::VPR;
   int k_read[D / 32], v_read[TILE / 32];
@@ -1508,6 +1655,21 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
 #pragma unroll
     for (int i = 0; i < D / 32; ++i) asm volatile("" : "+v"(qreg[qb][i].v));
 
+#ifdef Q3_SPAN
+  // the first keys' tiles, then the others
+  const int main_lo = tile_lo, main_hi = tile_hi, main_my_lo = my_lo, main_my_hi = my_hi;
+  tile_lo = my_lo = keep_lo;
+  tile_hi = keep_hi;
+  my_hi = pos_max >= 0 ? keep_hi : 0;
+#pragma nounroll
+  for (int source = 0; source < 2; ++source) {
+  if (source == 1) {
+    tile_lo = main_lo;
+    tile_hi = main_hi;
+    my_lo = main_my_lo;
+    my_hi = main_my_hi;
+  }
+#endif
 #ifdef Q3_POOLED
   // the runs first, then the tokens: what the tile loop works with is exchanged in between
   const bf16_t *token_k = k_cache, *token_v = v_cache;
@@ -1558,9 +1720,9 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
       for (int i = tid; page_base + i <= last_page; i += 256) {
         const int pg = bt_row[page_base + i];
         sh_pages[i] = pg;
-        const long long at = 2 * (long long)(min(max(pg, 0), num_pages - 1) * Hkv + g_kv) * (long long)page_elems;
-        sh_kaddr[i] = reinterpret_cast<long long>(k_cache) + at;
-        sh_vaddr[i] = reinterpret_cast<long long>(v_cache) + at;
+        const long long head = 2 * (long long)(min(max(pg, 0), num_pages - 1) * Hkv + g_kv);
+        sh_kaddr[i] = reinterpret_cast<long long>(k_cache) + head * (long long)page_elems;
+        sh_vaddr[i] = reinterpret_cast<long long>(v_cache) + head * (long long)page_elems_v;
       }
     }
     __syncthreads();
@@ -1595,7 +1757,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
           Pack16 a[D / 32];
 #pragma unroll
           for (int i = 0; i < D / 32; ++i)
-            a[i].u = *reinterpret_cast<const uint4*>(ks + (16 / SM::RPW) * 256 * kb4 + k_read[i]);
+            a[i].u = *reinterpret_cast<const uint4*>(ks + 16 * SM::CPR * 16 * kb4 + k_read[i]);
 #pragma unroll
           for (int qb = 0; qb < 2; ++qb) {
             f32x4_t c = {0.f, 0.f, 0.f, 0.f};
@@ -1606,12 +1768,18 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
           }
         }
         // no key of the tile is hidden from any row of this wavefront?
+#ifdef Q3_SPAN
+        const bool full = key0 + TILE - 1 <= pos_min && (key0 >= latest_lo || key0 + TILE <= window.keep);
+        const row_spans_t<2>& tile_span = row_spans;
+#else
         const bool full = key0 + TILE - 1 <= pos_min && (window == 0 || pos_max - key0 < window);
+        const int tile_span = window;
+#endif
         Pack16 p[2][KB4 / 2];
 #pragma unroll
         for (int qb = 0; qb < 2; ++qb)
-          softmax_tile<D / 16, KB4>(sc[qb], full, key0, grp, row_pos[qb], window, scale_log2, m_run[qb], l_run[qb],
-                                    acc[qb], p[qb]);
+          softmax_tile<DV / 16, KB4>(sc[qb], full, key0, grp, row_pos[qb], span_of(tile_span, qb), scale_log2, m_run[qb],
+                                     l_run[qb], acc[qb], p[qb]);
         // the values' operands (keys 4 grp .. 4 grp + 3 of blocks half and half + KB4 / 2) are
         // read one group of output columns ahead of the matrix instructions that use them
         Pack16 vt[4][KB4 / 2];
@@ -1633,8 +1801,8 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
         read_values(0, vt[0]);
         read_values(1, vt[1]);
 #pragma unroll
-        for (int nb = 0; nb < D / 16; ++nb) {
-          if (nb + 2 < D / 16) read_values(nb + 2, vt[(nb + 2) & 3]);
+        for (int nb = 0; nb < DV / 16; ++nb) {
+          if (nb + 2 < DV / 16) read_values(nb + 2, vt[(nb + 2) & 3]);
 #pragma unroll
           for (int half = 0; half < KB4 / 2; ++half)
 #pragma unroll
@@ -1646,7 +1814,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
         // its use, into the same registers, and waits for it every time): four operands (two reads each) ahead
         __builtin_amdgcn_sched_group_barrier(0x100, 8, 0);
 #pragma unroll
-        for (int i = 0; i < (D / 16) * (KB4 / 2) - 4; ++i) {
+        for (int i = 0; i < (DV / 16) * (KB4 / 2) - 4; ++i) {
           __builtin_amdgcn_sched_group_barrier(0x008, 2, 0);
           __builtin_amdgcn_sched_group_barrier(0x100, 2, 0);
         }
@@ -1657,7 +1825,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
       __syncthreads();
     }
   }
-#ifdef Q3_POOLED
+#if defined(Q3_POOLED) || defined(Q3_SPAN)
   }
 #endif
 #pragma unroll
@@ -1668,9 +1836,9 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
     if (row_pos[qb] < 0) continue;
     if (key_splits > 1) {
       const size_t slot = ((size_t)row_tok[qb] * Hq + row_head[qb]) * key_splits + split;
-      float* o = part_acc + slot * D + 4 * grp;
+      float* o = part_acc + slot * DV + 4 * grp;
 #pragma unroll
-      for (int nb = 0; nb < D / 16; ++nb)
+      for (int nb = 0; nb < DV / 16; ++nb)
         *reinterpret_cast<float4*>(o + 16 * nb) =
             make_float4(acc[qb][nb][0], acc[qb][nb][1], acc[qb][nb][2], acc[qb][nb][3]);
 #ifdef Q3_SIGMOID
@@ -1685,16 +1853,16 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
 #else
     const float inv = 1.f / l;
 #endif
-    bf16_t* o = out + (size_t)row_tok[qb] * Hq * D + (size_t)row_head[qb] * D + 4 * grp;
+    bf16_t* o = out + (size_t)row_tok[qb] * Hq * DV + (size_t)row_head[qb] * DV + 4 * grp;
 #pragma unroll
-    for (int nb = 0; nb < D / 16; ++nb) {
+    for (int nb = 0; nb < DV / 16; ++nb) {
       union {
         uint2 u;
         bf16_t e[4];
       } pk;
 #pragma unroll
       for (int j = 0; j < 4; ++j)
-        pk.e[j] = float_to_bf16(acc[qb][nb][j] * inv Q3_OPEN(row_tok[qb], row_head[qb], D, 16 * nb + 4 * grp + j));
+        pk.e[j] = float_to_bf16(acc[qb][nb][j] * inv Q3_OPEN(row_tok[qb], row_head[qb], DV, 16 * nb + 4 * grp + j));
       *reinterpret_cast<uint2*>(o + 16 * nb) = pk.u;
     }
   }
@@ -1772,7 +1940,7 @@ static int prompt_tokens_per_block(int total_tokens, int G, int Hkv, int key_spl
   return tpb;
 }
 
-template <int D>
+template <int D, int DV = D>
 static int launch_fast(const void* q, int q_stride, void* out, const void* k_cache, const void* v_cache,
                        int num_pages, const int* block_table, int bt_stride, const int* cu_q, const int* kv_lens,
                        int B, int total_tokens, int Hq, int Hkv, int page, float scale, int window, int max_q_len,
@@ -1780,6 +1948,9 @@ static int launch_fast(const void* q, int q_stride, void* out, const void* k_cac
                        const float* sink, hipStream_t stream) {
   const int G = Hq / Hkv;
   const score_scale_t scale_log2 = make_score_scale(scale);
+  const span_t span = make_span(window);
+  // keys of 192 numbers: tiles of 32, so that two blocks still share a CU's shared memory
+  constexpr int TILE = D > 128 ? 32 : PF_TILE;
 #ifdef Q3_POOLED
   if (window <= 0 || g_runs.k == nullptr || g_runs.pool <= 0) return Q3_ERR_BAD_ARGUMENT;
 #endif
@@ -1787,7 +1958,7 @@ static int launch_fast(const void* q, int q_stride, void* out, const void* k_cac
   if (window != 0 || g_score_bias == nullptr || sink != nullptr) return Q3_ERR_BAD_ARGUMENT;
 #endif
   if (min_q_len * G <= 16) {
-#ifndef Q3_POOLED
+#if !defined(Q3_POOLED) && !defined(Q3_SPAN)
     if (window == 0)
       hipLaunchKernelGGL((attn_decode_kernel<D, false, float, true>), dim3(splits, Hkv, B), dim3(256), 0, stream,
                          (const bf16_t*)q, q_stride, (bf16_t*)out, (const bf16_t*)k_cache, (const bf16_t*)v_cache,
@@ -1795,12 +1966,12 @@ static int launch_fast(const void* q, int q_stride, void* out, const void* k_cac
                          ws_acc, ws_ml, DecodePrep{}, sink Q3_BIAS_ARG Q3_RUNS_ARG Q3_GATE_ARG);
     else
 #endif
-      hipLaunchKernelGGL((attn_decode_kernel<D, false, float, false>), dim3(splits, Hkv, B), dim3(256), 0, stream,
+      hipLaunchKernelGGL((attn_decode_kernel<D, false, float, false, DV>), dim3(splits, Hkv, B), dim3(256), 0, stream,
                          (const bf16_t*)q, q_stride, (bf16_t*)out, (const bf16_t*)k_cache, (const bf16_t*)v_cache,
-                         num_pages, block_table, bt_stride, cu_q, kv_lens, Hq, Hkv, page, scale_log2, window, splits,
+                         num_pages, block_table, bt_stride, cu_q, kv_lens, Hq, Hkv, page, scale_log2, span, splits,
                          ws_acc, ws_ml, DecodePrep{}, sink Q3_BIAS_ARG Q3_RUNS_ARG Q3_GATE_ARG);
     if (splits > 1)
-      hipLaunchKernelGGL(attn_decode_reduce_kernel<D>, dim3(Hkv, B), dim3(256), 0, stream, (bf16_t*)out, cu_q, Hq,
+      hipLaunchKernelGGL(attn_decode_reduce_kernel<DV>, dim3(Hkv, B), dim3(256), 0, stream, (bf16_t*)out, cu_q, Hq,
                          Hkv, splits, ws_acc, ws_ml, sink Q3_GATE_ARG);
   }
   if (max_q_len * G > 16) {
@@ -1808,19 +1979,19 @@ static int launch_fast(const void* q, int q_stride, void* out, const void* k_cac
     const int tiles = (max_q_len + tokens_per_block - 1) / tokens_per_block;
     if (tiles * key_splits > 65535) return Q3_ERR_UNSUPPORTED;
     float* part_acc = prompt_ws;
-    float* part_ml = prompt_ws ? prompt_ws + (size_t)total_tokens * Hq * key_splits * D : nullptr;
-    hipLaunchKernelGGL((attn_prefill_kernel<D, PF_TILE, PF_STAGES>), dim3(Hkv, tiles * key_splits, B), dim3(256), 0,
+    float* part_ml = prompt_ws ? prompt_ws + (size_t)total_tokens * Hq * key_splits * DV : nullptr;
+    hipLaunchKernelGGL((attn_prefill_kernel<D, TILE, PF_STAGES, DV>), dim3(Hkv, tiles * key_splits, B), dim3(256), 0,
                        stream, (const bf16_t*)q, q_stride, (bf16_t*)out, (const bf16_t*)k_cache,
                        (const bf16_t*)v_cache, num_pages, block_table, bt_stride, cu_q, kv_lens, Hq, Hkv, page,
-                       scale_log2, window, tokens_per_block, key_splits, part_acc, part_ml, sink Q3_BIAS_ARG Q3_RUNS_ARG Q3_GATE_ARG);
+                       scale_log2, span, tokens_per_block, key_splits, part_acc, part_ml, sink Q3_BIAS_ARG Q3_RUNS_ARG Q3_GATE_ARG);
     if (key_splits > 1)
-      hipLaunchKernelGGL(attn_prefill_merge_kernel<D>, dim3(max_q_len, B), dim3(256), 0, stream,
+      hipLaunchKernelGGL(attn_prefill_merge_kernel<DV>, dim3(max_q_len, B), dim3(256), 0, stream,
                          (bf16_t*)out, cu_q, Hq, Hkv, key_splits, part_acc, part_ml, sink Q3_GATE_ARG);
   }
   return q3_launch_status();
 }
 
-#if !defined(Q3_POOLED) && !defined(Q3_SIGMOID)
+#if !defined(Q3_POOLED) && !defined(Q3_SIGMOID) && !defined(Q3_SPAN)
 template <int D, typename W>
 static int launch_decode_prep(const void* qkv, void* out, const void* k_cache, const void* v_cache, int num_pages,
                               const int* block_table, int bt_stride, const int* cu_q, const int* kv_lens, int B,
@@ -1847,13 +2018,30 @@ static int launch_decode_prep(const void* qkv, void* out, const void* k_cache, c
 // Whether the matrix-core kernels take this problem; otherwise the general kernel does.
 extern "C" int q3_paged_attention_fast_path(int Hq, int Hkv, int D, int page, int dtype) {
   if (dtype != Q3_BF16) return 0;
+#ifdef Q3_SPAN
+  if (D != 64 && D != 96 && D != 128 && D != 192) return 0;
+#else
   if (D != 64 && D != 128) return 0;
+#endif
   if (page < 16 || (page & (page - 1))) return 0;  // a power of two, at least 16
   if (Hq % Hkv || Hq / Hkv > 16) return 0;
   return 1;
 }
 
-// Floats of workspace the split decoding needs: accumulators, then (max, sum) pairs.
+#ifdef Q3_SPAN
+// Whether the kernels are built for keys of D numbers with values of DV.
+extern "C" int q3_span_attention_sizes(int D, int DV) {
+  switch (D) {
+    case 64: return DV == 64 || DV == 128;
+    case 96: return DV == 64 || DV == 96;
+    case 128: return DV == 64 || DV == 128;
+    case 192: return DV == 128;
+  }
+  return 0;
+}
+#endif
+
+// Floats of workspace the split decoding needs: accumulators, then (max, sum) pairs (`D` the values' size).
 extern "C" long q3_paged_attention_workspace(int B, int Hkv, int D, int splits) {
   return splits > 1 ? (long)B * Hkv * splits * 16 * (D + 2) : 0;
 }
@@ -1887,6 +2075,29 @@ extern "C" int q3_paged_attention(const void* q, int q_stride, void* out, const 
       return Q3_ERR_BAD_ARGUMENT;
     (void)max_kv_len;
     float* ws_acc = workspace;
+#ifdef Q3_SPAN
+    const int DV = g_span_value_dim;
+    if (!q3_span_attention_sizes(D, DV) || window < 0 || g_span_chunk < 0 || g_span_keep < 0 || (window > 0 && g_span_chunk > 0))
+      return Q3_ERR_BAD_ARGUMENT;
+    float* ws_ml = workspace ? workspace + (size_t)B * Hkv * splits * 16 * DV : nullptr;
+#define Q3_SPAN_LAUNCH(KD, VD)                                                                                           \
+  if (D == KD && DV == VD)                                                                                               \
+  return launch_fast<KD, VD>(q, q_stride, out, k_cache, v_cache, num_pages, block_table, bt_stride, cu_q, kv_lens, B, T_, \
+                             Hq, Hkv, page, scale, window, max_q_len, min_q_len, splits, ws_acc, ws_ml, prompt_splits,    \
+                             prompt_workspace, sink, stream)
+    Q3_SPAN_LAUNCH(64, 64);
+    Q3_SPAN_LAUNCH(64, 128);
+    Q3_SPAN_LAUNCH(96, 64);
+    Q3_SPAN_LAUNCH(96, 96);
+    Q3_SPAN_LAUNCH(128, 64);
+    Q3_SPAN_LAUNCH(128, 128);
+    Q3_SPAN_LAUNCH(192, 128);
+#undef Q3_SPAN_LAUNCH
+    return Q3_ERR_UNSUPPORTED;
+  }
+  return Q3_ERR_UNSUPPORTED;
+}
+#else
     float* ws_ml = workspace ? workspace + (size_t)B * Hkv * splits * 16 * D : nullptr;
     if (D == 64)
       return launch_fast<64>(q, q_stride, out, k_cache, v_cache, num_pages, block_table, bt_stride, cu_q, kv_lens,
@@ -1904,8 +2115,9 @@ extern "C" int q3_paged_attention(const void* q, int q_stride, void* out, const 
                                                         D, page, scale, window, max_q_len, sink, stream));
   return Q3_ERR_BAD_ARGUMENT;
 }
+#endif
 
-#if !defined(Q3_POOLED) && !defined(Q3_SIGMOID)
+#if !defined(Q3_POOLED) && !defined(Q3_SIGMOID) && !defined(Q3_SPAN)
 // Whether `q3_decode_attention` takes a step of single tokens with these sizes: what the
 // matrix-core kernels take, with a rotation (if any) over the whole head.
 extern "C" int q3_decode_attention_takes(int Hq, int Hkv, int D, int page, int dtype, int rotary_dim) {

@@ -31,13 +31,14 @@ __device__ inline float moe_gated(float g, float u, int act) {
 // is. `mode` 2: s = sigmoid(z); the choice goes by c = s + correction[e] and only among the experts of
 // `keep` of the `groups` equal groups of neighbours, those whose two largest c sum highest (the lowest
 // group among equals; the others' c count as minus infinity); weight_k = s_k as it is, without the
-// correction. Every lane holds every reduced number; what one lane writes to shared memory and
+// correction. `mode` 3: the same choice with s = softmax(z) over all E and a group judged by its largest c;
+// weight_k = s_k / (sum of the chosen s + 1e-20). Weights are multiplied by `scale`. Every lane holds every reduced number; what one lane writes to shared memory and
 // another reads is separated by the wavefront's barrier.
 // ---------------------------------------------------------------------------
 __global__ __launch_bounds__(256) void moe_pick_kernel(const float* __restrict__ logits, long row_stride, int n_tokens,
                                                        int E, int top, int mode, const float* __restrict__ correction,
-                                                       int groups, int keep, int* __restrict__ chosen,
-                                                       float* __restrict__ weights) {
+                                                       int groups, int keep, float scale,
+                                                       int* __restrict__ chosen, float* __restrict__ weights) {
   extern __shared__ float smem[];
   const int wave = threadIdx.x / Q3_WAVE, lane = threadIdx.x % Q3_WAVE;
   const int t = blockIdx.x * (blockDim.x / Q3_WAVE) + wave;
@@ -46,9 +47,8 @@ __global__ __launch_bounds__(256) void moe_pick_kernel(const float* __restrict__
   float* picked = z + E;
   float* group_score = picked + top;
   const float* src = logits + (size_t)t * row_stride;
-  float total = 1.f;
-  if (mode == 0) {
-    float biggest = -INFINITY;
+  float total = 1.f, biggest = -INFINITY;
+  if (mode == 0 || mode == 3) {
     for (int e = lane; e < E; e += Q3_WAVE) biggest = fmaxf(biggest, src[e]);
     biggest = wave_max(biggest);
     total = 0.f;
@@ -58,15 +58,17 @@ __global__ __launch_bounds__(256) void moe_pick_kernel(const float* __restrict__
       total += p;
     }
     total = wave_sum(total);
+    if (mode == 3)                                           // a lane reads what it wrote itself
+      for (int e = lane; e < E; e += Q3_WAVE) z[e] = z[e] / total + correction[e];
   } else if (mode == 1) {
     for (int e = lane; e < E; e += Q3_WAVE) z[e] = src[e];
   } else {
     for (int e = lane; e < E; e += Q3_WAVE) z[e] = 1.f / (1.f + expf(-src[e])) + correction[e];
   }
   __builtin_amdgcn_wave_barrier();
-  if (mode == 2 && keep < groups) {
+  if (mode >= 2 && keep < groups) {
     const int size = E / groups;
-    for (int g = lane; g < groups; g += Q3_WAVE) {          // a group a lane: the sum of its two largest
+    for (int g = lane; g < groups; g += Q3_WAVE) {          // a group a lane: the sum of its two largest, or its largest
       float first = -INFINITY, second = -INFINITY;
       for (int i = 0; i < size; ++i) {
         const float c = z[g * size + i];
@@ -77,7 +79,7 @@ __global__ __launch_bounds__(256) void moe_pick_kernel(const float* __restrict__
           second = c;
         }
       }
-      group_score[g] = size > 1 ? first + second : first;
+      group_score[g] = mode == 2 && size > 1 ? first + second : first;
     }
     __builtin_amdgcn_wave_barrier();
     // an expert stays if fewer than `keep` groups stand before its own (a higher score, or an equal one
@@ -116,7 +118,9 @@ __global__ __launch_bounds__(256) void moe_pick_kernel(const float* __restrict__
       }
     }
     if (at >= E) at = 0;          // logits that are no numbers: stay inside the operands
-    const float score = mode == 0 ? best / total : 1.f / (1.f + expf(-(mode == 1 ? best : src[at])));
+    const float score = mode == 0   ? best / total
+                        : mode == 3 ? expf(src[at] - biggest) / total
+                                    : 1.f / (1.f + expf(-(mode == 1 ? best : src[at])));
     picked_sum += score;
     __builtin_amdgcn_wave_barrier();
     picked[k] = score;
@@ -124,12 +128,13 @@ __global__ __launch_bounds__(256) void moe_pick_kernel(const float* __restrict__
     if (lane == 0) chosen[(size_t)t * top + k] = at;
     __builtin_amdgcn_wave_barrier();
   }
-  const float inv = mode == 0 ? 1.f / (picked_sum + 1e-20f) : 1.f;
+  const float inv = mode == 0 || mode == 3 ? scale / (picked_sum + 1e-20f) : scale;
   for (int k = lane; k < top; k += Q3_WAVE) weights[(size_t)t * top + k] = picked[k] * inv;
 }
 
 // ---------------------------------------------------------------------------
-// Pairs in the order of their experts. One block. `chosen` (P) names each pair's expert.
+// Pairs in the order of their experts. One block. `chosen` (P) names each pair's expert; a pair of a number
+// that is no expert's (a choice that gives its input back) gets no slot, slot_of_pair -1.
 //   offsets[e] .. offsets[e+1]: the slots of expert e;  pair_of_slot[slot] = pair;
 //   slot_of_pair[pair] = slot;  tiles of `tile_rows` slots that never cross an expert's end:
 //   tile_expert[i], tile_first[i] (first slot), n_tiles[0].
@@ -171,6 +176,8 @@ __global__ void moe_align_kernel(const int* __restrict__ chosen, int P, int E, i
       const int slot = atomicAdd(&cursor[e], 1);
       pair_of_slot[slot] = p;
       slot_of_pair[p] = slot;
+    } else {
+      slot_of_pair[p] = -1;
     }
   }
 }
@@ -632,10 +639,12 @@ __global__ __launch_bounds__(64 * GT_WM * 2) void moe_linear_tiles_kernel(
 // out[t, :] = sum_k weights[t, k] * y[slot_of_pair[t * top + k], :] (+ shared[t, :]), float32 sums in
 // the order k = 0, 1, ..., the shared expert last; rounded once. Without `weights` every weight is 1
 // (experts whose inputs carried the weight). With `shared_gate` (one float32 logit per token, the
-// tokens' `gate_stride` apart) the shared row is multiplied by sigmoid(shared_gate[t]).
+// tokens' `gate_stride` apart) the shared row is multiplied by sigmoid(shared_gate[t]). A pair without a slot
+// counts with the token's own row of `self`, its input, or not at all where there is no `self`.
 template <typename T>
 __global__ void moe_combine_kernel(const T* __restrict__ y, const int* __restrict__ slot_of_pair,
-                                   const float* __restrict__ weights, const T* __restrict__ shared,
+                                   const float* __restrict__ weights, const T* __restrict__ self,
+                                   const T* __restrict__ shared,
                                    const float* __restrict__ shared_gate, long gate_stride,
                                    T* __restrict__ out, int width, int top) {
   __shared__ int slots[64];
@@ -650,9 +659,12 @@ __global__ void moe_combine_kernel(const T* __restrict__ y, const int* __restric
   const int j = blockIdx.y * blockDim.x + threadIdx.x;
   if (j >= width) return;
   float acc = 0.f;
-  for (int k = 0; k < kept; ++k) acc += share[k] * to_float(y[(size_t)slots[k] * width + j]);
-  for (int k = kept; k < top; ++k)
-    acc += (weights ? weights[(size_t)t * top + k] : 1.f) * to_float(y[(size_t)slot_of_pair[(size_t)t * top + k] * width + j]);
+  const float own = self ? to_float(self[(size_t)t * width + j]) : 0.f;
+  for (int k = 0; k < kept; ++k) acc += share[k] * (slots[k] < 0 ? own : to_float(y[(size_t)slots[k] * width + j]));
+  for (int k = kept; k < top; ++k) {
+    const int slot = slot_of_pair[(size_t)t * top + k];
+    acc += (weights ? weights[(size_t)t * top + k] : 1.f) * (slot < 0 ? own : to_float(y[(size_t)slot * width + j]));
+  }
   if (shared) {
     const float open = shared_gate ? 1.f / (1.f + expf(-shared_gate[(size_t)t * gate_stride])) : 1.f;
     acc += open * to_float(shared[(size_t)t * width + j]);
@@ -661,17 +673,17 @@ __global__ void moe_combine_kernel(const T* __restrict__ y, const int* __restric
 }
 
 extern "C" int q3_moe_pick(const float* logits, long row_stride, int n_tokens, int E, int top, int mode,
-                           const float* correction, int groups, int keep, int* chosen, float* weights,
+                           const float* correction, int groups, int keep, float scale, int* chosen, float* weights,
                            hipStream_t stream) {
-  if (n_tokens <= 0 || E <= 0 || top <= 0 || top > E || E > 4096 || mode < 0 || mode > 2 || row_stride < E)
+  if (n_tokens <= 0 || E <= 0 || top <= 0 || top > E || E > 4096 || mode < 0 || mode > 3 || row_stride < E)
     return Q3_ERR_BAD_ARGUMENT;
-  if (mode != 2) groups = keep = 1;
-  if (mode == 2 && (!correction || groups <= 0 || E % groups || keep <= 0 || keep > groups || top > keep * (E / groups)))
+  if (mode < 2) groups = keep = 1;
+  if (mode >= 2 && (!correction || groups <= 0 || E % groups || keep <= 0 || keep > groups || top > keep * (E / groups)))
     return Q3_ERR_BAD_ARGUMENT;
   const int waves = 4;
   const size_t smem = (size_t)waves * (E + top + groups) * sizeof(float);
   hipLaunchKernelGGL(moe_pick_kernel, dim3((n_tokens + waves - 1) / waves), dim3(waves * Q3_WAVE), smem, stream, logits,
-                     row_stride, n_tokens, E, top, mode, correction, groups, keep, chosen, weights);
+                     row_stride, n_tokens, E, top, mode, correction, groups, keep, scale, chosen, weights);
   return q3_launch_status();
 }
 
@@ -753,7 +765,7 @@ extern "C" int q3_moe_linear(const void* x, const int* pair_of_slot, int gather,
   return q3_launch_status();
 }
 
-extern "C" int q3_moe_combine(const void* y, const int* slot_of_pair, const float* weights, const void* shared,
+extern "C" int q3_moe_combine(const void* y, const int* slot_of_pair, const float* weights, const void* self, const void* shared,
                               const float* shared_gate, long gate_stride, void* out, int n_tokens, int width, int top,
                               int dtype, hipStream_t stream) {
   if (n_tokens <= 0 || width <= 0 || top <= 0 || (shared_gate && !shared)) return Q3_ERR_BAD_ARGUMENT;
@@ -763,7 +775,7 @@ extern "C" int q3_moe_combine(const void* y, const int* slot_of_pair, const floa
   Q3_DISPATCH_DTYPE(dtype, TT,
                     hipLaunchKernelGGL(moe_combine_kernel<TT>, dim3(n_tokens, (width + threads - 1) / threads),
                                        dim3(threads), 0, stream, (const TT*)y,
-                                       slot_of_pair, weights, (const TT*)shared, shared_gate, gate_stride, (TT*)out,
+                                       slot_of_pair, weights, (const TT*)self, (const TT*)shared, shared_gate, gate_stride, (TT*)out,
                                        width, top));
   return q3_launch_status();
 }

@@ -69,12 +69,16 @@ __global__ void softcap_prepare_kernel(const float* __restrict__ rows, long row_
   }
 }
 
-// Queries, keys and values without norms, turned by the position, i and i + half together. grid (T,
+// Queries, keys and values turned by the position, i and i + half together. grid (T,
 // shares): a token's heads (queries', then keys') go over the wavefronts of its blocks in turn. The row is [q: H dim | k: G dim | v: G vdim | ...] float32,
 // `bias` covers q, k and v (null: none); with `values_are_keys` there is no v and a token's value is
 // its key before it turns. The first 2 * half numbers of every head of q and k turn by position *
 // inv_freq[i], cos and sin multiplied by `factor`; they are formed once per token, in shared memory. q
 // goes to `q_out`, k and v into the token's place in the cache.
+//
+// `norm.on`: a head of q or k is divided by its own root mean square and multiplied by `q_weight` or
+// `k_weight` (dim numbers that the heads share; null: by nothing) before it turns. `mix.first`: a token's
+// value is (1 - share) v + share first, first's rows [G vdim] a stride apart.
 //
 // `runs` (single tokens only): a token that ends a run of `pool` tokens also leaves the means of the
 // run's keys and values, as the cache holds them, in the run's place: the others' are read from the
@@ -85,6 +89,17 @@ struct RunPlaces {
   void* v;               // (pages, G, vdim, page)
   const int* table;
   int width, pool;
+};
+struct HeadNorm {
+  int on;
+  float eps;
+  const float* q_weight;
+  const float* k_weight;
+};
+struct ValueMix {
+  const float* first;
+  long stride;
+  const float* share;
 };
 
 // The sum of one number of a head over tokens first .. last - 1, in their order, from a paged cache: token j's
@@ -115,7 +130,7 @@ __global__ void __launch_bounds__(256) turn_prepare_kernel(
     const float* __restrict__ rows, long row_stride, const float* __restrict__ bias, const float* __restrict__ inv_freq,
     int half, float factor, const int* __restrict__ positions, const int* __restrict__ seq_index,
     const int* __restrict__ block_table, int table_width, TA* k_cache, TA* v_cache, int page, TA* __restrict__ q_out,
-    int H, int G, int dim, int vdim, int values_are_keys, RunPlaces runs) {
+    int H, int G, int dim, int vdim, int values_are_keys, RunPlaces runs, HeadNorm norm, ValueMix mix) {
   __shared__ float cs[Q3_TURN_HALF_MOST], sn[Q3_TURN_HALF_MOST];
   const int t = blockIdx.x;
   const int lane = threadIdx.x % Q3_WAVE, waves = blockDim.x / Q3_WAVE * gridDim.y;
@@ -139,25 +154,38 @@ __global__ void __launch_bounds__(256) turn_prepare_kernel(
     run_off = r % page;
   }
   __syncthreads();
-  auto turned = [&](const float* x, const float* add, int e) {
-    const float own = x[e] + (add ? add[e] : 0.f);
+  // the factor of a head's numbers: one over its root mean square, in every lane
+  auto head_scale = [&](const float* x, const float* add) {
+    if (!norm.on) return 1.f;
+    float acc = 0.f;
+    for (int e = lane; e < dim; e += Q3_WAVE) {
+      const float z = x[e] + (add ? add[e] : 0.f);
+      acc += z * z;
+    }
+    return rsqrtf(wave_sum(acc) / (float)dim + norm.eps);
+  };
+  auto turned = [&](const float* x, const float* add, float scale, const float* weight, int e) {
+    const float own = (x[e] + (add ? add[e] : 0.f)) * (weight ? scale * weight[e] : scale);
     if (e >= 2 * half) return own;
     const int p = e < half ? e + half : e - half;
-    const float other = x[p] + (add ? add[p] : 0.f);
+    const float other = (x[p] + (add ? add[p] : 0.f)) * (weight ? scale * weight[p] : scale);
     return e < half ? own * cs[e] - other * sn[e] : own * cs[p] + other * sn[p];
   };
   for (int h = wave; h < H; h += waves) {
     const float* x = row + h * dim;
     const float* add = bias ? bias + h * dim : nullptr;
-    for (int e = lane; e < dim; e += Q3_WAVE) q_out[(size_t)t * nq + h * dim + e] = from_float<TA>(turned(x, add, e));
+    const float scale = head_scale(x, add);
+    for (int e = lane; e < dim; e += Q3_WAVE)
+      q_out[(size_t)t * nq + h * dim + e] = from_float<TA>(turned(x, add, scale, norm.q_weight, e));
   }
   if (pg < 0) return;
   int g = wave - H % waves;                    // the wavefront after the last query head's takes the first key head
   for (g = g < 0 ? g + waves : g; g < G; g += waves) {
     const float* x = row + nq + g * dim;
     const float* add = bias ? bias + nq + g * dim : nullptr;
+    const float scale = head_scale(x, add);
     for (int e = lane; e < dim; e += Q3_WAVE) {
-      const TA key = from_float<TA>(turned(x, add, e));
+      const TA key = from_float<TA>(turned(x, add, scale, norm.k_weight, e));
       k_cache[(((size_t)pg * G + g) * page + off) * dim + e] = key;
       if (run_page >= 0) {
         const float sum = sum_over_tokens<TA>(k_cache, table, pos - runs.pool + 1, pos, page, G, g, (size_t)page * dim, e, dim) +
@@ -168,7 +196,9 @@ __global__ void __launch_bounds__(256) turn_prepare_kernel(
     const float* y = values_are_keys ? x : row + nq + nk + g * vdim;
     const float* add_v = values_are_keys ? add : (bias ? bias + nq + nk + g * vdim : nullptr);
     for (int e = lane; e < vdim; e += Q3_WAVE) {
-      const TA value = from_float<TA>(y[e] + (add_v ? add_v[e] : 0.f));
+      float own = y[e] + (add_v ? add_v[e] : 0.f);
+      if (mix.first) own = (1.f - *mix.share) * own + *mix.share * mix.first[(size_t)t * mix.stride + g * vdim + e];
+      const TA value = from_float<TA>(own);
       v_cache[(((size_t)pg * G + g) * vdim + e) * page + off] = value;
       if (run_page >= 0) {
         const float sum = sum_over_tokens<TA>(v_cache, table, pos - runs.pool + 1, pos, page, G, g, (size_t)page * vdim,
@@ -184,13 +214,19 @@ extern "C" int q3_turn_prepare(const float* rows, long row_stride, const float* 
                                float factor, const int* positions, const int* seq_index, const int* block_table,
                                int table_width, void* k_cache, void* v_cache, int page, void* q_out, int T, int H, int G,
                                int dim, int vdim, int values_are_keys, void* run_k, void* run_v, const int* run_table,
-                               int run_width, int pool, int act_dtype, hipStream_t stream) {
+                               int run_width, int pool, int norm_on, float norm_eps, const float* q_weight,
+                               const float* k_weight, const float* mix_first, long mix_stride, const float* mix_share,
+                               int act_dtype, hipStream_t stream) {
   if (T <= 0 || H <= 0 || G <= 0 || H % G || dim <= 0 || vdim <= 0 || half < 0 || 2 * half > dim || !k_cache || !v_cache ||
       !block_table || page <= 0 || table_width <= 0 || (half > 0 && !inv_freq) || (values_are_keys && dim != vdim))
     return Q3_ERR_BAD_ARGUMENT;
   if (run_k && (!run_v || !run_table || run_width <= 0 || pool <= 0)) return Q3_ERR_BAD_ARGUMENT;
+  if ((mix_first && (!mix_share || values_are_keys)) || (q_weight == nullptr) != (k_weight == nullptr) || (q_weight && !norm_on))
+    return Q3_ERR_BAD_ARGUMENT;
   if (half > Q3_TURN_HALF_MOST) return Q3_ERR_UNSUPPORTED;
   const RunPlaces runs{run_k, run_v, run_table, run_width, pool};
+  const HeadNorm norm{norm_on, norm_eps, q_weight, k_weight};
+  const ValueMix mix{mix_first, mix_stride, mix_share};
   // few tokens: a wavefront per head; many: the tokens fill the chip, and share their cosines among more heads
   const int most = (H + G + 3) / 4;
   const int shares = T >= 1024 ? 1 : (T >= 256 ? (most < 2 ? most : 2) : (most < 64 ? most : 64));
@@ -198,7 +234,7 @@ extern "C" int q3_turn_prepare(const float* rows, long row_stride, const float* 
                     hipLaunchKernelGGL(turn_prepare_kernel<TA>, dim3(T, shares), dim3(256), 0, stream, rows, row_stride, bias,
                                        inv_freq, half, factor, positions, seq_index, block_table, table_width,
                                        (TA*)k_cache, (TA*)v_cache, page, (TA*)q_out, H, G, dim, vdim, values_are_keys,
-                                       runs));
+                                       runs, norm, mix));
   return q3_launch_status();
 }
 
@@ -261,13 +297,15 @@ extern "C" int q3_pool_runs(const void* k_cache, const void* v_cache, const int*
 // value and is not scaled. With `runs` the token also sees one key and value per run of `pool` tokens
 // that ends at its position minus the window or before, in the same softmax, ahead of the tokens.
 // With `score_bias` (H floats) there is no softmax: a key counts with sigmoid(score + score_bias[h]).
+// With `chunk` the token sees the keys of its own stretch of `chunk` positions, counted from the sequence's
+// first; the first `keep` keys are seen besides, ahead of the others.
 #define Q3_CAP_DIM_MOST 512
 #define Q3_CAP_VSLICES 8
 template <typename TA>
 __global__ void __launch_bounds__(64) softcap_attention_kernel(
     const TA* __restrict__ q, const TA* __restrict__ k_cache, const TA* __restrict__ v_cache,
     const int* __restrict__ block_table, int table_width, const int* __restrict__ seq_index,
-    const int* __restrict__ positions, float scale, float cap, int window, const float* __restrict__ gate,
+    const int* __restrict__ positions, float scale, float cap, int window, int chunk, int keep, const float* __restrict__ gate,
     long gate_stride, int gate_wide, TA* __restrict__ out, int H, int G, int dim, int vdim, int page, int v_transposed,
     const float* __restrict__ sink, RunPlaces runs, const float* __restrict__ score_bias) {
   __shared__ float sq[Q3_CAP_DIM_MOST];
@@ -334,8 +372,10 @@ __global__ void __launch_bounds__(64) softcap_attention_kernel(
     const int seen = (pos - window + 1) / runs.pool;
     walk((const TA*)runs.k, (const TA*)runs.v, runs.table + (size_t)seq_index[t] * runs.width, 0, seen - 1);
   }
-  walk(k_cache, v_cache, block_table + (size_t)seq_index[t] * table_width,
-       window > 0 ? (pos - window + 1 > 0 ? pos - window + 1 : 0) : 0, pos);
+  const int* table = block_table + (size_t)seq_index[t] * table_width;
+  const int lo = chunk > 0 ? pos - pos % chunk : (window > 0 ? max(0, pos - window + 1) : 0);
+  if (keep > 0 && lo > 0) walk(k_cache, v_cache, table, 0, min(keep, lo) - 1);
+  walk(k_cache, v_cache, table, lo, pos);
   if (sink) l += expf(sink[h] - m);
   const float norm = weighed ? 1.f : 1.f / l;
 #pragma unroll
@@ -444,7 +484,7 @@ extern "C" int q3_softcap_prepare(const float* rows, long row_stride, const floa
 // `run_k` null: no runs. `score_bias` null: a softmax.
 extern "C" int q3_softcap_attention(const void* q, const void* k_cache, const void* v_cache, const int* block_table,
                                     int table_width, const int* seq_index, const int* positions, float scale, float cap,
-                                    int window, const float* gate, long gate_stride, int gate_wide, void* out, int T,
+                                    int window, int chunk, int keep, const float* gate, long gate_stride, int gate_wide, void* out, int T,
                                     int H, int G, int dim, int vdim, int page, int v_transposed, const float* sink,
                                     const void* run_k, const void* run_v, const int* run_table, int run_width, int pool,
                                     const float* score_bias, int act_dtype, hipStream_t stream) {
@@ -454,12 +494,13 @@ extern "C" int q3_softcap_attention(const void* q, const void* k_cache, const vo
   if (run_k && (!run_v || !run_table || run_width <= 0 || pool <= 0 || window <= 0 || !v_transposed))
     return Q3_ERR_BAD_ARGUMENT;
   if (score_bias && (sink || run_k)) return Q3_ERR_BAD_ARGUMENT;
+  if (chunk < 0 || keep < 0 || (chunk > 0 && window > 0) || (run_k && (chunk > 0 || keep > 0))) return Q3_ERR_BAD_ARGUMENT;
   if (dim > Q3_CAP_DIM_MOST || vdim > 64 * Q3_CAP_VSLICES) return Q3_ERR_UNSUPPORTED;
   const RunPlaces runs{const_cast<void*>(run_k), const_cast<void*>(run_v), run_table, run_width, pool};
   Q3_DISPATCH_DTYPE(act_dtype, TA,
                     hipLaunchKernelGGL(softcap_attention_kernel<TA>, dim3(T, H), dim3(64), 0, stream, (const TA*)q,
                                        (const TA*)k_cache, (const TA*)v_cache, block_table, table_width, seq_index,
-                                       positions, scale, cap, window, gate, gate_stride, gate_wide, (TA*)out, H, G, dim,
+                                       positions, scale, cap, window, chunk, keep, gate, gate_stride, gate_wide, (TA*)out, H, G, dim,
                                        vdim, page, v_transposed, sink, runs, score_bias));
   return q3_launch_status();
 }

@@ -40,6 +40,7 @@ class StepBatch:
     max_kv_len_portions: int       # the same among the entries that bring more than one token
     q_lens: list                   # host copies
     kv_lens_host: list
+    carried: dict = field(default_factory=dict)    # what one layer leaves for later layers of the same step, by name
 
 
 @dataclass

@@ -123,7 +123,7 @@ class _DecodeGraph:
         storage = runner.storage
         self.description = DecodeDescription(
             B, widths, self.host, [storage.spare_page(g) for g in range(len(m.groups))], storage.spare_slot,
-            [grp.window > 0 for grp in m.groups])
+            [grp.gives_back for grp in m.groups])
         self.graph = None
         self.logits = None
         self.copied = torch.cuda.Event()

@@ -152,6 +152,7 @@ class DecoderModel:
                                                                next_norm=entry() if entry else None)
             if self.observer is not None:
                 self.observer(i, x, pending)
+        getattr(batch, "carried", {}).clear()     # what layers left for each other belongs to this pass alone
         h = self.final_norm.forward(x, delta=pending, rows=batch.logits_rows)
         return self.head.forward(h)
 

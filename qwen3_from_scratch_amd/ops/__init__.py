@@ -604,10 +604,10 @@ def _latent_splits(T, B, H, max_q_len, max_kv_len, window):
     return max(1, min(512 // tiles, keys // 128, 32))
 
 
-MOE_SCORING = {"softmax": 0, "sigmoid": 1, "sigmoid_groups": 2}
+MOE_SCORING = {"softmax": 0, "sigmoid": 1, "sigmoid_groups": 2, "softmax_groups": 3}
 
 
-def moe_route(h, router, top, tiled=None, scoring="softmax", correction=None, groups=1, keep=1, experts=None):
+def moe_route(h, router, top, tiled=None, scoring="softmax", correction=None, groups=1, keep=1, experts=None, scale=1.0):
     """Per token the `top` experts with the largest scores and their weights: h (T, width),
     router (E, width) of h's dtype (`tiled`: its tile-ordered copy, if the caller keeps one). The
     logits are a product with float32 sums and a float32 result; scores, the choice and the weights
@@ -617,33 +617,35 @@ def moe_route(h, router, top, tiled=None, scoring="softmax", correction=None, gr
     sigmoid(z) for itself and the weights are the chosen scores as they are. With "sigmoid_groups" the
     choice goes by sigmoid(z) + correction (`correction` float32 (E,)) and only among the experts of `keep`
     of the `groups` equal groups of neighbouring experts, those groups whose two largest such scores sum
-    highest; the weights are sigmoid(z) of the chosen, without the correction.
+    highest; the weights are sigmoid(z) of the chosen, without the correction. "softmax_groups": the same
+    with scores = softmax over all experts, a group judged by its largest score with the correction, and
+    weights divided by their sum as for "softmax". `scale` multiplies the weights.
 
     `experts`: the router's first `experts` rows are the experts'; what further rows it has are other
     numbers per token that ride on the same product (a gate, say), and their float32 results come back
     as a third value, (T, rows - experts) with rows apart."""
     _dev(h, router, correction)
-    _need(scoring in MOE_SCORING, "scoring is softmax or sigmoid")
+    _need(scoring in MOE_SCORING, "scoring is one of %s" % ", ".join(sorted(MOE_SCORING)))
     _need(h.dim() == 2 and router.dim() == 2 and h.shape[1] == router.shape[1] and h.dtype in _DT
           and router.dtype == h.dtype, "h (T, width) and router (E, width) of one dtype")
     T, rows = h.shape[0], router.shape[0]
     E = rows if experts is None else int(experts)
     _need(1 <= E <= rows and 1 <= top <= E, "experts must lie in 1..rows of the router, top in 1..experts")
-    if scoring == "sigmoid_groups":
+    if scoring.endswith("_groups"):
         _need(correction is not None, "the grouped choice needs a correction")
         _f32(correction, (E,), "correction")
         _need(groups >= 1 and E % groups == 0 and 1 <= keep <= groups and top <= keep * (E // groups),
               "groups divide the experts, keep lies in 1..groups, and the kept groups hold at least top experts")
     else:
-        _need(correction is None and groups == 1 and keep == 1, "a correction and groups belong to sigmoid_groups")
+        _need(correction is None and groups == 1 and keep == 1, "a correction and groups belong to the grouped scorings")
     chosen = torch.empty((T, top), dtype=torch.int32, device=h.device)
     weights = torch.empty((T, top), dtype=torch.float32, device=h.device)
     logits = None
     if T:
         logits = linear(h, router, out_dtype=torch.float32, tiled=tiled)
         _check(library("moe").q3_moe_pick(_ptr(logits), ctypes.c_long(rows), T, E, top, MOE_SCORING[scoring],
-                                          _ptr(correction), int(groups), int(keep), _ptr(chosen), _ptr(weights),
-                                          _stream()), "moe_route")
+                                          _ptr(correction), int(groups), int(keep), ctypes.c_float(scale), _ptr(chosen),
+                                          _ptr(weights), _stream()), "moe_route")
     if experts is None:
         return chosen, weights
     if logits is None:
@@ -693,7 +695,7 @@ def moe_experts(h, chosen, weights, up, down, shared=None, activation="erf"):
                                  GELU_KINDS[activation], _DT[h.dtype], stream), "moe_linear")
         _check(lib.q3_moe_linear(_ptr(hidden), _ptr(pair_of_slot), 0, 1, _ptr(down), _ptr(y), *tiles, width, ff, -1,
                                  _DT[h.dtype], stream), "moe_linear")
-    _check(lib.q3_moe_combine(_ptr(y), _ptr(slot_of_pair), _ptr(weights), _ptr(shared), None, ctypes.c_long(0), _ptr(out),
+    _check(lib.q3_moe_combine(_ptr(y), _ptr(slot_of_pair), _ptr(weights), None, _ptr(shared), None, ctypes.c_long(0), _ptr(out),
                               T, width, top, _DT[h.dtype], stream), "moe_combine")
     return out
 
@@ -752,7 +754,7 @@ def moe_gated_experts(h, chosen, weights, gate_up, down, limit, slope):
     else:
         _check(lib.q3_moe_linear(_ptr(hidden), _ptr(pair_of_slot), 0, 1, _ptr(down), _ptr(y), *tiles, width, ff, -1,
                                  _DT[h.dtype], stream), "moe_linear")
-    _check(lib.q3_moe_combine(_ptr(y), _ptr(slot_of_pair), None, None, None, ctypes.c_long(0), _ptr(out), T, width, top,
+    _check(lib.q3_moe_combine(_ptr(y), _ptr(slot_of_pair), None, None, None, None, ctypes.c_long(0), _ptr(out), T, width, top,
                               _DT[h.dtype], stream), "moe_combine")
     return out
 
@@ -760,14 +762,15 @@ def moe_gated_experts(h, chosen, weights, gate_up, down, limit, slope):
 _MOE_ACT_GATED = 2      # the experts' product kernels: epilogue codes from here on are gated units, in the order of GATE_KINDS
 
 
-def moe_glu_experts(h, chosen, weights, gate_up, down, activation="silu", shared=None, shared_gate=None):
+def moe_glu_experts(h, chosen, weights, gate_up, down, activation="silu", shared=None, shared_gate=None, identity=0):
     """sum_k weights[t, k] * down[e] (act(gate[e] h[t]) * (up[e] h[t])), e = chosen[t, k]: experts that are
     gated units without biases, weighted on their results. h (T, width), gate_up (E, 2 ff, width) with rows
     2j the gate's and 2j + 1 the other branch's, down (E, width, ff), `activation` one of `GATE_KINDS`;
     `shared` (T, width) is added last, multiplied by sigmoid(shared_gate[t]) when `shared_gate` (float32
     (T,) or (T, 1), rows possibly apart: a logit per token) is given. Returns (T, width). The pairs are
     sorted by expert on the GPU as in `moe_experts`; the gated unit is the epilogue of the first product,
-    from its float32 sums; a token's sum is formed in float32 in the order of its choices."""
+    from its float32 sums; a token's sum is formed in float32 in the order of its choices. With `identity`
+    choices may also be numbers E .. E + identity - 1, whose result is h[t] itself."""
     _dev(h, chosen, weights, gate_up, down, shared)
     T, width = h.shape
     E, ff = down.shape[0], down.shape[2]
@@ -776,6 +779,7 @@ def moe_glu_experts(h, chosen, weights, gate_up, down, activation="silu", shared
           and down.shape == (E, width, ff), "gate_up (E, 2 ff, width) and down (E, width, ff) of h's dtype")
     _need(chosen.shape == (T, top) and chosen.dtype == torch.int32 and weights.shape == (T, top)
           and weights.dtype == torch.float32 and weights.is_contiguous(), "chosen int32 (T, top), weights float32 (T, top)")
+    _need(not identity or h.is_contiguous(), "experts that give their input back need its rows side by side")
     _need(shared is None or (shared.shape == (T, width) and shared.dtype == h.dtype), "shared (T, width)")
     _need(activation in GATE_KINDS, "activation is one of %s" % ", ".join(sorted(GATE_KINDS)))
     gate_stride = 0
@@ -808,7 +812,7 @@ def moe_glu_experts(h, chosen, weights, gate_up, down, activation="silu", shared
     else:
         _check(lib.q3_moe_linear(_ptr(hidden), _ptr(pair_of_slot), 0, 1, _ptr(down), _ptr(y), *tiles, width, ff, -1,
                                  _DT[h.dtype], stream), "moe_linear")
-    _check(lib.q3_moe_combine(_ptr(y), _ptr(slot_of_pair), _ptr(weights), _ptr(shared), _ptr(shared_gate),
+    _check(lib.q3_moe_combine(_ptr(y), _ptr(slot_of_pair), _ptr(weights), _ptr(h) if identity else None, _ptr(shared), _ptr(shared_gate),
                               ctypes.c_long(gate_stride), _ptr(out), T, width, top, _DT[h.dtype], stream), "moe_combine")
     return out
 
@@ -1171,8 +1175,9 @@ def _runs_args(runs, kv_heads, page, dim, vdim, dtype):
 
 
 def turn_prepare(rows, bias, heads, kv_heads, dim, vdim, inv_freq, factor, positions, seq_index, out_dtype, block_table,
-                 k_cache, v_cache, values_are_keys=False, runs=None, cu_seqlens_q=None, kv_lens=None, max_q_len=0):
-    """Queries, keys and values of a step from the float32 rows of their joint product, without norms.
+                 k_cache, v_cache, values_are_keys=False, runs=None, cu_seqlens_q=None, kv_lens=None, max_q_len=0,
+                 norm_eps=None, q_weight=None, k_weight=None, mix=None):
+    """Queries, keys and values of a step from the float32 rows of their joint product.
 
     rows float32 (T, n) laid out [q: heads dim | k: kv_heads dim | v: kv_heads vdim | ...], rows possibly
     apart; bias float32 over q, k and v is added (None: none). With `values_are_keys` there is no v: a
@@ -1180,6 +1185,11 @@ def turn_prepare(rows, bias, heads, kv_heads, dim, vdim, inv_freq, factor, posit
     head of q and k turn by position * inv_freq[i], i and i + len(inv_freq) together, cos and sin
     multiplied by `factor`. Returns q (T, heads, dim) of `out_dtype`; keys (pages, kv_heads, page, dim)
     and values (pages, kv_heads, vdim, page) receive the tokens at their positions.
+
+    `norm_eps` (None: no norm): every head of q and k is divided by its own root mean square, eps inside the
+    root, and multiplied by `q_weight` or `k_weight`, float32 (dim,) shared by the heads (None: by nothing),
+    before it turns; a norm without weights is the same number behind the turn. `mix` = (first float32 (T,
+    kv_heads vdim), rows possibly apart; share float32 (1,)): a token's value is (1 - share) v + share first.
 
     `runs` (see `_runs_args`): every run of tokens that this step completes also leaves the means of its
     keys and values, as the cache holds them; `cu_seqlens_q`, `kv_lens` and `max_q_len` then say what the
@@ -1205,6 +1215,18 @@ def turn_prepare(rows, bias, heads, kv_heads, dim, vdim, inv_freq, factor, posit
     _need(k_cache.shape[1:] == (kv_heads, page, dim) and v_cache.dim() == 4 and v_cache.shape[1:] == (kv_heads, vdim, page)
           and k_cache.dtype == out_dtype and v_cache.dtype == out_dtype,
           "keys (pages, kv_heads, page, dim) and values (pages, kv_heads, vdim, page) of out_dtype")
+    _need(norm_eps is not None or (q_weight is None and k_weight is None), "weights belong to a norm")
+    _need((q_weight is None) == (k_weight is None), "weights for both of queries and keys, or for neither")
+    for weight in (q_weight, k_weight):
+        if weight is not None:
+            _f32(weight, (dim,), "q_weight and k_weight")
+    first, first_stride, share = None, 0, None
+    if mix is not None:
+        first, share = mix
+        first_stride = _rows_view(first, "the values that are mixed in")
+        _need(first.shape == (T, kv_heads * vdim) and first.dtype == torch.float32 and not values_are_keys and runs is None,
+              "values that are mixed in are float32 (T, kv_heads vdim), and values are not keys and have no runs")
+        _f32(share, (1,), "share")
     run_args = _runs_args(runs, kv_heads, page, dim, vdim, out_dtype)
     single = False
     if runs is not None:
@@ -1221,7 +1243,9 @@ def turn_prepare(rows, bias, heads, kv_heads, dim, vdim, inv_freq, factor, posit
             _ptr(rows), ctypes.c_long(rows.stride(0)), _ptr(bias), _ptr(inv_freq), half, ctypes.c_float(factor),
             _ptr(positions), _ptr(seq_index), _ptr(block_table), block_table.shape[1], _ptr(k_cache), _ptr(v_cache), page,
             _ptr(q), T, heads, kv_heads, dim, vdim, 1 if values_are_keys else 0,
-            *(run_args if single else (None, None, None, 0, 0)), _DT[out_dtype], _stream()), "turn_prepare")
+            *(run_args if single else (None, None, None, 0, 0)), 0 if norm_eps is None else 1,
+            ctypes.c_float(norm_eps or 0.0), _ptr(q_weight), _ptr(k_weight), _ptr(first), ctypes.c_long(first_stride),
+            _ptr(share), _DT[out_dtype], _stream()), "turn_prepare")
         if runs is not None and not single:
             _check(lib.q3_pool_runs(
                 _ptr(k_cache), _ptr(v_cache), _ptr(block_table), block_table.shape[1], _ptr(cu_seqlens_q), _ptr(kv_lens),
@@ -1318,7 +1342,7 @@ def channel_delta(conv, b_logits, a_logits, gate, dt_bias, a_log, norm_weight, e
 
 def softcap_attention(q, k_cache, v_cache, block_table, cu_seqlens_q, kv_lens, seq_index, positions, max_q_len,
                       max_kv_len, scale, softcap, window=0, gate=None, values_transposed=False, min_q_len=1,
-                      max_kv_len_of_many=None, sink=None, runs=None, sigmoid_bias=None):
+                      max_kv_len_of_many=None, sink=None, runs=None, sigmoid_bias=None, chunk=0, keep_first=0, span=False):
     """Causal softmax attention over a paged cache whose keys and values differ in size.
 
     q (T, heads, dim); keys (pages, kv_heads, page, dim), values (pages, kv_heads, page, vdim); the
@@ -1332,6 +1356,10 @@ def softcap_attention(q, k_cache, v_cache, block_table, cu_seqlens_q, kv_lens, s
     `runs` (see `_runs_args`; with a window and transposed values): the token at position i also sees one
     key and value per run of tokens that ends at i - window or before, in the same softmax.
     `sigmoid_bias` float32 (heads,): no softmax; a key counts with sigmoid(score + sigmoid_bias[h]).
+    `chunk` > 0 (in a window's place): the token at position i sees the keys j <= i with j // chunk == i //
+    chunk. `keep_first`: the keys at positions below it are seen whatever the window or chunk. `span` says
+    that bfloat16 of the sizes that `span_sizes` takes, keys and values of different sizes among them, is to
+    run on the matrix cores in the build for such spans (with transposed values).
 
     With `values_transposed` the values are (pages, kv_heads, vdim, page), and bfloat16 with equal key
     and value sizes of 64 or 128 then runs on the matrix cores, through the kernels of
@@ -1366,7 +1394,14 @@ def softcap_attention(q, k_cache, v_cache, block_table, cu_seqlens_q, kv_lens, s
         _dev(sigmoid_bias)
         _need(sink is None and runs is None and softcap == 0 and window == 0,
               "sigmoid weights take no sink, no runs, no cap and no window")
-    if T and values_transposed and dim == vdim and q.dtype == torch.bfloat16 \
+    spans = span or chunk > 0 or keep_first > 0
+    _need(not spans or (runs is None and sigmoid_bias is None and softcap == 0 and chunk >= 0 and keep_first >= 0
+                        and not (chunk and window)), "a span is a window or a chunk, without runs, sigmoid weights and a cap")
+    if T and spans and values_transposed and span_sizes(H, G, dim, vdim, page, q.dtype):
+        return paged_attention(q, H, k_cache, v_cache, block_table, cu_seqlens_q, kv_lens, max_q_len, max_kv_len, scale,
+                               window=window, min_q_len=min_q_len, max_kv_len_of_many=max_kv_len_of_many, sink=sink, gate=gate,
+                               span=(int(chunk), int(keep_first)))
+    if T and not spans and values_transposed and dim == vdim and q.dtype == torch.bfloat16 \
             and library("attention").q3_paged_attention_fast_path(H, G, dim, page, _DT[q.dtype]):
         out = paged_attention(q, H, k_cache, v_cache, block_table, cu_seqlens_q, kv_lens, max_q_len, max_kv_len, scale,
                               window=window, min_q_len=min_q_len, max_kv_len_of_many=max_kv_len_of_many, softcap=softcap,
@@ -1380,7 +1415,7 @@ def softcap_attention(q, k_cache, v_cache, block_table, cu_seqlens_q, kv_lens, s
     if T:
         _check(library("softcap").q3_softcap_attention(
             _ptr(q), _ptr(k_cache), _ptr(v_cache), _ptr(block_table), block_table.shape[1], _ptr(seq_index),
-            _ptr(positions), ctypes.c_float(scale), ctypes.c_float(softcap), int(window), _ptr(gate),
+            _ptr(positions), ctypes.c_float(scale), ctypes.c_float(softcap), int(window), int(chunk), int(keep_first), _ptr(gate),
             ctypes.c_long(stride), wide, _ptr(out), T, H, G, dim, vdim, page, 1 if values_transposed else 0, _ptr(sink),
             *run_args, _ptr(sigmoid_bias), _DT[q.dtype], _stream()), "softcap_attention")
     return out
@@ -1493,16 +1528,18 @@ def qk_norm_rope_store(qkv, num_q_heads, num_kv_heads, head_dim, positions, seq_
 
 def paged_attention(q, num_q_heads, k_cache, v_cache, block_table, cu_seqlens_q, kv_lens,
                     max_q_len, max_kv_len, scale, window=0, out=None, min_q_len=1, max_kv_len_of_many=None, softcap=0.0,
-                    sink=None, runs=None, sigmoid_bias=None, gate=None):
+                    sink=None, runs=None, sigmoid_bias=None, gate=None, span=None):
     """Causal softmax attention of packed query rows over paged keys and values.
     `softcap` > 0: a score s enters the softmax as softcap * tanh(s * scale / softcap); that form
     exists for the sizes the matrix cores take (a second build of the same kernels) and no other.
     `sink` float32 (Hq,): exp(sink[h]) joins the denominator of head h's softmax (no key, no value).
     `runs` (keys, values, block table, tokens per run; see `_runs_args`) with a window: a row at position p
     also sees one key and value per run that ends at p - window or before. `sigmoid_bias` float32 (Hq,): no
-    softmax, a key counts with sigmoid(s * scale + sigmoid_bias[h]). These two are builds of their own as well,
-    and they alone take `gate` float32 (T, Hq) or (T, Hq D), rows possibly apart, whose sigmoid multiplies the
-    result where it is written.
+    softmax, a key counts with sigmoid(s * scale + sigmoid_bias[h]). `span` = (chunk, keep_first): a row at
+    position p sees, instead of a window, the keys of its own stretch of `chunk` positions (0: what `window`
+    says), and the keys before `keep_first` besides; the values may differ from the keys in size
+    (`span_sizes`). These three are builds of their own as well, and they alone take `gate` float32 (T, Hq) or
+    (T, Hq D), rows possibly apart, whose sigmoid multiplies the result where it is written.
 
     q is (T, Hq, D) seen through a row stride (a view of the qkv buffer is
     fine). Keys are cached as (pages, Hkv, page, D), values as
@@ -1532,7 +1569,8 @@ def paged_attention(q, num_q_heads, k_cache, v_cache, block_table, cu_seqlens_q,
           "q and the caches must share bfloat16 or float32")
     _need(k_cache.dim() == 4 and k_cache.shape[3] == D, "the key cache must be (pages, Hkv, page, D)")
     Hkv, page = k_cache.shape[1], k_cache.shape[2]
-    _need(v_cache.shape == (k_cache.shape[0], Hkv, D, page), "the value cache must be (pages, Hkv, D, page)")
+    vdim = v_cache.shape[2] if span is not None and v_cache.dim() == 4 else D       # in that build alone they may differ
+    _need(v_cache.shape == (k_cache.shape[0], Hkv, vdim, page), "the value cache must be (pages, Hkv, D, page)")
     _need(Hq % Hkv == 0, "query heads must be a multiple of key heads")
     _need(D % 16 == 0 and 16 <= D <= 256, "head_dim must be a multiple of 16 in 16..256, found %d" % D)
     B = kv_lens.shape[0]
@@ -1543,17 +1581,17 @@ def paged_attention(q, num_q_heads, k_cache, v_cache, block_table, cu_seqlens_q,
     _need(block_table.shape[1] * page >= max_kv_len, "block_table is narrower than the longest sequence")
     _need(1 <= min_q_len <= max_q_len, "need 1 <= min_q_len <= max_q_len")
     if out is None:
-        out = torch.empty((T, Hq * D), dtype=q.dtype, device=q.device)
-    _need(out.shape == (T, Hq * D) and out.dtype == q.dtype, "out must be (T, Hq D)")
+        out = torch.empty((T, Hq * vdim), dtype=q.dtype, device=q.device)
+    _need(out.shape == (T, Hq * vdim) and out.dtype == q.dtype, "out must be (T, Hq D)")
     if T and B:
         kinds = [kind for kind, on in (("capped", softcap > 0), ("pooled", runs is not None),
-                                       ("sigmoid", sigmoid_bias is not None)) if on]
-        _need(len(kinds) <= 1, "capped scores, runs and sigmoid weights exclude each other")
+                                       ("sigmoid", sigmoid_bias is not None), ("span", span is not None)) if on]
+        _need(len(kinds) <= 1, "capped scores, runs, sigmoid weights and spans exclude each other")
         lib = library("_".join(["attention"] + kinds))
         if kinds:
             _need(lib.q3_paged_attention_fast_path(Hq, Hkv, D, page, _DT[q.dtype]) and q.stride(0) % 8 == 0,
                   "capped scores, runs and sigmoid weights need bfloat16, a head size of 64 or 128 and pages of a power "
-                  "of two from 16")
+                  "of two from 16; spans the sizes of span_sizes")
         if softcap > 0:
             lib.q3_set_score_cap.restype = None
             lib.q3_set_score_cap(ctypes.c_float(softcap))
@@ -1572,12 +1610,22 @@ def paged_attention(q, num_q_heads, k_cache, v_cache, block_table, cu_seqlens_q,
             _f32(sigmoid_bias, (Hq,), "sigmoid_bias")
             lib.q3_set_sigmoid_bias.restype = None
             lib.q3_set_sigmoid_bias(_ptr(sigmoid_bias))
-        _need(gate is None or runs is not None or sigmoid_bias is not None, "a gate comes with runs or sigmoid weights only")
-        if runs is not None or sigmoid_bias is not None:
+        if span is not None:
+            chunk, keep = int(span[0]), int(span[1])
+            _need(span_sizes(Hq, Hkv, D, vdim, page, q.dtype) and chunk >= 0 and keep >= 0 and not (chunk and window),
+                  "a span is a chunk or a window, and first keys, of sizes that span_sizes takes")
+            lib.q3_set_span.restype = None
+            lib.q3_set_span(chunk, keep, vdim)
+            if chunk or window:
+                visible = min(visible, (chunk or window) + keep)
+                longest = min(longest, (chunk or window) + keep)
+        _need(gate is None or runs is not None or sigmoid_bias is not None or span is not None,
+              "a gate comes with runs, sigmoid weights or spans only")
+        if runs is not None or sigmoid_bias is not None or span is not None:
             gate_stride = 0
             if gate is not None:
                 gate_stride = _rows_view(gate, "gate")
-                _need(gate.shape in ((T, Hq), (T, Hq * D)) and gate.dtype == torch.float32, "gate must be float32 (T, Hq) or (T, Hq D)")
+                _need(gate.shape in ((T, Hq), (T, Hq * vdim)) and gate.dtype == torch.float32, "gate must be float32 (T, Hq) or (T, Hq D)")
             lib.q3_set_gate.restype = None
             lib.q3_set_gate(_ptr(gate), ctypes.c_long(gate_stride), 1 if gate is not None and gate.shape[1] != Hq else 0)
         splits, workspace, prompt_splits, prompt_workspace = 1, None, 1, None
@@ -1586,12 +1634,12 @@ def paged_attention(q, num_q_heads, k_cache, v_cache, block_table, cu_seqlens_q,
                 splits = _splits(B, Hkv, visible)   # few rows per sequence: the keys go over several blocks
                 if splits > 1:
                     lib.q3_paged_attention_workspace.restype = ctypes.c_long
-                    n = lib.q3_paged_attention_workspace(B, Hkv, D, splits)
+                    n = lib.q3_paged_attention_workspace(B, Hkv, vdim, splits)
                     workspace = torch.empty((n,), dtype=torch.float32, device=q.device)
             if max_q_len * (Hq // Hkv) > 16:           # few long sequences over many keys: likewise
                 prompt_splits = lib.q3_paged_attention_prompt_splits(T, Hq, Hkv, int(longest))
                 if prompt_splits > 1:
-                    prompt_workspace = torch.empty((T * Hq * prompt_splits * (D + 2),), dtype=torch.float32,
+                    prompt_workspace = torch.empty((T * Hq * prompt_splits * (vdim + 2),), dtype=torch.float32,
                                                    device=q.device)
         _check(lib.q3_paged_attention(
             _ptr(q), q.stride(0), _ptr(out), _ptr(k_cache), _ptr(v_cache), k_cache.shape[0],
@@ -1601,6 +1649,15 @@ def paged_attention(q, num_q_heads, k_cache, v_cache, block_table, cu_seqlens_q,
             _stream()),
             "paged_attention")
     return out
+
+
+def span_sizes(heads, kv_heads, dim, vdim, page, dtype):
+    """Whether spans of these sizes run on the matrix cores (see `paged_attention`)."""
+    if dtype != torch.bfloat16:
+        return False
+    lib = library("attention_span")
+    return bool(lib.q3_paged_attention_fast_path(heads, kv_heads, dim, page, _DT[dtype])
+                and lib.q3_span_attention_sizes(dim, vdim))
 
 
 def _splits(B, Hkv, max_kv_len):

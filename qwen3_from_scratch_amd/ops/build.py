@@ -30,7 +30,7 @@ FLAGS = [
     "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
     "-Wno-unused-command-line-argument",
 ]
-MODULES = ("elementwise", "norm", "rotary", "attention", "attention_capped", "attention_pooled", "attention_sigmoid", "latent", "moe",
+MODULES = ("elementwise", "norm", "rotary", "attention", "attention_capped", "attention_pooled", "attention_sigmoid", "attention_span", "latent", "moe",
            "hyper", "recurrent", "mlstm", "delta", "softcap", "gemm", "matmul", "sampling", "probes")
 # what a module links besides the HIP runtime
 LINKS = {"matmul": ["-lhipblaslt"]}

@@ -246,7 +246,9 @@ class CacheNeed:
 
     paged: the tensors that grow by one element per token (`PagedTensor`s: for softmax
     attention a request's keys and values; another mixer may page one tensor, or tensors of
-    different widths), all tokens kept (window == 0) or the last `window`. state: a tensor of
+    different widths), all tokens kept (window == 0), the last `window`, or (`chunk` > 0) those of the
+    current stretch of `chunk` tokens, counted from a request's first; the first `keep_first` tokens
+    stay besides. state: a tensor of
     fixed `state_shape` and `state_dtype` per request. A mixer may need neither, either or
     both. Mixers whose needs are equal share page numbers: one block table serves them all.
 
@@ -259,12 +261,17 @@ class CacheNeed:
 
     paged: tuple = ()
     window: int = 0
+    chunk: int = 0
+    keep_first: int = 0
     state_shape: tuple = ()
     state_dtype: torch.dtype = torch.float32
     runs: tuple = ()
     run_length: int = 0
 
     def __post_init__(self):
+        if min(self.window, self.chunk, self.keep_first) < 0 or (self.window and self.chunk):
+            raise ValueError("a window or a chunk, neither negative; found window %d, chunk %d, keep_first %d"
+                             % (self.window, self.chunk, self.keep_first))
         object.__setattr__(self, "paged", tuple(self.paged))
         object.__setattr__(self, "runs", tuple(self.runs))
         if bool(self.runs) != (self.run_length > 0):

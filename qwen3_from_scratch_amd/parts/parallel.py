@@ -44,7 +44,7 @@ class ParallelMixers(Part):
             for t in need.paged:
                 paged.append(PagedTensor(name + "." + t.name, t.shape, t.token_axis, t.dtype))
             if need.paged:
-                windows.add(need.window)
+                windows.add((need.window, need.chunk, need.keep_first))
             if need.has_state:
                 if len(need.state_shape) != 1 or need.state_dtype != torch.float32:
                     raise ValueError("sides of a parallel mixer keep their state as one float32 vector")
@@ -52,8 +52,9 @@ class ParallelMixers(Part):
                 at += need.state_shape[0]
         if len(windows) > 1:
             raise ValueError("the sides of a parallel mixer page behind different windows")
-        return CacheNeed(paged=tuple(paged), window=windows.pop() if windows else 0, state_shape=(at,) if at else (),
-                         state_dtype=torch.float32)
+        window, chunk, keep_first = windows.pop() if windows else (0, 0, 0)
+        return CacheNeed(paged=tuple(paged), window=window, chunk=chunk, keep_first=keep_first,
+                         state_shape=(at,) if at else (), state_dtype=torch.float32)
 
     def tensors(self):
         names = {}

@@ -113,17 +113,21 @@ class GatedExperts(Part):
 
 @register_part("feed_forward", "grouped_experts")
 class GroupedExperts(Part):
-    """z = W_router h (float32), s = sigmoid(z), every expert for itself. A token's `top` experts are
+    """z = W_router h (float32), s = sigmoid(z), every expert for itself (`scoring` "sigmoid"), or softmax(z)
+    over all of them ("softmax"). A token's `top` experts are
     those with the largest s + correction (`correction`, a number per expert that enters the choice
     only), taken from `keep` of the `groups` equal groups of neighbouring experts: a group's score is
-    the sum of its two largest s + correction, the best groups are kept, and an expert of another
-    group cannot be chosen whatever its score. The weights are the chosen experts' s as they are.
+    the sum of its two largest s + correction ("softmax": its largest), the best groups are kept, and an
+    expert of another group cannot be chosen whatever its score. The weights are the chosen experts' s as
+    they are ("softmax": divided by their sum + 1e-20), times `scale`. The router has `identity` further
+    choices behind the experts, which give the layer's input back, have no tensors and are chosen, grouped
+    and weighted like experts.
     Each expert is a gated unit without biases, W_down (act(W_gate h) * (W_up h)), and the layer's
     result is the weighted sum of the chosen experts' results. A shared expert of the same form
     (inner size `shared_ff`, 0: none) serves every token and is added, multiplied by sigmoid(w_sg . h),
     one number per token.
 
-    Tensors: router (experts, hidden), correction (experts), e<i>.gate and e<i>.up (expert_ff, hidden),
+    Tensors: router (experts + identity, hidden), correction (experts + identity), e<i>.gate and e<i>.up (expert_ff, hidden),
     e<i>.down (hidden, expert_ff), shared.gate, shared.up (shared_ff, hidden), shared.down (hidden,
     shared_ff), shared.sg (1, hidden). The experts' matrices are kept stacked, gate and up as one with
     their rows interleaved; the shared expert's gate vector is one more row of the router's matrix, so
@@ -133,13 +137,17 @@ class GroupedExperts(Part):
     graph_safe = True
 
     def __init__(self, prefix, precision, device, hidden_size, experts, top, expert_ff, groups=1, keep=1, shared_ff=0,
-                 activation="silu"):
+                 activation="silu", scoring="sigmoid", identity=0, scale=1.0):
         super().__init__(prefix, precision, device)
-        if not 1 <= top <= experts:
-            raise ValueError("top (%d) must lie in 1..experts (%d)" % (top, experts))
-        if groups < 1 or experts % groups or not 1 <= keep <= groups or top > keep * (experts // groups):
+        choices = experts + identity
+        if identity < 0 or not 1 <= top <= choices:
+            raise ValueError("top (%d) must lie in 1..experts (%d)" % (top, choices))
+        if groups < 1 or choices % groups or not 1 <= keep <= groups or top > keep * (choices // groups):
             raise ValueError("groups (%d) must divide the experts (%d), keep (%d) lie in 1..groups, and the kept groups "
-                             "hold at least top (%d) experts" % (groups, experts, keep, top))
+                             "hold at least top (%d) experts" % (groups, choices, keep, top))
+        if scoring not in ("sigmoid", "softmax"):
+            raise ValueError("scoring is sigmoid or softmax, not %r" % (scoring,))
+        self.choices, self.identity, self.scoring, self.scale = choices, int(identity), scoring + "_groups", float(scale)
         if activation not in ops.GATE_KINDS:
             raise ValueError("activation is one of %s" % ", ".join(sorted(ops.GATE_KINDS)))
         self.hidden_size, self.experts, self.top, self.expert_ff = hidden_size, experts, top, expert_ff
@@ -148,7 +156,7 @@ class GroupedExperts(Part):
 
     def tensors(self):
         W = self.hidden_size
-        names = {self._name("router"): (self.experts, W), self._name("correction"): TensorShape((self.experts,), "bias")}
+        names = {self._name("router"): (self.choices, W), self._name("correction"): TensorShape((self.choices,), "bias")}
         for e in range(self.experts):
             names[self._name("e%d.gate" % e)] = (self.expert_ff, W)
             names[self._name("e%d.up" % e)] = (self.expert_ff, W)
@@ -186,8 +194,8 @@ class GroupedExperts(Part):
 
     def forward(self, x, batch=None):
         chosen, weights, rest = ops.moe_route(x, self.router.weight, self.top, tiled=self.router.tiled,
-                                              scoring="sigmoid_groups", correction=self.correction, groups=self.groups,
-                                              keep=self.keep, experts=self.experts)
+                                              scoring=self.scoring, correction=self.correction, groups=self.groups,
+                                              keep=self.keep, experts=self.choices, scale=self.scale)
         shared = shared_gate = None
         if self.shared_ff:
             if self.activation == "silu":
@@ -196,4 +204,4 @@ class GroupedExperts(Part):
                 hidden = ops.gated_act(self.shared_gate_up.forward(x), self.activation)
             shared, shared_gate = self.shared_down.forward(hidden), rest
         return ops.moe_glu_experts(x, chosen, weights, self.gate_up, self.down, activation=self.activation,
-                                   shared=shared, shared_gate=shared_gate)
+                                   shared=shared, shared_gate=shared_gate, identity=self.identity)

@@ -333,30 +333,34 @@ def latent_attention(q, cache, value_dim, block_table, cu_seqlens_q, kv_lens, ma
     return res.to(q.dtype)
 
 
-def moe_route(h, router, top, tiled=None, scoring="softmax", correction=None, groups=1, keep=1, experts=None):
+def moe_route(h, router, top, tiled=None, scoring="softmax", correction=None, groups=1, keep=1, experts=None, scale=1.0):
     z = h.float() @ router.float().T
     if experts is not None:
-        chosen, weights = moe_route(h, router[:experts], top, scoring=scoring, correction=correction, groups=groups, keep=keep)
+        chosen, weights = moe_route(h, router[:experts], top, scoring=scoring, correction=correction, groups=groups, keep=keep,
+                                    scale=scale)
         return chosen, weights, z[:, experts:]
-    if scoring == "sigmoid_groups":
+    if scoring in ("sigmoid_groups", "softmax_groups"):
         T, E = z.shape
-        score = torch.sigmoid(z)
+        score = torch.sigmoid(z) if scoring == "sigmoid_groups" else torch.softmax(z, dim=-1)
         choice = score + correction
         if keep < groups:
             size = E // groups
             grouped = choice.view(T, groups, size)
-            of_group = grouped.topk(min(2, size), dim=-1).values.sum(dim=-1)
+            of_group = grouped.topk(min(2, size) if scoring == "sigmoid_groups" else 1, dim=-1).values.sum(dim=-1)
             kept = torch.zeros((T, groups), dtype=torch.bool)
             kept[torch.arange(T)[:, None], of_group.topk(keep, dim=-1).indices] = True
             choice = grouped.masked_fill(~kept[:, :, None], float("-inf")).reshape(T, E)
         chosen = choice.topk(top, dim=-1).indices
-        return chosen.to(torch.int32), score.gather(1, chosen)
+        weights = score.gather(1, chosen)
+        if scoring == "softmax_groups":
+            weights = weights / (weights.sum(dim=-1, keepdim=True) + 1e-20)
+        return chosen.to(torch.int32), weights * scale
     if scoring == "sigmoid":
         best, chosen = torch.topk(z, top, dim=-1)
-        return chosen.to(torch.int32), torch.sigmoid(best)
+        return chosen.to(torch.int32), torch.sigmoid(best) * scale
     s = torch.softmax(z, dim=-1)
     best, chosen = torch.topk(s, top, dim=-1)
-    return chosen.to(torch.int32), best / (best.sum(dim=-1, keepdim=True) + 1e-20)
+    return chosen.to(torch.int32), best / (best.sum(dim=-1, keepdim=True) + 1e-20) * scale
 
 
 def moe_gated_experts(h, chosen, weights, gate_up, down, limit, slope):
@@ -370,13 +374,16 @@ def moe_gated_experts(h, chosen, weights, gate_up, down, limit, slope):
     return out.to(h.dtype)
 
 
-def moe_glu_experts(h, chosen, weights, gate_up, down, activation="silu", shared=None, shared_gate=None):
+def moe_glu_experts(h, chosen, weights, gate_up, down, activation="silu", shared=None, shared_gate=None, identity=0):
     T, top = chosen.shape
     out = torch.zeros((T, h.shape[1]), dtype=torch.float32, device=h.device)
     for k in range(top):
         e = chosen[:, k].long()
+        back = e >= down.shape[0]                                              # these give their input back
+        e = e.masked_fill(back, 0)
         both = torch.einsum("ti,tfi->tf", h.float(), gate_up[e].float())       # the gated unit sees unrounded sums
         y = torch.einsum("tf,twf->tw", gated_act(both, activation).to(h.dtype).float(), down[e].float()).to(h.dtype)
+        y = torch.where(back[:, None], h, y)
         out += weights[:, k, None] * y.float()
     if shared is not None:
         out += shared.float() * (torch.sigmoid(shared_gate.reshape(T, 1)) if shared_gate is not None else 1.0)
@@ -606,7 +613,7 @@ def channel_delta(conv, b_logits, a_logits, gate, dt_bias, a_log, norm_weight, e
 
 def softcap_attention(q, k_cache, v_cache, block_table, cu_seqlens_q, kv_lens, seq_index, positions, max_q_len,
                       max_kv_len, scale, softcap, window=0, gate=None, values_transposed=False, min_q_len=1,
-                      max_kv_len_of_many=None, sink=None, runs=None, sigmoid_bias=None):
+                      max_kv_len_of_many=None, sink=None, runs=None, sigmoid_bias=None, chunk=0, keep_first=0, span=False):
     T, H, dim = q.shape
     if values_transposed:
         v_cache = v_cache.transpose(2, 3)
@@ -626,7 +633,10 @@ def softcap_attention(q, k_cache, v_cache, block_table, cu_seqlens_q, kv_lens, s
         kpos = torch.arange(L, device=q.device)[None, :]
         hidden = kpos > qpos
         if window > 0:
-            hidden = hidden | (qpos - kpos >= window)
+            hidden = hidden | ((qpos - kpos >= window) & (kpos >= keep_first))
+        if chunk > 0:
+            hidden = hidden | ((torch.div(qpos, chunk, rounding_mode="floor") != torch.div(kpos, chunk, rounding_mode="floor"))
+                               & (kpos >= keep_first))
         if runs is not None and L // runs[3]:              # the runs' means stand before the tokens
             rk, rv, table, pool = runs
             many = L // pool
@@ -656,7 +666,8 @@ def softcap_attention(q, k_cache, v_cache, block_table, cu_seqlens_q, kv_lens, s
 
 
 def turn_prepare(rows, bias, heads, kv_heads, dim, vdim, inv_freq, factor, positions, seq_index, out_dtype, block_table,
-                 k_cache, v_cache, values_are_keys=False, runs=None, cu_seqlens_q=None, kv_lens=None, max_q_len=0):
+                 k_cache, v_cache, values_are_keys=False, runs=None, cu_seqlens_q=None, kv_lens=None, max_q_len=0,
+                 norm_eps=None, q_weight=None, k_weight=None, mix=None):
     T = rows.shape[0]
     nq, nk = heads * dim, kv_heads * dim
     n = nq + nk + (0 if values_are_keys else kv_heads * vdim)
@@ -665,6 +676,12 @@ def turn_prepare(rows, bias, heads, kv_heads, dim, vdim, inv_freq, factor, posit
         z = z + bias.float()
     q, k = z[:, :nq].reshape(T, heads, dim), z[:, nq:nq + nk].reshape(T, kv_heads, dim)
     v = k if values_are_keys else z[:, nq + nk:].reshape(T, kv_heads, vdim)
+    if norm_eps is not None:
+        q, k = (x * torch.rsqrt((x * x).mean(dim=-1, keepdim=True) + norm_eps) for x in (q, k))
+        if q_weight is not None:
+            q, k = q * q_weight, k * k_weight
+    if mix is not None:
+        v = (1.0 - mix[1]) * v + mix[1] * mix[0].reshape(T, kv_heads, vdim)
 
     def turn(x):
         if inv_freq is None:
