@@ -2,7 +2,7 @@
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch B] [--layers L]
                     [--shape 8b|14b|32b|0.6b] [--prompt P] [--context C]
-                    [--workload decode|continuous|served|prefix|products|kodisun|surasun|dufinex|fidevik|zedotar]
+                    [--workload decode|continuous|served|prefix|products|kodisun|surasun|dufinex|fidevik|zedotar|bemizen]
 
 Random bfloat16 weights, uniform-random prompts of 2,048 tokens, greedy decoding
 through the engine's own step loop (scheduler, step function, sampling). A
@@ -966,6 +966,127 @@ def zedotar(args, sync):
     return 0
 
 
+BEMIZEN_SHAPES = {
+    # (width, (heads, key heads, key size, value size, rotated, chunk), (heads, key heads, key size, value size, rotated,
+    #  window, first tokens), experts, that give their input back, top, groups, keep, expert_ff, layers)
+    "base": (2048, (16, 4, 128, 128, 64, 1024), (16, 4, 192, 128, 192, 512, 64), 64, 8, 6, 8, 4, 768, 4),
+    "wide": (4096, (32, 8, 128, 128, 32, 2048), (64, 8, 96, 64, 96, 1024, 32), 30, 2, 4, 4, 2, 2048, 2),
+}
+
+
+def bemizen(args, sync):
+    """Prefill and decode throughput of the Bemizen design at sizes that resemble a real model's layers
+    (random weights, a few layers, a vocabulary of 32,768), beside Fidevik, the closest of the other designs
+    (grouped-head attention, experts in groups by corrected scores), at the same width, layer count, heads
+    and experts, with its attention over all tokens, keys and values of 128, in every layer. Both go through
+    the engine's own loop: one prompt in one step, then greedy decoding at batch 8 and 64 behind prompts of
+    1,024 tokens. `frac` prices a prompt's multiply-adds (the products with a token's share of the experts,
+    the attention's visible pairs) against the bfloat16 matrix peak, and a decode step's bytes (the weights
+    once, of the experts those a batch can reach, the keys and values its requests see) against the HBM peak."""
+    import torch
+
+    from qwen3_from_scratch_amd.config.bemizen_config import BemizenConfig
+    from qwen3_from_scratch_amd.config.fidevik_config import FidevikConfig
+    from qwen3_from_scratch_amd.engine import SyncEngine, random_model
+
+    vocab, prompt_len, decode_prompt, context = 32768, args.prefill_tokens, 1024, 4096
+    results = {}
+
+    def seen(m, pos):
+        """How many keys the token at `pos` sees."""
+        mask = m.get("mask")
+        if mask is None:
+            return pos + 1
+        if "keep_first" in mask:
+            lo = max(0, pos - mask["size"] + 1)
+            return pos + 1 - lo + min(lo, mask["keep_first"])
+        return pos % mask["size"] + 1
+
+    for shape in ([args.bemizen_shape] if args.bemizen_shape != "all" else sorted(BEMIZEN_SHAPES)):
+        W, one, two, E, back, top, groups, keep, ff, n_layers = BEMIZEN_SHAPES[shape]
+        n_layers = args.layers or n_layers
+        mixers = [("attention", {"heads": one[0], "kv_heads": one[1], "dim": one[2], "vdim": one[3], "scale": one[2] ** -0.5,
+                                 "rot": {"dims": one[4], "base": 10000.0}, "mask": {"size": one[5]}, "v_mix": True}),
+                  ("attention_2", {"heads": two[0], "kv_heads": two[1], "dim": two[2], "vdim": two[3], "scale": two[2] ** -0.5,
+                                   "rot": {"dims": two[4], "base": 50000.0},
+                                   "mask": {"size": two[5], "keep_first": two[6]}, "v_mix": one[1] * one[3] == two[1] * two[3]})]
+        moe = {"kind": "moe", "expert": {"ff": ff},
+               "router": {"experts": E, "identity": back, "top": top, "scale": 2.0, "groups": {"count": groups, "keep": keep}}}
+        new = {"architecture": "Bemizen", "vocab": vocab, "width": W, "norm": {"eps": 1e-5},
+               "layers": [{"type": mixers[i % 2][0], "mixer": mixers[i % 2][1], "mlp": moe} for i in range(n_layers)]}
+        like = {"type": "attention", "mixer": {"heads": one[0], "kv_heads": one[1], "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+                                               "rot": {"dims": 64, "base": 10000.0}},
+                "mlp": {"kind": "moe", "router": {"experts": E + back, "top": top, "groups": {"count": groups, "keep": keep}},
+                        "expert": {"ff": ff}}}
+        other = {"architecture": "Fidevik", "vocab": vocab, "width": W, "norm": {"eps": 1e-5}, "logit_scale": 1.0,
+                 "layers": [like] * n_layers}
+        for name, config in (("bemizen", BemizenConfig.from_dict(new)), ("fidevik", FidevikConfig.from_dict(other))):
+            if args.bemizen_only and name != args.bemizen_only:
+                continue
+            model = random_model(config, dtype=args.dtype, device="cuda:0", seed=0, std=0.02)
+            gen = torch.Generator().manual_seed(1)
+            entry = {}
+            tensors = {key: t for key, t in model.tensors().items() if key.startswith("l") and len(t) == 2}
+            expert_numbers = sum(t[0] * t[1] for key, t in tensors.items() if ".mlp.e" in key)
+            matrices = sum(t[0] * t[1] for key, t in tensors.items() if ".mlp.e" not in key)
+            listed = [layer["mixer"] for layer in config.to_dict()["layers"]]
+            share = top / (E + back)
+            if "prefill" in args.phases:
+                room = prompt_len + 64
+                engine = SyncEngine(model=model, path="", dtype=args.dtype, device="cuda:0", max_len=room, block_size=BLOCK,
+                                    num_blocks=-(-room // BLOCK), max_num_seqs=1, max_num_tokens=prompt_len,
+                                    chunked_prefill_size=prompt_len, enable_prefix_cache=False)
+                timings = []
+                for _ in range(4):
+                    engine.add_request(torch.randint(0, vocab, (prompt_len,), generator=gen).tolist(),
+                                       engine.default_params(1, temperature=0.0, ignore_eos=True))
+                    sync()
+                    t0 = time.perf_counter()
+                    engine.step()
+                    sync()
+                    timings.append(time.perf_counter() - t0)
+                    while engine.scheduler.has_work():
+                        engine.step()
+                seconds = sorted(timings[1:])[1]
+                pairs = sum(m["heads"] * (m["dim"] + m["vdim"]) * sum(seen(m, p) for p in range(prompt_len)) for m in listed)
+                flops = 2.0 * prompt_len * (matrices + share * expert_numbers) + 2.0 * vocab * W + 2.0 * pairs
+                entry["prefill"] = {"tokens": prompt_len, "tokens_per_s": round(prompt_len / seconds, 1),
+                                    "ms": round(seconds * 1e3, 3), "frac": round(flops / seconds / PEAK_FLOPS[args.dtype], 4)}
+                del engine
+            for batch in ((8, 64) if "decode" in args.phases else ()):
+                engine = SyncEngine(model=model, path="", dtype=args.dtype, device="cuda:0", max_len=context,
+                                    block_size=BLOCK, num_blocks=batch * (context // BLOCK), max_num_seqs=batch,
+                                    max_num_tokens=max(2048, batch), chunked_prefill_size=2048, enable_prefix_cache=False)
+                params = engine.default_params(context - decode_prompt - 1, temperature=0.0, ignore_eos=True)
+                requests = [engine.add_request(torch.randint(0, vocab, (decode_prompt,), generator=gen).tolist(), params)
+                            for _ in range(batch)]
+                while any(r.is_prefill for r in requests) or len(engine.scheduler.waiting):
+                    engine.step()
+                for _ in range(args.warmup):
+                    engine.step()
+                sync()
+                t0 = time.perf_counter()
+                for _ in range(args.steps):
+                    engine.step()
+                sync()
+                step_s = (time.perf_counter() - t0) / args.steps
+                at = decode_prompt + args.warmup + args.steps // 2
+                cached = sum(m["kv_heads"] * (m["dim"] + m["vdim"]) * seen(m, at) for m in listed)
+                need = 2 * (matrices + min(1.0, batch * share) * expert_numbers + vocab * W) + batch * 2 * cached
+                entry["decode_b%d" % batch] = {"tokens_per_s": round(batch / step_s, 1), "ms_per_step": round(step_s * 1e3, 3),
+                                               "frac_hbm": round(need / step_s / PEAK_HBM, 4)}
+                del engine
+            results.setdefault(shape, {})[name] = entry
+            del model
+            torch.cuda.empty_cache()
+        results[shape]["sizes"] = {"width": W, "attention": mixers[0][1], "attention_2": mixers[1][1], "mlp": moe, "vocab": vocab,
+                                   "layers": n_layers}
+    print(json.dumps({"metric": "Bemizen beside Fidevik at equal size: prefill and decode tokens/s",
+                      "unit": "tokens/s", "n_gpus": 1, "higher_is_better": True, "dtype": "bf16", "data": "synthetic",
+                      "steps": args.steps, "warmup": args.warmup, "shapes": results}))
+    return 0
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -978,13 +1099,13 @@ def main():
     ap.add_argument("--prompt", type=int, default=2048, help="tokens every request holds when decoding starts")
     ap.add_argument("--context", type=int, default=8192, help="tokens of cache per request")
     ap.add_argument("--workload", default="decode", choices=["decode", "continuous", "served", "prefix", "products", "kodisun", "surasun", "dufinex", "fidevik",
-                                                                 "zedotar"],
+                                                                 "zedotar", "bemizen"],
                     help="continuous: 64 requests at once, prompts of 128 to 4,096 tokens, 64 to 512 generated "
                          "tokens each, prompts in portions of 512 (its own JSON line; --steps and --warmup unused); "
                          "prefix: 64 requests that share their first 2,048 tokens, with the prefix index on and off; "
                          "products: a layer's four products by the chosen kernel and by each tile shape of the "
                          "hand-written one; kodisun, surasun: that design beside the dense decoder at equal size; dufinex, "
-                         "zedotar: that design beside Surasun at equal size; fidevik: beside Kodisun")
+                         "zedotar: that design beside Surasun at equal size; fidevik: beside Kodisun; bemizen: beside Fidevik")
     ap.add_argument("--kodisun-shape", default="all", choices=["all"] + sorted(KODISUN_SHAPES))
     ap.add_argument("--kodisun-only", default="", choices=["", "kodisun", "qwen3_dense"], help="one of the two models")
     ap.add_argument("--surasun-shape", default="all", choices=["all"] + sorted(SURASUN_SHAPES))
@@ -995,8 +1116,10 @@ def main():
     ap.add_argument("--fidevik-only", default="", choices=["", "fidevik", "kodisun"], help="one of the two models")
     ap.add_argument("--zedotar-shape", default="all", choices=["all"] + sorted(ZEDOTAR_SHAPES))
     ap.add_argument("--zedotar-only", default="", choices=["", "zedotar", "surasun"], help="one of the two models")
+    ap.add_argument("--bemizen-shape", default="all", choices=["all"] + sorted(BEMIZEN_SHAPES))
+    ap.add_argument("--bemizen-only", default="", choices=["", "bemizen", "fidevik"], help="one of the two models")
     ap.add_argument("--phases", default="prefill,decode",
-                    help="of --workload kodisun, surasun, dufinex, fidevik or zedotar: prefill, decode or both")
+                    help="of --workload kodisun, surasun, dufinex, fidevik, zedotar or bemizen: prefill, decode or both")
     ap.add_argument("--single-copy", action="store_true",
                     help="hold the matrices once (no tile-ordered copy for steps of few rows): half the weights' memory, slower decoding")
     ap.add_argument("--no-points", action="store_true", help="skip the batch-1 and batch-64 points")
@@ -1036,6 +1159,10 @@ def main():
         torch.cuda.set_device(0)
         args.steps, args.warmup = min(args.steps, 32), min(args.warmup, 8)
         return zedotar(args, torch.cuda.synchronize)
+    if args.workload == "bemizen":
+        torch.cuda.set_device(0)
+        args.steps, args.warmup = min(args.steps, 32), min(args.warmup, 8)
+        return bemizen(args, torch.cuda.synchronize)
     shape_name, raw = SHAPES[args.shape]
     raw = dict(raw)
     prompt_len, context = args.prompt, args.context
