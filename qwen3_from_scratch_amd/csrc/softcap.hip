@@ -210,6 +210,101 @@ __global__ void __launch_bounds__(256) turn_prepare_kernel(
   }
 }
 
+// The same for sizes in steps of four and no runs, in 16-byte accesses: LPH lanes to a head, so that a wavefront
+// works on 64 / LPH heads (queries', then keys', then values') at once. A lane holds four numbers of the part
+// that turns and the four they turn with, or four of what passes, or four of a value.
+__device__ inline void put4(float* at, float4 v) { *reinterpret_cast<float4*>(at) = v; }
+__device__ inline void put4(bf16_t* at, float4 v) {
+  union {
+    uint2 u;
+    __bf16 e[4];
+  } pk;
+  pk.e[0] = (__bf16)v.x; pk.e[1] = (__bf16)v.y; pk.e[2] = (__bf16)v.z; pk.e[3] = (__bf16)v.w;
+  *reinterpret_cast<uint2*>(at) = pk.u;
+}
+__device__ inline void put1(float* at, float v) { *at = v; }
+__device__ inline void put1(bf16_t* at, float v) { *reinterpret_cast<__bf16*>(at) = (__bf16)v; }
+__device__ inline float4 get4(const float* at) { return *reinterpret_cast<const float4*>(at); }
+__device__ inline float4 plus4(float4 a, float4 b) { return make_float4(a.x + b.x, a.y + b.y, a.z + b.z, a.w + b.w); }
+__device__ inline float4 times4(float4 a, float4 b) { return make_float4(a.x * b.x, a.y * b.y, a.z * b.z, a.w * b.w); }
+__device__ inline float4 scaled4(float4 a, float f) { return make_float4(a.x * f, a.y * f, a.z * f, a.w * f); }
+__device__ inline float squares4(float4 a) { return a.x * a.x + a.y * a.y + a.z * a.z + a.w * a.w; }
+
+template <typename TA, int LPH>
+__global__ void __launch_bounds__(256) turn_prepare_vec_kernel(
+    const float* __restrict__ rows, long row_stride, const float* __restrict__ bias, const float* __restrict__ inv_freq,
+    int half, float factor, const int* __restrict__ positions, const int* __restrict__ seq_index,
+    const int* __restrict__ block_table, int table_width, TA* __restrict__ k_cache, TA* __restrict__ v_cache, int page,
+    TA* __restrict__ q_out, int H, int G, int dim, int vdim, int values_are_keys, HeadNorm norm, ValueMix mix) {
+  __shared__ __align__(16) float cs[Q3_TURN_HALF_MOST], sn[Q3_TURN_HALF_MOST];
+  constexpr int PER = Q3_WAVE / LPH;
+  const int t = blockIdx.x;
+  const int lane = threadIdx.x % Q3_WAVE, l = lane % LPH;
+  const int step = blockDim.x / Q3_WAVE * gridDim.y * PER;
+  const int first_item = (blockIdx.y * (blockDim.x / Q3_WAVE) + threadIdx.x / Q3_WAVE) * PER + lane / LPH;
+  const float* row = rows + (size_t)t * row_stride;
+  const int heads = H + G, items = H + 2 * G, turning = half / 4, lanes = turning + (dim - 2 * half) / 4;
+  const int pos = positions[t];
+  for (int i = threadIdx.x; i < half; i += blockDim.x) {
+    float s, c;
+    sincosf((float)pos * inv_freq[i], &s, &c);
+    cs[i] = c * factor;
+    sn[i] = s * factor;
+  }
+  const int pg = pos / page < table_width ? block_table[(size_t)seq_index[t] * table_width + pos / page] : -1;
+  const int off = pos % page;
+  const float share = mix.first ? *mix.share : 0.f;
+  const bool turns = l < turning, holds = l < lanes;
+  const int at = turns ? 4 * l : 2 * half + 4 * (l - turning);    // where this lane's first four numbers stand in a head
+  const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f);
+  __syncthreads();
+  for (int item = first_item; item < items; item += step) {
+    if (item < heads) {
+      const float* x = row + (size_t)item * dim;
+      float4 a = holds ? get4(x + at) : zero, b = turns ? get4(x + half + at) : zero;
+      if (bias) {
+        const float* add = bias + (size_t)item * dim;
+        if (holds) a = plus4(a, get4(add + at));
+        if (turns) b = plus4(b, get4(add + half + at));
+      }
+      if (norm.on) {
+        float acc = squares4(a) + squares4(b);
+#pragma unroll
+        for (int o = LPH / 2; o > 0; o >>= 1) acc += __shfl_xor(acc, o, Q3_WAVE);
+        const float scale = rsqrtf(acc / (float)dim + norm.eps);
+        a = scaled4(a, scale);
+        b = scaled4(b, scale);
+        const float* weight = item < H ? norm.q_weight : norm.k_weight;
+        if (weight) {
+          if (holds) a = times4(a, get4(weight + at));
+          if (turns) b = times4(b, get4(weight + half + at));
+        }
+      }
+      TA* dst = item < H ? q_out + ((size_t)t * H + item) * dim
+                         : k_cache + (((size_t)max(pg, 0) * G + item - H) * page + off) * dim;
+      if (item >= H && pg < 0) continue;
+      if (turns) {
+        const float4 c = get4(cs + at), s = get4(sn + at);
+        put4(dst + half + at, make_float4(b.x * c.x + a.x * s.x, b.y * c.y + a.y * s.y, b.z * c.z + a.z * s.z, b.w * c.w + a.w * s.w));
+        a = make_float4(a.x * c.x - b.x * s.x, a.y * c.y - b.y * s.y, a.z * c.z - b.z * s.z, a.w * c.w - b.w * s.w);
+      }
+      if (holds) put4(dst + at, a);
+    } else if (pg >= 0 && 4 * l < vdim) {
+      const int g = item - heads;
+      const size_t from = values_are_keys ? (size_t)(H + g) * dim : (size_t)heads * dim + (size_t)g * vdim;
+      float4 v = get4(row + from + 4 * l);
+      if (bias) v = plus4(v, get4(bias + from + 4 * l));
+      if (mix.first)
+        v = plus4(scaled4(v, 1.f - share), scaled4(get4(mix.first + (size_t)t * mix.stride + (size_t)g * vdim + 4 * l), share));
+      TA* dst = v_cache + (((size_t)pg * G + g) * vdim + 4 * l) * page + off;
+      put1(dst, v.x);
+      put1(dst + page, v.y);
+      put1(dst + 2 * (size_t)page, v.z);
+      put1(dst + 3 * (size_t)page, v.w);
+    }
+  }
+}
+
 extern "C" int q3_turn_prepare(const float* rows, long row_stride, const float* bias, const float* inv_freq, int half,
                                float factor, const int* positions, const int* seq_index, const int* block_table,
                                int table_width, void* k_cache, void* v_cache, int page, void* q_out, int T, int H, int G,
@@ -228,6 +323,30 @@ extern "C" int q3_turn_prepare(const float* rows, long row_stride, const float* 
   const HeadNorm norm{norm_on, norm_eps, q_weight, k_weight};
   const ValueMix mix{mix_first, mix_stride, mix_share};
   // few tokens: a wavefront per head; many: the tokens fill the chip, and share their cosines among more heads
+  const auto aligned = [](const void* p) { return ((uintptr_t)p & 15) == 0; };
+  int lanes = half / 4 + (dim - 2 * half) / 4;
+  if (vdim / 4 > lanes) lanes = vdim / 4;
+  if (!run_k && half % 4 == 0 && dim % 4 == 0 && vdim % 4 == 0 && lanes <= 64 && row_stride % 4 == 0 && mix_stride % 4 == 0 &&
+      aligned(rows) && aligned(bias) && aligned(q_weight) && aligned(k_weight) && aligned(mix_first) && aligned(k_cache) &&
+      aligned(q_out)) {
+    const int lph = lanes <= 16 ? 16 : lanes <= 32 ? 32 : 64;
+    const int waves = ((H + 2 * G) * lph + Q3_WAVE - 1) / Q3_WAVE, blocks = (waves + 3) / 4;
+    const int shares = T >= 1024 ? 1 : (T >= 256 ? (blocks < 2 ? blocks : 2) : (blocks < 64 ? blocks : 64));
+#define Q3_TURN_VEC(LPH)                                                                                                     \
+  Q3_DISPATCH_DTYPE(act_dtype, TA,                                                                                         \
+                    hipLaunchKernelGGL((turn_prepare_vec_kernel<TA, LPH>), dim3(T, shares), dim3(256), 0, stream, rows,      \
+                                       row_stride, bias, inv_freq, half, factor, positions, seq_index, block_table,         \
+                                       table_width, (TA*)k_cache, (TA*)v_cache, page, (TA*)q_out, H, G, dim, vdim,          \
+                                       values_are_keys, norm, mix))
+    if (lph == 16)
+      Q3_TURN_VEC(16);
+    else if (lph == 32)
+      Q3_TURN_VEC(32);
+    else
+      Q3_TURN_VEC(64);
+#undef Q3_TURN_VEC
+    return q3_launch_status();
+  }
   const int most = (H + G + 3) / 4;
   const int shares = T >= 1024 ? 1 : (T >= 256 ? (most < 2 ? most : 2) : (most < 64 ? most : 64));
   Q3_DISPATCH_DTYPE(act_dtype, TA,

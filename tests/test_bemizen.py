@@ -291,10 +291,11 @@ def test_a_turn_leaves_the_root_mean_square():
     assert turned[[1, 3, 4, 5]].tolist() == [0.0, 0.0, 2.0, 6.0]
 
 
-def _prepare_inputs(T, H, G, d, dv, half, seed=1):
+def _prepare_inputs(T, H, G, d, dv, half, seed=1, more=5, ahead=2):
+    """Rows with `more` columns behind them, values to mix in with `ahead` columns before them."""
     g = torch.Generator().manual_seed(seed)
-    rows = torch.randn((T, H * d + G * (d + dv) + 5), generator=g) * 2.0
-    first = torch.randn((T, G * dv + 3), generator=g)[:, 2:2 + G * dv]
+    rows = torch.randn((T, H * d + G * (d + dv) + more), generator=g) * 2.0
+    first = torch.randn((T, G * dv + 2 * ahead), generator=g)[:, ahead:ahead + G * dv]
     qw, kw = torch.rand(d, generator=g) + 0.5, torch.rand(d, generator=g) + 0.5
     inv_freq = (torch.rand(half, generator=g) + 0.01) if half else None
     return rows, first, torch.tensor([0.37]), qw, kw, inv_freq
@@ -514,17 +515,22 @@ def _packed(q_lens, kv):
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 @pytest.mark.parametrize("H,G,d,dv,half,page", [(4, 2, 16, 24, 4, 8), (16, 4, 64, 64, 32, 16), (3, 1, 7, 5, 0, 16), (2, 2, 1, 3, 0, 4),
                                                 (6, 3, 128, 128, 16, 16), (2, 2, 300, 10, 129, 16), (8, 2, 96, 64, 48, 16),
-                                                (4, 1, 192, 128, 96, 32), (5, 1, 130, 512, 65, 16), (3, 3, 512, 40, 256, 16)])
+                                                (4, 1, 192, 128, 96, 32), (5, 1, 130, 512, 65, 16), (3, 3, 512, 40, 256, 16),
+                                                (12, 4, 256, 256, 128, 16), (9, 3, 128, 20, 4, 16)])
 def test_prepare_kernel(dtype, H, G, d, dv, half, page):
     """Norms per head with a weight, without one and none, and values mixed or as they are: portions beside
     single tokens, single tokens alone, a long prompt, at positions beyond 100,000 too; rows that lie apart."""
     import torch_ops
     from qwen3_from_scratch_amd import ops
 
-    for q_lens, kv, ahead in (([37, 1, 2, 5], [90, 41, 2, 66], 0), ([1, 1, 1, 1, 1], [9, 16, 67, 1, 33], 0), ([1100], [1101], 0),
-                              ([3], [9], 100000)):
+    cases = (([37, 1, 2, 5], [90, 41, 2, 66], 0), ([1, 1, 1, 1, 1], [9, 16, 67, 1, 33], 0), ([1100], [1101], 0), ([3], [9], 100000))
+    # rows and values whose addresses allow 16-byte accesses (then sizes in steps of four take them), and others
+    for (q_lens, kv, ahead), (more, before) in ((c, m) for c in cases for m in ((5, 2), (8, 4))):
         T = sum(q_lens)
-        rows, first, share, qw, kw, inv_freq = (t.cuda() if t is not None else None for t in _prepare_inputs(T, H, G, d, dv, half))
+        rows, first, share, qw, kw, inv_freq = (t if t is None else t.cuda()
+                                                for t in _prepare_inputs(T, H, G, d, dv, half, more=more, ahead=before))
+        if before == 4:                                  # a view again, as the product's rows give it
+            first = torch.nn.functional.pad(first, (before, before))[:, before:-before]
         _, _, pos, seq = _packed(q_lens, kv)
         if ahead:
             table = torch.full((1, (ahead + 9) // page + 1), -1, dtype=torch.int32)
@@ -543,7 +549,7 @@ def test_prepare_kernel(dtype, H, G, d, dv, half, page):
                 out.append((q, kc, vc))
             tol = (4e-5 if dtype == torch.float32 else 6e-2) * (4 if d == 1 else 1) + (2e-2 if ahead else 0.0)
             for a, b in zip(*out):
-                assert float((a.float() - b.float()).abs().max()) <= tol, (norm, q_lens)
+                assert float((a.float() - b.float()).abs().max()) <= tol, (norm, q_lens, more)
 
 
 SPANS = [dict(chunk=9), dict(window=11, keep_first=5), dict(chunk=70), dict(window=50, keep_first=21), dict(window=1, keep_first=1),
