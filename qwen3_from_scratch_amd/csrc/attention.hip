@@ -691,19 +691,20 @@ __device__ __forceinline__ void attend_span(const Pack16 (&qreg)[1][D / 32], con
   auto addr_of = [&](const TilePages& p, int s) {
     return tile_addr_of(p, k_cache, v_cache, num_pages, Hkv, g_kv, page, D, DV, key_of(s));
   };
-  Pack16 a_cur[2][D / 32], v_cur[DV / 16], a_nxt[2][D / 32], v_nxt[DV / 16];
-  {
-    const TileAddr t = addr_of(tile_pages(bt_row, bt_stride, page, key_of(first)), first);
-    load_keys<D>(a_cur, t);
-    load_values<DV>(v_cur, t, page);
-  }
+  // (keys of 192 numbers leave no registers for a second tile's values: those are asked for a turn later)
+  constexpr bool VALUES_AHEAD = D <= 128;
+  Pack16 a_cur[2][D / 32], v_cur[DV / 16], a_nxt[2][D / 32], v_nxt[VALUES_AHEAD ? DV / 16 : 1];
+  TileAddr t_cur = addr_of(tile_pages(bt_row, bt_stride, page, key_of(first)), first);
+  load_keys<D>(a_cur, t_cur);
+  if constexpr (VALUES_AHEAD) load_values<DV>(v_cur, t_cur, page);
   TilePages p_nxt = tile_pages(bt_row, bt_stride, page, key_of(first + step));
   for (int s = first; s < last; s += step) {
     const bool more = s + step < last;
+    if constexpr (!VALUES_AHEAD) load_values<DV>(v_cur, t_cur, page);
     if (more) {
-      const TileAddr t = addr_of(p_nxt, s + step);
-      load_keys<D>(a_nxt, t);
-      load_values<DV>(v_nxt, t, page);
+      t_cur = addr_of(p_nxt, s + step);
+      load_keys<D>(a_nxt, t_cur);
+      if constexpr (VALUES_AHEAD) load_values<DV>(v_nxt, t_cur, page);
       p_nxt = tile_pages(bt_row, bt_stride, page, key_of(s + 2 * step));
     }
     attend_tile<D, 1, DV>(qreg, a_cur, v_cur, key_of(s), kv_len, row_pos, span, scale_log2, acc, m_run, l_run);
@@ -712,8 +713,10 @@ __device__ __forceinline__ void attend_span(const Pack16 (&qreg)[1][D / 32], con
       for (int kb = 0; kb < 2; ++kb)
 #pragma unroll
         for (int i = 0; i < D / 32; ++i) a_cur[kb][i] = a_nxt[kb][i];
+      if constexpr (VALUES_AHEAD) {
 #pragma unroll
-      for (int nb = 0; nb < DV / 16; ++nb) v_cur[nb] = v_nxt[nb];
+        for (int nb = 0; nb < DV / 16; ++nb) v_cur[nb] = v_nxt[nb];
+      }
     }
   }
 }
