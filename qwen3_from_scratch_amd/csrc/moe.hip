@@ -268,7 +268,7 @@ union MoePack {
 #define MMA_TM 64
 #define MMA_MT 4
 
-template <int NS>
+template <int NS, int U>
 __global__ __launch_bounds__(256) void moe_linear_mma_kernel(
     const bf16_t* __restrict__ x, const int* __restrict__ pair_of_slot, int gather, int pairs_per_row,
     const bf16_t* __restrict__ w, bf16_t* __restrict__ out, const int* __restrict__ tile_expert,
@@ -305,10 +305,7 @@ __global__ __launch_bounds__(256) void moe_linear_mma_kernel(
 #pragma unroll
     for (int ns = 0; ns < NS; ++ns) acc[mt][ns] = moe_f32x4_t{0.f, 0.f, 0.f, 0.f};
   const int row_blocks = (rows + 15) >> 4;          // the same for every lane
-  // U steps of 32 k are asked for together before their matrix instructions run. One slab a
-  // wavefront is the case of few rows, where the weights stream from memory and what counts is
-  // how many loads are on their way.
-  constexpr int U = NS == 1 ? 4 : 2;
+  // U steps of 32 k are asked for together before their matrix instructions run.
   for (int k0 = 0; k0 < K; k0 += 32 * U) {
     MoePack a[U][NS], b[U][MMA_MT];
 #pragma unroll
@@ -703,11 +700,12 @@ extern "C" int q3_moe_align(const int* chosen, int P, int E, int tile_rows, int*
   return q3_launch_status();
 }
 
-// The matrix-core product: bfloat16, K a multiple of 32, tiles of 64 slots.
+// The matrix-core product: bfloat16, K a multiple of 32, tiles of 64 slots (or 128, or 256). `n_pairs`,
+// `n_experts`: the step's (token, choice) pairs and the experts they are spread over.
 extern "C" int q3_moe_linear_mma(const void* x, const int* pair_of_slot, int gather, int pairs_per_row, const void* w,
                                  void* out, const int* tile_expert, const int* tile_first, const int* offsets,
-                                 const int* n_tiles, int max_tiles, int N, int K, int act, int tile_rows,
-                                 hipStream_t stream) {
+                                 const int* n_tiles, int max_tiles, int N, int K, int act, int tile_rows, int n_pairs,
+                                 int n_experts, hipStream_t stream) {
   if (max_tiles <= 0 || N <= 0 || K <= 0 || K % 32 || pairs_per_row <= 0 || act < -1 || act > MOE_ACT_MOST ||
       (act >= MOE_ACT_GATED && N % 2) ||
       (tile_rows != MMA_TM && tile_rows != BIG_TM && tile_rows != GT_BM))
@@ -735,17 +733,27 @@ extern "C" int q3_moe_linear_mma(const void* x, const int* pair_of_slot, int gat
                        pairs_per_row, (const bf16_t*)w, (bf16_t*)out, tile_expert, tile_first, offsets, n_tiles, N, K, act);
     return q3_launch_status();
   }
-  // few blocks (steps of few tokens): one slab of 16 columns per wavefront, so that more blocks stream the weights
-  const bool narrow = (long)max_tiles * ((N + 255) / 256) < 512;
-  const int per_block = narrow ? 64 : 256;
+  // How many slabs of 16 columns a wavefront takes (NS) and how many steps of k it asks for at once (U), measured
+  // over weights that come from memory (64 experts of 2,048 x 768, 6 a token; 30 and 32 of 4,096 x 2,048, 4 a token):
+  // an expert with a row or so, one slab and short batches (8 tokens: 58 us a first product of 201 MB where one slab
+  // and four steps take 69 and four slabs 85; 123 us for 604 MB, where those take 243 and 174); with more rows four
+  // slabs if their blocks fill the chip's CUs twice (64 tokens: 207 us for 1,007 MB, with two slabs 258, with one 273),
+  // two otherwise (94 us for 403 MB, 107 and 114).
+  const bool thin = 4L * n_pairs <= 5L * n_experts;
+  const bool wide = !thin && (long)max_tiles * ((N + 255) / 256) >= 480;
+  const int per_block = thin ? 64 : wide ? 256 : 128;
   const dim3 grid(max_tiles, (N + per_block - 1) / per_block);
   if (grid.y > 65535) return Q3_ERR_UNSUPPORTED;
-  if (narrow)
-    hipLaunchKernelGGL(moe_linear_mma_kernel<1>, grid, dim3(256), 0, stream, (const bf16_t*)x, pair_of_slot, gather,
-                       pairs_per_row, (const bf16_t*)w, (bf16_t*)out, tile_expert, tile_first, offsets, n_tiles, N, K, act);
+#define Q3_MOE_MMA(NS, U)                                                                                                    \
+  hipLaunchKernelGGL((moe_linear_mma_kernel<NS, U>), grid, dim3(256), 0, stream, (const bf16_t*)x, pair_of_slot, gather,    \
+                     pairs_per_row, (const bf16_t*)w, (bf16_t*)out, tile_expert, tile_first, offsets, n_tiles, N, K, act)
+  if (thin)
+    Q3_MOE_MMA(1, 2);
+  else if (wide)
+    Q3_MOE_MMA(4, 4);
   else
-    hipLaunchKernelGGL(moe_linear_mma_kernel<4>, grid, dim3(256), 0, stream, (const bf16_t*)x, pair_of_slot, gather,
-                       pairs_per_row, (const bf16_t*)w, (bf16_t*)out, tile_expert, tile_first, offsets, n_tiles, N, K, act);
+    Q3_MOE_MMA(2, 4);
+#undef Q3_MOE_MMA
   return q3_launch_status();
 }
 

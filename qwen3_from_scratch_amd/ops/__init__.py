@@ -687,9 +687,9 @@ def moe_experts(h, chosen, weights, up, down, shared=None, activation="erf"):
     y = torch.empty((P, width), dtype=h.dtype, device=h.device)
     if cores:
         _check(lib.q3_moe_linear_mma(_ptr(h), _ptr(pair_of_slot), 1, top, _ptr(up), _ptr(hidden), *tiles, ff, width,
-                                     GELU_KINDS[activation], tile_rows, stream), "moe_linear")
+                                     GELU_KINDS[activation], tile_rows, P, E, stream), "moe_linear")
         _check(lib.q3_moe_linear_mma(_ptr(hidden), _ptr(pair_of_slot), 0, 1, _ptr(down), _ptr(y), *tiles, width, ff,
-                                     -1, tile_rows, stream), "moe_linear")
+                                     -1, tile_rows, P, E, stream), "moe_linear")
     else:
         _check(lib.q3_moe_linear(_ptr(h), _ptr(pair_of_slot), 1, top, _ptr(up), _ptr(hidden), *tiles, ff, width,
                                  GELU_KINDS[activation], _DT[h.dtype], stream), "moe_linear")
@@ -743,14 +743,14 @@ def moe_gated_experts(h, chosen, weights, gate_up, down, limit, slope):
     stream = _stream()
     if cores:
         _check(lib.q3_moe_linear_mma(_ptr(h), _ptr(pair_of_slot), 1, top, _ptr(gate_up), _ptr(both), *tiles, 2 * ff, width,
-                                     -1, tile_rows, stream), "moe_linear")
+                                     -1, tile_rows, P, E, stream), "moe_linear")
     else:
         _check(lib.q3_moe_linear(_ptr(h), _ptr(pair_of_slot), 1, top, _ptr(gate_up), _ptr(both), *tiles, 2 * ff, width, -1,
                                  _DT[h.dtype], stream), "moe_linear")
     hidden = glu_clamped(both, limit, slope, scale=weights.view(-1), scale_index=pair_of_slot)
     if cores:
         _check(lib.q3_moe_linear_mma(_ptr(hidden), _ptr(pair_of_slot), 0, 1, _ptr(down), _ptr(y), *tiles, width, ff,
-                                     -1, tile_rows, stream), "moe_linear")
+                                     -1, tile_rows, P, E, stream), "moe_linear")
     else:
         _check(lib.q3_moe_linear(_ptr(hidden), _ptr(pair_of_slot), 0, 1, _ptr(down), _ptr(y), *tiles, width, ff, -1,
                                  _DT[h.dtype], stream), "moe_linear")
@@ -802,13 +802,13 @@ def moe_glu_experts(h, chosen, weights, gate_up, down, activation="silu", shared
     gated = _MOE_ACT_GATED + GATE_KINDS[activation]      # the gated unit is the first product's epilogue, on unrounded sums
     if cores:
         _check(lib.q3_moe_linear_mma(_ptr(h), _ptr(pair_of_slot), 1, top, _ptr(gate_up), _ptr(hidden), *tiles, 2 * ff, width,
-                                     gated, tile_rows, stream), "moe_linear")
+                                     gated, tile_rows, P, E, stream), "moe_linear")
     else:
         _check(lib.q3_moe_linear(_ptr(h), _ptr(pair_of_slot), 1, top, _ptr(gate_up), _ptr(hidden), *tiles, 2 * ff, width,
                                  gated, _DT[h.dtype], stream), "moe_linear")
     if cores:
         _check(lib.q3_moe_linear_mma(_ptr(hidden), _ptr(pair_of_slot), 0, 1, _ptr(down), _ptr(y), *tiles, width, ff,
-                                     -1, tile_rows, stream), "moe_linear")
+                                     -1, tile_rows, P, E, stream), "moe_linear")
     else:
         _check(lib.q3_moe_linear(_ptr(hidden), _ptr(pair_of_slot), 0, 1, _ptr(down), _ptr(y), *tiles, width, ff, -1,
                                  _DT[h.dtype], stream), "moe_linear")

@@ -705,7 +705,8 @@ def test_grouped_softmax_router_kernel(dtype, T, width, E, top, groups, keep, mo
 @pytest.mark.gpu
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 @pytest.mark.parametrize("T,width,ff,E,back,top", [(1, 64, 32, 7, 2, 3), (50, 48, 24, 5, 1, 2), (333, 128, 96, 6, 6, 3),
-                                                   (17, 40, 20, 1, 3, 4), (700, 96, 160, 3, 2, 2), (900, 64, 64, 2, 1, 2)])
+                                                   (17, 40, 20, 1, 3, 4), (700, 96, 160, 3, 2, 2), (900, 64, 64, 2, 1, 2),
+                                                   (300, 64, 640, 100, 4, 3), (20, 64, 640, 100, 4, 3)])
 def test_experts_with_identities(dtype, T, width, ff, E, back, top):
     import torch_ops
     from qwen3_from_scratch_amd import ops
